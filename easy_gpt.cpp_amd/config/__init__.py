@@ -4,6 +4,7 @@ from .kezolix import KezolixConfig
 from .nebanex import NebanexConfig
 from .pekasun import PekasunConfig
 from .qwen2 import Qwen2Config
+from .tipezen import TipezenConfig
 from .registry import (
     Architecture,
     UnknownArchitectureError,
@@ -23,6 +24,7 @@ __all__ = [
     "NebanexConfig",
     "PekasunConfig",
     "Qwen2Config",
+    "TipezenConfig",
     "UnknownArchitectureError",
     "load_model_config",
     "read_json",

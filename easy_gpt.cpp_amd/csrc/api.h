@@ -23,8 +23,9 @@ int egpt_add_rmsnorm(void* h, int fixed, const void* delta, int delta_splits, in
                      const void* weight, float eps, void* out, int n_rows, int hidden, int dtype, void* stream);
 // row_ss (may be null) float32 [ss_splits, n_tokens]: gate_up are float32 partial sums that still lack each row's factor
 // 1/sqrt(sum_s row_ss[s][t] / hidden + eps)
+// act (here and in the products below that end or begin with it): the gate's activation, 0 silu, 1 the tanh form of gelu
 int egpt_swiglu(const void* gate_up, int n_splits, const float* row_ss, int ss_splits, int hidden, float eps, void* out,
-                int n_tokens, int inter, int dtype, void* stream);
+                int n_tokens, int inter, int act, int dtype, void* stream);
 // qkv_out [n_tokens, (nq + 2 nkv) hd] of the activation type; may be qkv_in itself when n_splits == 0.
 // row_ss != null: the product still lacks each row's factor 1 / sqrt(sum_s row_ss[s][row] / hidden + eps).
 // cos_sin != null: the angles' cosines and sines from egpt_rope_table ([n_tokens][rotary_dim / 2][2]) instead of
@@ -115,12 +116,12 @@ int egpt_gemm_skinny_norm(const void* h_in, int h_fixed, float* h_out, const flo
                           int n_splits, int waves, void* stream);
 int egpt_gemm_skinny_swiglu(const float* gate_up, int gu_splits, const float* ss_in, int ss_splits, int hidden,
                             float eps, const void* w, float* out, void* acc_fixed, int m, int n, int k, int n_splits,
-                            int waves, void* stream);
+                            int waves, int act, void* stream);
 int egpt_gemm_skinny_attn(const float* part_o, const float* part_ml, int a_splits, int nq, int hd, const void* w,
                           float* out, void* acc_fixed, int m, int n, int n_splits, int waves, void* stream);
 // Gate/up product with SwiGLU for up to 64 rows (see gemm_gate_up.hip): out bfloat16 [m][inter] from x bfloat16 [m][k]
 // and w bfloat16 [2 * inter][k] (gate rows, then up rows); k % 8 == 0.
-int egpt_gemm_gate_up_swiglu(const void* x, const void* w, void* out, int m, int inter, int k, int groups, void* stream);
+int egpt_gemm_gate_up_swiglu(const void* x, const void* w, void* out, int m, int inter, int k, int groups, int act, void* stream);
 // ---- mixers that norm or rotate single heads (head_prep.hip), and their attention (attention_window.hip)
 // out [n_tokens][hidden] = table[id] / sqrt(mean(table[id]^2) + eps) * weight: an embedding with its norm, as the
 // residual stream (float32, or fixed point with fixed != 0).  In the three functions below row_ss (may be null)
@@ -137,10 +138,14 @@ int egpt_embed_rmsnorm(const int32_t* ids, const void* table, const void* weight
 // are no value columns and value head g is key head g as projected (dv == dk), 16 the rotation pairs place 2i with
 // 2i + 1 instead of i with i + rot_dims / 2.  rot_dims > 0: the first rot_dims places of query and key heads turn by
 // the angles in cos_sin float32 [n_tokens][rot_dims / 2][2] (cos, sin; both times mag).
+// values_out (may be null): the value heads as float32 [n_tokens][nkv * dv]; mix_with (may be null) float32 of that shape: what is
+// stored is (1 - mix) * value + mix * mix_with (values_out is not mixed); gates_out float32 [n_tokens][n_gates]: sigmoids of the
+// n_gates columns from gate_off on (n_gates 0: none).
 int egpt_head_norm_store(const void* proj, int n_splits, const float* row_ss, int ss_splits, int hidden, float norm_eps,
                          int row_width, void* q_out, const void* q_weight, const void* k_weight, float eps, int flags,
                          const float* cos_sin, int rot_dims, float mag, const int32_t* slots, void* k_cache, void* v_cache,
-                         int n_tokens, int nq, int nkv, int dk, int dv, int page_size, int dtype, void* stream);
+                         int n_tokens, int nq, int nkv, int dk, int dv, int page_size, float* values_out, const float* mix_with,
+                         float mix, int n_gates, int gate_off, float* gates_out, int dtype, void* stream);
 // proj rows of row_width values: [nq heads of (dim | rot) | rank | rot | ...].  q_plain [n_tokens][nq][dim] takes the
 // heads' unrotated parts; q_full [n_tokens][nq][rank + rot] their rotated parts behind the first rank places.  The
 // latent (normed with c_weight [rank]) and the rotated shared key are stored as key [pages][1][page_size][rank + rot],
@@ -163,13 +168,15 @@ int egpt_sigmoid_gate(const void* x, int heads, const void* gate, int gate_split
 // head and distance (dist_bias float32 [nq][dist_far + 1], null: none): key j of a query at position p gets
 // dist_bias[head][min(p - j, dist_far)] added to its scaled score.  block > 0: key j is seen only if it lies in the
 // query's block of positions, floor(j / block) == floor(p / block).  slopes float32 [nq] (null: none): the scaled score
-// of key j loses slopes[head] * (p - j) (the matrix-core kernel takes a bias table or slopes, not both).  q [n_tokens][nq][dk],
+// of key j loses slopes[head] * (p - j) (the matrix-core kernel takes a bias table or slopes, not both).  softcap c > 0: the
+// scaled score s becomes c tanh(s / c) (neither bias nor slopes then; the sink is not capped).  head_gate float32 [n_tokens][nq]
+// (null: none): a factor on each head's output.  q [n_tokens][nq][dk],
 // out [n_tokens][nq][dv]; the other operands as egpt_paged_attention.
 int egpt_window_attention(const void* q, void* out, const void* k_cache, const void* v_cache, const int32_t* block_table,
                           int table_width, const int32_t* q_start, const int32_t* q_len, const int32_t* kv_len,
                           int n_seqs, int n_tokens, int nq, int nkv, int dk, int dv, int page_size, float scale,
                           int window, int keep_first, const float* sink, const float* dist_bias, int dist_far, int block,
-                          const float* slopes, int dtype, void* stream);
+                          const float* slopes, float softcap, const float* head_gate, int dtype, void* stream);
 // The same on the matrix cores: dk a multiple of 4 (float32) or 8 (bfloat16) up to 256, dv a multiple of 16 up to 256,
 // page_size a multiple of 16.  row_tiles: tiles of 16 rows to a workgroup of four wavefronts: 8 (32 rows to a wavefront)
 // or 4 (16).  With
@@ -179,8 +186,8 @@ int egpt_window_attention_tiled(const void* q, void* out, float* part_o, float* 
                                 const void* v_cache, const int32_t* block_table, int table_width, const int32_t* q_start,
                                 const int32_t* q_len, const int32_t* kv_len, int n_seqs, int n_tokens, int nq, int nkv,
                                 int dk, int dv, int page_size, float scale, int window, int keep_first, const float* sink,
-                                const float* dist_bias, int dist_far, int block, const float* slopes, int n_splits,
-                                int row_tiles, int dtype, void* stream);
+                                const float* dist_bias, int dist_far, int block, const float* slopes, float softcap,
+                                const float* head_gate, int n_splits, int row_tiles, int dtype, void* stream);
 // ---- residual stream and logits (stream_ops.hip)
 // out[t] = table[ids[t]] * factor as the float32 residual stream.
 int egpt_embed_scaled(const int32_t* ids, const void* table, float factor, float* out, int n_tokens, int hidden, int vocab,
@@ -205,7 +212,15 @@ int egpt_embed_positions(const int32_t* ids, const int32_t* positions, const voi
 int egpt_post_norm_add(const float* h, const void* y, int y_splits, const void* y2, int y2_splits, float fy, float fy2,
                        const void* post_w, float eps, float mult, float* hist, int n_hist, const float* mix, float* h_out,
                        const void* next_w, void* out, int n_rows, int hidden, int dtype, void* stream);
-// x = cap * tanh(x / cap) in place.
+// n_streams residual streams x float32 [n_streams][rows][hidden], stream_stride values apart (0: all are the same one).  With a
+// pending output y (a product of y_rows rows; null: none) they become x'_t = sum_s mix[s][t] x_s + out_w[t] * scale * y (scale
+// float32 [hidden] or null), written to x_out (null: not kept; x itself with up to 8 streams and equal strides); then u = sum_s
+// in_w[s] x'_s (in_w null: the plain sum) and out = rmsnorm(u) * norm_w in the activation type.  rows int32 [n_rows] (null:
+// all): only those are read and nothing is kept.
+int egpt_connect_streams(const float* x, long long stream_stride, int n_streams, const void* y, int y_splits, int y_rows,
+                         const float* scale, const float* mix, const float* out_w, const float* in_w, float* x_out,
+                         long long out_stride, const int32_t* rows, const void* norm_w, float eps, void* out, int n_rows,
+                         int hidden, int dtype, void* stream);
 // x <- x * scale; then, with cap > 0, x <- cap * tanh(x / cap)
 int egpt_tanh_cap(float* x, float scale, float cap, long long n, void* stream);
 // ---- head_prep.hip: norms over a whole projection, a position factor on the queries, the store into pages
@@ -213,7 +228,7 @@ int egpt_whole_norm_store(const void* proj, int n_splits, int row_width, const v
                           const void* q_weight, const void* k_weight, float eps, const int32_t* positions, float coef,
                           int every, const int32_t* slots, void* k_cache, void* v_cache, int n_tokens, int nq, int nkv,
                           int dk, int dv, int page_size, int dtype, void* stream);
-// out = per-head rmsnorm(x) * weight[dv] * silu(gate columns gate_off.. of a product row); x float32 [n_tokens][heads][dv]
+// out = per-head rmsnorm(x) * weight[dv] (null: no weight) * silu(gate columns gate_off.. of a product row); x float32 [n_tokens][heads][dv]
 // (x_splits 0) or partial sums [x_splits][n_tokens][heads][dv]; gate null: no gate
 // (x rows are x_width values wide, the heads from place 0; x_is_act: x is one tensor of the activation type; gate_act: 0
 // silu, 1 sigmoid, 2 the gate's columns are the factor itself)
@@ -232,13 +247,26 @@ int egpt_bounded_gate(const void* z, int z_splits, int z_width, int z_off, const
 // float32 [slots][heads][dk][dv] is read from and written to states[slot[b]] (fresh[b] != 0: it starts at zero).
 // q, k, v: columns q_off, k_off, v_off of a product row of proj_width values.  out float32 [egpt_scan_key_splits(dk)][n_tokens][heads][dv]:
 // partial sums over ranges of the key channels, for the consumer to add.  q_silu: q_t is silu of its columns;
-// tied_keys: k_t = 1 - decay_t (k_off is not read).
+// tied_keys: k_t = 1 - decay_t (k_off is not read).  rot_dims > 0: the first rot_dims places of queries and keys turn by the
+// angles in cos_sin float32 [n_tokens][rot_dims / 2][2] (both times mag; place i with i + rot_dims / 2, interleaved: 2i with
+// 2i + 1; neither SiLU nor tied keys then); keys are multiplied by k_scale.
 int egpt_scan_key_splits(int dk);
 int egpt_decayed_state_scan(const void* proj, int n_splits, int proj_width, int q_off, int k_off, int v_off, float q_scale,
                             const float* decay, float* states, const int32_t* slots, const unsigned char* fresh,
                             const int32_t* q_start, const int32_t* q_len, int n_seqs, int n_tokens, float* out, int heads,
                             int dk, int dv, int q_silu, int tied_keys, int k_silu, int v_silu, const float* head_decay,
-                            int dtype, void* stream);
+                            const float* cos_sin, int rot_dims, float mag, int interleaved, float k_scale, int dtype, void* stream);
+// ---- constant_decay.hip: S_t = d_h S_(t-1) + (k_scale k_t) v_t^T, o_t = S_t^T q_t with queries and keys rotated as above, from the
+// product to the gated heads: out [n_tokens][heads * dv] = o / rms(o) per head * norm_w [dv] (null: no weight) * act(gate columns),
+// gate_act 0 silu, 1 sigmoid.  powers float32 [heads][65]: d_h^0 .. d_h^64.  n_chunks > 0: in chunks of egpt_decay_chunk(dk, dv)
+// tokens, n_chunks being at least the number of all requests' chunks and chunk_states float32 [n_chunks][heads][dk][dv]
+// scratch; n_chunks == 0: token by token.  dk, dv up to 256 (egpt_decay_chunk is 0 beyond).
+int egpt_decay_chunk(int dk, int dv);
+int egpt_constant_decay(const void* proj, int n_splits, int proj_width, int q_off, int k_off, int v_off, int g_off, float k_scale,
+                        const float* cos_sin, int rot_dims, int interleaved, float mag, const float* powers, float* states,
+                        const int32_t* slots, const unsigned char* fresh, const int32_t* q_start, const int32_t* q_len, int n_seqs,
+                        int n_tokens, float* chunk_states, int n_chunks, const void* norm_w, float eps, int gate_act, void* out,
+                        int heads, int dk, int dv, int dtype, void* stream);
 // The columns col0.. of a product row as inputs of `channels` short causal convolutions over time (weights [channels][taps],
 // the last tap the current token's; the taps - 1 inputs before a step's first token come from the request's record and
 // the record is brought up to date behind), SiLU, unit vectors head by head over the first unit_heads * unit_dim channels

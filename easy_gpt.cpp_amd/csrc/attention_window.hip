@@ -1,13 +1,14 @@
 // Softmax attention over the paged cache with separate key and value sizes, a window that keeps the first tokens,
 // a sink in the softmax, a learned bias per head and distance, keys visible only within the query's own block of
-// positions, and a penalty per head that grows with the distance; ragged batches (prompt portions and single decoded tokens in one launch).
+// positions, a penalty per head that grows with the distance, a tanh cap on the scores and a gate per head on the output; ragged batches (prompt portions and single decoded tokens in one launch).
 //
 // Query i of request b stands at position p = kv_len[b] - q_len[b] + i and sees key j if j <= p and
 // (window == 0 or p - j < window or j < keep_first).  score = (q . k) * scale over the key size dk; the softmax is
 // over the visible keys, and with a sink its denominator also holds exp(sink[head]), which has no key and no value
 // and is not scaled; with a distance bias [nq][far + 1] the score of key j gets bias[head][min(p - j, far)] added, unscaled;
 // with block > 0 a key is seen only if floor(j / block) == floor(p / block) (blocks are counted from position 0 of the
-// request, wherever a step cuts it); with slopes [nq] the score of key j loses slopes[head] * (p - j), unscaled;
+// request, wherever a step cuts it); with slopes [nq] the score of key j loses slopes[head] * (p - j), unscaled; with a cap c > 0
+// the scaled score s becomes c tanh(s / c) (the sink is not capped); with a head gate [T][nq] a head's output is multiplied by it;
 // the output is the weighted sum of the values of size dv.  Query head h reads key/value head
 // h / (nq / nkv).  Queries q [T][nq][dk]; keys in pages [page][kv head][offset][dk], values in pages
 // [page][kv head][dv][offset]; nothing that is not visible is read, so pages need no clearing and pages that a window
@@ -82,7 +83,8 @@ __global__ __launch_bounds__(64 * kSimpleWaves) void window_attention_simple_ker
     const int32_t* __restrict__ block_table, int table_width, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ q_len, const int32_t* __restrict__ kv_len, int n_seqs, int nq, int nkv, int dk, int dv,
     int page_size, float scale, int window, int keep_first, const float* __restrict__ sink,
-    const float* __restrict__ dist_bias, int dist_far, int block, const float* __restrict__ slopes) {
+    const float* __restrict__ dist_bias, int dist_far, int block, const float* __restrict__ slopes, float softcap,
+    const float* __restrict__ head_gate) {
     constexpr int kMaxOwn = kWidest / kWave;
     __shared__ __attribute__((aligned(16))) float q_s[kWidest];
     __shared__ float part_ml[kSimpleWaves][2];
@@ -109,6 +111,7 @@ __global__ __launch_bounds__(64 * kSimpleWaves) void window_attention_simple_ker
             const long page = table[j / page_size];
             const T* kr = k_cache + ((page * nkv + kvh) * page_size + j % page_size) * dk;
             s = dot_row(q_s, kr, dk) * scale;
+            if (softcap > 0.f) s = softcap * tanhf(s / softcap);
             if (dist_bias) s += dist_bias[static_cast<size_t>(h) * (dist_far + 1) + min(p - j, dist_far)];
             if (slopes) s -= slopes[h] * static_cast<float>(p - j);
         }
@@ -150,7 +153,7 @@ __global__ __launch_bounds__(64 * kSimpleWaves) void window_attention_simple_ker
     for (int w = 0; w < kSimpleWaves; ++w) m_all = fmaxf(m_all, part_ml[w][0]);
     float l_all = sink ? expf(sink[h] - m_all) : 0.f;
     for (int w = 0; w < kSimpleWaves; ++w) l_all = fmaf(part_ml[w][1], expf(part_ml[w][0] - m_all), l_all);
-    const float inv_l = 1.0f / l_all;
+    const float inv_l = (head_gate ? head_gate[static_cast<size_t>(t) * nq + h] : 1.0f) / l_all;
     T* o = out + (static_cast<size_t>(t) * nq + h) * dv;
 #pragma unroll
     for (int r = 0; r < kMaxOwn; ++r) {
@@ -220,6 +223,14 @@ __device__ __forceinline__ void store_four(T* dst, float a, float b, float c, fl
     }
 }
 
+// tanh for a cap on scores: float32 by the math library; beside bfloat16 products 1 - 2 / (exp(2 x) + 1), whose absolute
+// error is that of float32 numbers near 1
+template <typename T>
+__device__ __forceinline__ float bounded_tanh(float x) {
+    if constexpr (sizeof(T) == 4) return tanhf(x);
+    else return fmaf(-2.0f, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(x * 2.8853900817779268f) + 1.0f), 1.0f);
+}
+
 struct WindowArgs {
     const void* q;
     void* out;
@@ -235,6 +246,8 @@ struct WindowArgs {
     const float* dist_bias;  // [nq][dist_far + 1] or null
     int dist_far;
     const float* slopes;     // [nq] or null
+    const float* head_gate;  // [n_tokens][nq] or null: factors on the heads' outputs
+    float softcap;           // > 0: scores become softcap * tanh(score / softcap)
     int block;               // keys are seen within the query's block of this many positions (0: no blocks)
     int table_width, n_seqs, n_tokens, nq, nkv, dk, dv, page_size, window, keep_first, n_splits;
     int page_shift;          // log2 of the page size if that is a power of two, else -1
@@ -548,6 +561,18 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
                     }
+            } else if (a.softcap > 0.f) {
+                const float inner = scale / a.softcap;
+#pragma unroll
+                for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+                    for (int v = 0; v < 4; ++v) {
+                        const int key = key0 + kt * 16 + lg * 4 + v;
+                        const bool seen = whole || (key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first));
+                        const float sc = seen ? a.softcap * bounded_tanh<T>(acc[w][kt][v] * inner) : -INFINITY;
+                        acc[w][kt][v] = sc;
+                        mx = fmaxf(mx, sc);
+                    }
             } else if (whole) {
 #pragma unroll
                 for (int kt = 0; kt < NKT; ++kt)
@@ -644,7 +669,8 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
             weight = __builtin_amdgcn_exp2f((m_run[w] - m_all) * kLog2e);
             l = l * weight + __builtin_amdgcn_exp2f((sk - m_all) * kLog2e);
         }
-        const float inv = weight / l;
+        float inv = weight / l;
+        if (a.head_gate != nullptr) inv *= a.head_gate[static_cast<size_t>(tok[w]) * nq + head[w]];
         T* op = static_cast<T*>(a.out) + (static_cast<size_t>(tok[w]) * nq + head[w]) * dv + lg * 4;
 #pragma unroll
         for (int d = 0; d < DT; ++d)
@@ -658,7 +684,8 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
 template <typename T>
 __global__ __launch_bounds__(kWave) void window_attention_fold_kernel(const float* __restrict__ part_o,
                                                                     const float* __restrict__ part_ml,
-                                                                    const float* __restrict__ sink, T* __restrict__ out,
+                                                                    const float* __restrict__ sink,
+                                                                    const float* __restrict__ head_gate, T* __restrict__ out,
                                                                     int n_rows, int nq, int dv, int n_splits) {
     __shared__ float weights[kWave];           // at most 64 splits
     const int row = blockIdx.x, lane = threadIdx.x;
@@ -675,7 +702,7 @@ __global__ __launch_bounds__(kWave) void window_attention_fold_kernel(const floa
     if (sink) l_all += expf(sink[row % nq] - m_all);
     weights[lane] = w;
     __syncthreads();
-    const float inv = 1.0f / l_all;
+    const float inv = (head_gate ? head_gate[row] : 1.0f) / l_all;
     for (int d = lane; d < dv; d += kWave) {
         float acc = 0.f;
         for (int s = 0; s < n_splits; ++s)
@@ -735,10 +762,11 @@ extern "C" int egpt_window_attention(const void* q, void* out, const void* k_cac
                                      const int32_t* q_len, const int32_t* kv_len, int n_seqs, int n_tokens, int nq,
                                      int nkv, int dk, int dv, int page_size, float scale, int window, int keep_first,
                                      const float* sink, const float* dist_bias, int dist_far, int block, const float* slopes,
-                                     int dtype, void* stream) {
+                                     float softcap, const float* head_gate, int dtype, void* stream) {
     if (!q || !out || !k_cache || !v_cache || !block_table || !q_start || !q_len || !kv_len) return EGPT_BAD_ARGUMENT;
     if (n_seqs <= 0 || n_tokens < 0 || nq <= 0 || nkv <= 0 || nq % nkv != 0 || dk <= 0 || dv <= 0 || page_size <= 0 ||
-        table_width <= 0 || window < 0 || keep_first < 0 || (dtype != 0 && dtype != 1) || (dist_bias && dist_far < 0) || block < 0)
+        table_width <= 0 || window < 0 || keep_first < 0 || (dtype != 0 && dtype != 1) || (dist_bias && dist_far < 0) || block < 0 ||
+        !(softcap >= 0.f) || (softcap > 0.f && (dist_bias || slopes)))
         return EGPT_BAD_ARGUMENT;
     if (dk > kWidest || dv > kWidest || nq > 65535) return EGPT_UNSUPPORTED_SIZE;
     if (n_tokens == 0) return EGPT_OK;
@@ -748,12 +776,12 @@ extern "C" int egpt_window_attention(const void* q, void* out, const void* k_cac
         window_attention_simple_kernel<float><<<grid, kWave * kSimpleWaves, 0, s>>>(
             static_cast<const float*>(q), static_cast<float*>(out), static_cast<const float*>(k_cache),
             static_cast<const float*>(v_cache), block_table, table_width, q_start, q_len, kv_len, n_seqs, nq, nkv, dk,
-            dv, page_size, scale, window, keep_first, sink, dist_bias, dist_far, block, slopes);
+            dv, page_size, scale, window, keep_first, sink, dist_bias, dist_far, block, slopes, softcap, head_gate);
     else
         window_attention_simple_kernel<bf16_t><<<grid, kWave * kSimpleWaves, 0, s>>>(
             static_cast<const bf16_t*>(q), static_cast<bf16_t*>(out), static_cast<const bf16_t*>(k_cache),
             static_cast<const bf16_t*>(v_cache), block_table, table_width, q_start, q_len, kv_len, n_seqs, nq, nkv, dk,
-            dv, page_size, scale, window, keep_first, sink, dist_bias, dist_far, block, slopes);
+            dv, page_size, scale, window, keep_first, sink, dist_bias, dist_far, block, slopes, softcap, head_gate);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }
@@ -763,12 +791,13 @@ extern "C" int egpt_window_attention_tiled(const void* q, void* out, float* part
                                            const int32_t* q_start, const int32_t* q_len, const int32_t* kv_len, int n_seqs,
                                            int n_tokens, int nq, int nkv, int dk, int dv, int page_size, float scale,
                                            int window, int keep_first, const float* sink, const float* dist_bias,
-                                           int dist_far, int block, const float* slopes, int n_splits, int row_tiles, int dtype,
-                                           void* stream) {
+                                           int dist_far, int block, const float* slopes, float softcap, const float* head_gate,
+                                           int n_splits, int row_tiles, int dtype, void* stream) {
     if (!q || !out || !k_cache || !v_cache || !block_table || !q_start || !q_len || !kv_len) return EGPT_BAD_ARGUMENT;
     if (n_seqs <= 0 || n_tokens < 0 || nq <= 0 || nkv <= 0 || nq % nkv != 0 || dk <= 0 || dv <= 0 || page_size <= 0 ||
         table_width <= 0 || window < 0 || keep_first < 0 || n_splits < 1 || (dtype != 0 && dtype != 1) ||
-        (row_tiles != 4 && row_tiles != 8) || (dist_bias && dist_far < 0) || block < 0 || (dist_bias && slopes))
+        (row_tiles != 4 && row_tiles != 8) || (dist_bias && dist_far < 0) || block < 0 || (dist_bias && slopes) ||
+        !(softcap >= 0.f) || (softcap > 0.f && (dist_bias || slopes)))
         return EGPT_BAD_ARGUMENT;
     if (n_splits > 1 && (!part_o || !part_ml)) return EGPT_BAD_ARGUMENT;
     const int e = dtype == 0 ? 4 : 8;
@@ -779,6 +808,7 @@ extern "C" int egpt_window_attention_tiled(const void* q, void* out, float* part
     a.q = q; a.out = out; a.part_o = part_o; a.part_ml = part_ml; a.k_cache = k_cache; a.v_cache = v_cache;
     a.block_table = block_table; a.q_start = q_start; a.q_len = q_len; a.kv_len = kv_len; a.sink = sink;
     a.dist_bias = dist_bias; a.dist_far = dist_far; a.slopes = slopes; a.block = block;
+    a.softcap = softcap; a.head_gate = head_gate;
     a.table_width = table_width; a.n_seqs = n_seqs; a.n_tokens = n_tokens; a.nq = nq; a.nkv = nkv; a.dk = dk; a.dv = dv;
     a.page_size = page_size; a.window = window; a.keep_first = keep_first; a.n_splits = n_splits; a.scale = scale;
     a.page_shift = -1;
@@ -793,10 +823,10 @@ extern "C" int egpt_window_attention_tiled(const void* q, void* out, float* part
     EGPT_CHECK_LAUNCH();
     if (n_splits > 1) {
         if (dtype == 0)
-            window_attention_fold_kernel<float><<<n_tokens * nq, kWave, 0, s>>>(part_o, part_ml, sink, static_cast<float*>(out),
+            window_attention_fold_kernel<float><<<n_tokens * nq, kWave, 0, s>>>(part_o, part_ml, sink, head_gate, static_cast<float*>(out),
                                                                                n_tokens * nq, nq, dv, n_splits);
         else
-            window_attention_fold_kernel<bf16_t><<<n_tokens * nq, kWave, 0, s>>>(part_o, part_ml, sink,
+            window_attention_fold_kernel<bf16_t><<<n_tokens * nq, kWave, 0, s>>>(part_o, part_ml, sink, head_gate,
                                                                                 static_cast<bf16_t*>(out), n_tokens * nq, nq,
                                                                                 dv, n_splits);
         EGPT_CHECK_LAUNCH();

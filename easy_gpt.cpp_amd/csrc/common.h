@@ -42,6 +42,14 @@ __device__ __forceinline__ void rotate_pair(float a, float b, float c, float s, 
     rb = __fmaf_rn(a, s, __fmul_rn(b, c));
 }
 
+// The activation of a gated feed-forward's gate: 0 silu, z / (1 + exp(-z)); 1 the tanh form of gelu,
+// z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), which is z / (1 + exp(-2 sqrt(2 / pi) (z + 0.044715 z^3))).
+constexpr int kGateSilu = 0, kGateGeluTanh = 1;
+__device__ __forceinline__ float gate_exponent(float z, int act) {
+    return act == kGateSilu ? z : 1.5957691216057308f * fmaf(0.044715f * z * z, z, z);
+}
+__device__ __forceinline__ float gate_activation(float z, int act) { return z / (1.0f + expf(-gate_exponent(z, act))); }
+
 // The residual stream of steps of few tokens in 64-bit fixed point (units of 2^-32).  Several workgroups that split
 // a product's k range add their partial results straight into it with integer atomics: integer addition does not
 // care for the order, so the sum is the same bits whatever the scheduling, and the kernels that read the stream

@@ -173,16 +173,17 @@ __global__ __launch_bounds__(256) void add_rmsnorm_vec8_kernel(float* __restrict
 }
 
 // ----------------------------------------------------------------------------- SwiGLU
-// out = up * gate / (1 + exp(-gate))   (/root/reference/src/cuda/ops/mlp.cu:152-162); [gate | up] per row.
+// out = up * gate / (1 + exp(-gate))   (/root/reference/src/cuda/ops/mlp.cu:152-162); [gate | up] per row.  act names the
+// gate's activation (gate_activation in common.h).
 template <typename T>
-__global__ void swiglu_kernel(ProductView<T> gate_up, T* __restrict__ out, int n_tokens, int inter) {
+__global__ void swiglu_kernel(ProductView<T> gate_up, T* __restrict__ out, int n_tokens, int inter, int act) {
     const size_t total = static_cast<size_t>(n_tokens) * inter;
     for (size_t i = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; i < total;
          i += static_cast<size_t>(gridDim.x) * blockDim.x) {
         const size_t t = i / inter, j = i % inter;
         const float g = gate_up.at(t * 2 * inter + j);
         const float u = gate_up.at(t * 2 * inter + inter + j);
-        out[i] = from_float<T>(u * (g / (1.0f + expf(-g))));
+        out[i] = from_float<T>(u * gate_activation(g, act));
     }
 }
 
@@ -191,7 +192,7 @@ __global__ void swiglu_kernel(ProductView<T> gate_up, T* __restrict__ out, int n
 // up before the activation.  One row of workgroups per token.
 template <typename T>
 __global__ void swiglu_scaled_kernel(ProductView<float> gate_up, const float* __restrict__ row_ss, int ss_splits,
-                                     float inv_hidden, float eps, T* __restrict__ out, int n_tokens, int inter) {
+                                     float inv_hidden, float eps, T* __restrict__ out, int n_tokens, int inter, int act) {
     const size_t t = blockIdx.y;
     float ss = 0.f;
     for (int s = 0; s < ss_splits; ++s) ss += row_ss[static_cast<size_t>(s) * n_tokens + t];
@@ -199,14 +200,14 @@ __global__ void swiglu_scaled_kernel(ProductView<float> gate_up, const float* __
     for (int j = blockIdx.x * blockDim.x + threadIdx.x; j < inter; j += gridDim.x * blockDim.x) {
         const float g = scale_then_bias(gate_up.at(t * 2 * inter + j), scale, 0.f);
         const float u = scale_then_bias(gate_up.at(t * 2 * inter + inter + j), scale, 0.f);
-        out[t * inter + j] = from_float<T>(u * (g / (1.0f + expf(-g))));
+        out[t * inter + j] = from_float<T>(u * gate_activation(g, act));
     }
 }
 
 // bfloat16, eight features per thread (inter % 8 == 0, one tensor, no partial sums)
 template <typename GT>
 __global__ __launch_bounds__(256) void swiglu_vec8_kernel(const GT* __restrict__ gate_up, bf16_t* __restrict__ out,
-                                                          int n_tokens, int inter) {
+                                                          int n_tokens, int inter, int act) {
     const size_t chunks_per_row = inter / 8;
     const size_t total = static_cast<size_t>(n_tokens) * chunks_per_row;
     for (size_t c = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; c < total;
@@ -218,8 +219,8 @@ __global__ __launch_bounds__(256) void swiglu_vec8_kernel(const GT* __restrict__
         uint32_t ow[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            const float r0 = u[2 * i] * (g[2 * i] / (1.0f + expf(-g[2 * i])));
-            const float r1 = u[2 * i + 1] * (g[2 * i + 1] / (1.0f + expf(-g[2 * i + 1])));
+            const float r0 = u[2 * i] * gate_activation(g[2 * i], act);
+            const float r1 = u[2 * i + 1] * gate_activation(g[2 * i + 1], act);
             ow[i] = f32_to_bf16_bits(r0) | (static_cast<uint32_t>(f32_to_bf16_bits(r1)) << 16);
         }
         *reinterpret_cast<uint4*>(out + t * inter + j) = uint4{ow[0], ow[1], ow[2], ow[3]};
@@ -471,8 +472,8 @@ extern "C" int egpt_add_rmsnorm(void* h, int fixed, const void* delta, int delta
 }
 
 extern "C" int egpt_swiglu(const void* gate_up, int n_splits, const float* row_ss, int ss_splits, int hidden, float eps,
-                           void* out, int n_tokens, int inter, int dtype, void* stream) {
-    if (!gate_up || !out || n_tokens < 0 || inter <= 0 || n_splits < 0) return EGPT_BAD_ARGUMENT;
+                           void* out, int n_tokens, int inter, int act, int dtype, void* stream) {
+    if (!gate_up || !out || (act != kGateSilu && act != kGateGeluTanh) || n_tokens < 0 || inter <= 0 || n_splits < 0) return EGPT_BAD_ARGUMENT;
     if (n_tokens == 0) return EGPT_OK;
     hipStream_t s = static_cast<hipStream_t>(stream);
     const size_t total = static_cast<size_t>(n_tokens) * inter;
@@ -487,10 +488,10 @@ extern "C" int egpt_swiglu(const void* gate_up, int n_splits, const float* row_s
         const ProductView<float> view = make_view<float>(gate_up, n_splits, stride);
         if (dtype == 0)
             swiglu_scaled_kernel<float><<<grid, 256, 0, s>>>(view, row_ss, ss_splits, 1.0f / hidden, eps,
-                                                             static_cast<float*>(out), n_tokens, inter);
+                                                             static_cast<float*>(out), n_tokens, inter, act);
         else
             swiglu_scaled_kernel<bf16_t><<<grid, 256, 0, s>>>(view, row_ss, ss_splits, 1.0f / hidden, eps,
-                                                              static_cast<bf16_t*>(out), n_tokens, inter);
+                                                              static_cast<bf16_t*>(out), n_tokens, inter, act);
         EGPT_CHECK_LAUNCH();
         return EGPT_OK;
     }
@@ -499,19 +500,19 @@ extern "C" int egpt_swiglu(const void* gate_up, int n_splits, const float* row_s
         const int vblocks = static_cast<int>(chunks / 256 + 1 > 16384 ? 16384 : chunks / 256 + 1);
         if (n_splits == 0)
             swiglu_vec8_kernel<bf16_t><<<vblocks, 256, 0, s>>>(static_cast<const bf16_t*>(gate_up),
-                                                               static_cast<bf16_t*>(out), n_tokens, inter);
+                                                               static_cast<bf16_t*>(out), n_tokens, inter, act);
         else
             swiglu_vec8_kernel<float><<<vblocks, 256, 0, s>>>(static_cast<const float*>(gate_up),
-                                                              static_cast<bf16_t*>(out), n_tokens, inter);
+                                                              static_cast<bf16_t*>(out), n_tokens, inter, act);
         EGPT_CHECK_LAUNCH();
         return EGPT_OK;
     }
     if (dtype == 0)
         swiglu_kernel<float><<<blocks, 256, 0, s>>>(make_view<float>(gate_up, n_splits, stride),
-                                                    static_cast<float*>(out), n_tokens, inter);
+                                                    static_cast<float*>(out), n_tokens, inter, act);
     else if (dtype == 1)
         swiglu_kernel<bf16_t><<<blocks, 256, 0, s>>>(make_view<bf16_t>(gate_up, n_splits, stride),
-                                                     static_cast<bf16_t*>(out), n_tokens, inter);
+                                                     static_cast<bf16_t*>(out), n_tokens, inter, act);
     else
         return EGPT_BAD_ARGUMENT;
     EGPT_CHECK_LAUNCH();
@@ -599,4 +600,4 @@ extern "C" const char* egpt_error_string(int code) {
     }
 }
 
-extern "C" int egpt_abi_version(void) { return 24; }
+extern "C" int egpt_abi_version(void) { return 25; }

@@ -29,7 +29,7 @@ __device__ __forceinline__ uint4 load16_if(const bf16_t* p, bool ok) {
 template <int MT, int KC, int NG>
 __global__ __launch_bounds__(64 * kGuWaves) void gemm_gate_up_kernel(const bf16_t* __restrict__ x,
                                                                      const bf16_t* __restrict__ w,
-                                                                     bf16_t* __restrict__ out, int m, int inter, int k) {
+                                                                     bf16_t* __restrict__ out, int m, int inter, int k, int act) {
     __shared__ f32x4 part[kGuWaves][MT][NG][2][kWave];
     const int lane = threadIdx.x % kWave;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
@@ -124,32 +124,32 @@ __global__ __launch_bounds__(64 * kGuWaves) void gemm_gate_up_kernel(const bf16_
         for (int v = 0; v < 4; ++v) {
             const int row = tt * 16 + lg * 4 + v;
             if (row < m)
-                out[static_cast<size_t>(row) * inter + column] = from_float<bf16_t>(u[v] * (g[v] / (1.0f + expf(-g[v]))));
+                out[static_cast<size_t>(row) * inter + column] = from_float<bf16_t>(u[v] * gate_activation(g[v], act));
         }
     }
 }
 
 template <int MT, int NG>
-static void launch_gate_up(const bf16_t* x, const bf16_t* w, bf16_t* out, int m, int inter, int k, hipStream_t s) {
+static void launch_gate_up(const bf16_t* x, const bf16_t* w, bf16_t* out, int m, int inter, int k, int act, hipStream_t s) {
     const int blocks = (inter + kGuCols * NG - 1) / (kGuCols * NG);
     const int per_wave = ((k + 31) / 32 + kGuWaves - 1) / kGuWaves;
     [[maybe_unused]] const dim3 grid(blocks);
     // rounds of 7 or 8 chunks: the fewer rounds, and of those the fewer registers
     if ((per_wave + 7) / 8 < (per_wave + 6) / 7)
-        gemm_gate_up_kernel<MT, 8, NG><<<blocks, 64 * kGuWaves, 0, s>>>(x, w, out, m, inter, k);
+        gemm_gate_up_kernel<MT, 8, NG><<<blocks, 64 * kGuWaves, 0, s>>>(x, w, out, m, inter, k, act);
     else
-        gemm_gate_up_kernel<MT, 7, NG><<<blocks, 64 * kGuWaves, 0, s>>>(x, w, out, m, inter, k);
+        gemm_gate_up_kernel<MT, 7, NG><<<blocks, 64 * kGuWaves, 0, s>>>(x, w, out, m, inter, k, act);
 }
 
 }  // namespace egpt
 
 using namespace egpt;
 
-// out bfloat16 [m][inter] = SwiGLU of x w^T; x bfloat16 [m][k], w bfloat16 [2 * inter][k] (gate rows, then up rows);
+// out bfloat16 [m][inter] = SwiGLU of x w^T (or with another activation of the gate, gate_activation in common.h); x bfloat16 [m][k], w bfloat16 [2 * inter][k] (gate rows, then up rows);
 // m <= 64, k % 8 == 0.
 extern "C" int egpt_gemm_gate_up_swiglu(const void* x, const void* w, void* out, int m, int inter, int k, int groups,
-                                        void* stream) {
-    if (!x || !w || !out || m <= 0 || inter <= 0 || k <= 0) return EGPT_BAD_ARGUMENT;
+                                        int act, void* stream) {
+    if ((act != kGateSilu && act != kGateGeluTanh) || !x || !w || !out || m <= 0 || inter <= 0 || k <= 0) return EGPT_BAD_ARGUMENT;
     if (m > 64 || (k % 8) != 0 || (groups != 1 && groups != 2)) return EGPT_UNSUPPORTED_SIZE;
     const bf16_t* xb = static_cast<const bf16_t*>(x);
     const bf16_t* wb = static_cast<const bf16_t*>(w);
@@ -157,8 +157,8 @@ extern "C" int egpt_gemm_gate_up_swiglu(const void* x, const void* w, void* out,
     hipStream_t s = static_cast<hipStream_t>(stream);
 #define EGPT_GATE_UP(MT_)                                                        \
     do {                                                                         \
-        if (groups == 1) launch_gate_up<MT_, 1>(xb, wb, ob, m, inter, k, s);     \
-        else launch_gate_up<MT_, 2>(xb, wb, ob, m, inter, k, s);                 \
+        if (groups == 1) launch_gate_up<MT_, 1>(xb, wb, ob, m, inter, k, act, s); \
+        else launch_gate_up<MT_, 2>(xb, wb, ob, m, inter, k, act, s);             \
     } while (0)
     switch ((m + 15) / 16) {
         case 1: EGPT_GATE_UP(1); break;

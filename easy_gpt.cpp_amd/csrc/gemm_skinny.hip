@@ -57,6 +57,7 @@ struct SkinnyArgs {
     // kSwiglu: x[m][k] from gate_up [gu_splits][m][2k]
     const float* gu;
     int gu_splits;
+    int act;                   // the gate's activation (gate_activation in common.h)
     const float* ss_in;        // [ss_splits][m] or null
     int ss_splits;
     float inv_hidden, eps;
@@ -286,7 +287,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_skinny_kernel(SkinnyArgs a) {
 #pragma unroll
                 for (int j = 0; j < 8; ++j) {
                     const float gg = g[j] * inv;
-                    f[j] = (u[j] * inv) * gg * __builtin_amdgcn_rcpf(1.0f + __expf(-gg));
+                    f[j] = (u[j] * inv) * gg * __builtin_amdgcn_rcpf(1.0f + __expf(-gate_exponent(gg, a.act)));
                 }
             } else {  // kAttn
                 const int head = kc / a.hd, d = kc % a.hd;
@@ -682,8 +683,8 @@ extern "C" int egpt_gemm_skinny_norm(const void* h_in, int h_fixed, float* h_out
 // inv_rms[m] = 1 / sqrt(sum_s ss_in[s][m] / hidden + eps), or 1 if ss_in is null.
 extern "C" int egpt_gemm_skinny_swiglu(const float* gate_up, int gu_splits, const float* ss_in, int ss_splits,
                                        int hidden, float eps, const void* w, float* out, void* acc_fixed, int m, int n,
-                                       int k, int n_splits, int waves, void* stream) {
-    if (!gate_up || gu_splits < 1 || !w || (!out == !acc_fixed) || m <= 0 || n <= 0 || k <= 0 || (ss_in && (ss_splits < 1 || hidden < 1)) ||
+                                       int k, int n_splits, int waves, int act, void* stream) {
+    if (!gate_up || gu_splits < 1 || (act != kGateSilu && act != kGateGeluTanh) || !w || (!out == !acc_fixed) || m <= 0 || n <= 0 || k <= 0 || (ss_in && (ss_splits < 1 || hidden < 1)) ||
         (waves != 4 && waves != 8 && waves != 16))
         return EGPT_BAD_ARGUMENT;
     if (m > 16 || (k % 8) != 0) return EGPT_UNSUPPORTED_SIZE;
@@ -696,6 +697,7 @@ extern "C" int egpt_gemm_skinny_swiglu(const float* gate_up, int gu_splits, cons
     a.gu = gate_up; a.gu_splits = gu_splits; a.ss_in = ss_in; a.ss_splits = ss_splits;
     a.inv_hidden = ss_in ? 1.0f / static_cast<float>(hidden) : 0.f;
     a.eps = eps;
+    a.act = act;
     EGPT_SKINNY(1, kSwiglu, 8);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;

@@ -58,21 +58,44 @@ __global__ __launch_bounds__(256) void embed_rmsnorm_kernel(const int32_t* __res
 // place i with place i + rot_dims / 2, or with kInterleaved place 2i with place 2i + 1; behind the norm, or with
 // kNormAfterRotation before it.  Queries go to q_out [T][nq * dk]; keys and values to the pages at slots[t] (slots
 // null: nothing is stored).
+// Further operands (HeadExtras, all may be absent): values_out takes the value heads as float32 [T][nkv * dv] before any mixing;
+// with mix_with float32 [T][nkv * dv] a value becomes (1 - mix) * value + mix * mix_with, and that is what is stored; the n_gates
+// columns from gate_off on become sigmoids in gates_out float32 [T][n_gates] (a gate of one number per head, say).
 constexpr int kNormValues = 1, kNormPlain = 2, kNormAfterRotation = 4, kValuesAreKeys = 8, kInterleaved = 16;
+
+struct HeadExtras {
+    float* values_out;
+    const float* mix_with;
+    float mix;
+    int n_gates, gate_off;
+    float* gates_out;
+    __device__ __forceinline__ float value(size_t place, float v) const {      // place: token * (nkv * dv) + column
+        if (values_out != nullptr) values_out[place] = v;
+        return mix_with != nullptr ? (1.0f - mix) * v + mix * mix_with[place] : v;
+    }
+};
 
 template <typename T>
 __global__ __launch_bounds__(kWave) void head_norm_store_kernel(
     ProductView<T> proj, RowFactor factor, int row_width, T* __restrict__ q_out, const T* __restrict__ q_weight,
     const T* __restrict__ k_weight, float eps, int flags, const float* __restrict__ cos_sin, int rot_dims, float mag,
     const int32_t* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache, int nq, int nkv,
-    int dk, int dv, int page_size) {
+    int dk, int dv, int page_size, HeadExtras ex) {
     const int t = blockIdx.x, hh = blockIdx.y, lane = threadIdx.x;
+    if (hh >= nq + 2 * nkv) {                             // one more wavefront per token for the gates
+        const float f = factor.of(t);
+        for (int c = lane; c < ex.n_gates; c += kWave) {
+            const float z = proj.at(static_cast<size_t>(t) * row_width + ex.gate_off + c) * f;
+            ex.gates_out[static_cast<size_t>(t) * ex.n_gates + c] = 1.0f / (1.0f + expf(-z));
+        }
+        return;
+    }
     const int kind = hh < nq ? 0 : (hh < nq + nkv ? 1 : 2);
     const int head = kind == 0 ? hh : (kind == 1 ? hh - nq : hh - nq - nkv);
     const int width = kind == 2 ? dv : dk;
     const bool own_keys = kind == 2 && (flags & kValuesAreKeys);
     const int in_off = kind == 0 ? head * dk : ((kind == 1 || own_keys) ? nq * dk + head * dk : (nq + nkv) * dk + head * dv);
-    if (kind != 0 && slots == nullptr) return;
+    if (kind != 0 && slots == nullptr && (kind == 1 || ex.values_out == nullptr)) return;
     const T* weight = kind == 0 ? q_weight : (kind == 1 ? k_weight : nullptr);
     const bool normed = kind == 2 ? (flags & kNormValues) != 0 : (weight != nullptr || (flags & kNormPlain));
     const int rot = kind == 2 ? 0 : rot_dims;
@@ -113,7 +136,7 @@ __global__ __launch_bounds__(kWave) void head_norm_store_kernel(
     if (normed) inv = inv_rms(wave_sum(ss), 1.0f / static_cast<float>(width), eps);
     long page = 0;
     int off = 0;
-    if (kind != 0) {
+    if (kind != 0 && slots != nullptr) {
         page = slots[t] / page_size;
         off = slots[t] % page_size;
     }
@@ -133,8 +156,74 @@ __global__ __launch_bounds__(kWave) void head_norm_store_kernel(
             q_out[static_cast<size_t>(t) * nq * dk + head * dk + d] = from_float<T>(y);
         else if (kind == 1)
             k_cache[((page * nkv + head) * page_size + off) * dk + d] = from_float<T>(y);
-        else
-            v_cache[((page * nkv + head) * dv + d) * page_size + off] = from_float<T>(y);
+        else {
+            y = ex.value((static_cast<size_t>(t) * nkv + head) * dv + d, y);
+            if (slots != nullptr) v_cache[((page * nkv + head) * dv + d) * page_size + off] = from_float<T>(y);
+        }
+    }
+}
+
+// The same for heads that are not normed: nothing in a head depends on the rest of it, so a thread takes one pair of
+// places that turn together (or two neighbouring places that pass), one value, or one gate.  NT tokens to a row of
+// workgroups (grid x), a thread per item (grid y): the pairs token by token, then the values with the tokens of one feature
+// side by side (they are neighbours in a page), then the gates.
+template <typename T, int NT>
+__global__ __launch_bounds__(256) void head_turn_store_kernel(
+    ProductView<T> proj, RowFactor factor, int row_width, T* __restrict__ q_out, int flags, const float* __restrict__ cos_sin,
+    int rot_dims, float mag, const int32_t* __restrict__ slots, T* __restrict__ k_cache, T* __restrict__ v_cache, int n_tokens,
+    int nq, int nkv, int dk, int dv, int page_size, HeadExtras ex) {
+    const int half = rot_dims / 2, per_head = half + (dk - rot_dims + 1) / 2;
+    const int n_pairs = (nq + nkv) * per_head, n_values = nkv * dv;
+    int item = blockIdx.y * 256 + threadIdx.x;
+    const int t0 = blockIdx.x * NT;
+    if (item < NT * n_pairs) {
+        const int t = t0 + item / n_pairs, rem = item % n_pairs;
+        const int head = rem / per_head, s = rem % per_head;
+        if (t >= n_tokens || (head >= nq && slots == nullptr)) return;
+        const bool turned = s < half;
+        int a, b;
+        if (turned) {
+            a = (flags & kInterleaved) ? 2 * s : s;
+            b = (flags & kInterleaved) ? 2 * s + 1 : s + half;
+        } else {
+            a = rot_dims + 2 * (s - half);
+            b = a + 1;
+        }
+        const size_t base = static_cast<size_t>(t) * row_width + static_cast<size_t>(head) * dk;
+        const float rf = factor.of(t);
+        float x = proj.at(base + a) * rf, y = b < dk ? proj.at(base + b) * rf : 0.f;
+        if (turned) {
+            const float* cs = cos_sin + static_cast<size_t>(t) * rot_dims + 2 * s;
+            rotate_pair(x, y, cs[0] * mag, cs[1] * mag, x, y);
+        }
+        T* dst;
+        if (head < nq) {
+            dst = q_out + (static_cast<size_t>(t) * nq + head) * dk;
+        } else {
+            const long page = slots[t] / page_size;
+            dst = k_cache + ((page * nkv + (head - nq)) * page_size + slots[t] % page_size) * dk;
+        }
+        dst[a] = from_float<T>(x);
+        if (b < dk) dst[b] = from_float<T>(y);
+        return;
+    }
+    item -= NT * n_pairs;
+    if (item < NT * n_values) {
+        const int t = t0 + item % NT, c = item / NT;
+        if (t >= n_tokens || (slots == nullptr && ex.values_out == nullptr)) return;
+        const int src = (flags & kValuesAreKeys) ? nq * dk + c : (nq + nkv) * dk + c;
+        const float v = ex.value(static_cast<size_t>(t) * n_values + c, proj.at(static_cast<size_t>(t) * row_width + src) * factor.of(t));
+        if (slots == nullptr) return;
+        const long page = slots[t] / page_size;
+        v_cache[(page * n_values + c) * page_size + slots[t] % page_size] = from_float<T>(v);
+        return;
+    }
+    item -= NT * n_values;
+    if (item < NT * ex.n_gates) {
+        const int t = t0 + item / ex.n_gates, c = item % ex.n_gates;
+        if (t >= n_tokens) return;
+        const float z = proj.at(static_cast<size_t>(t) * row_width + ex.gate_off + c) * factor.of(t);
+        ex.gates_out[static_cast<size_t>(t) * ex.n_gates + c] = 1.0f / (1.0f + expf(-z));
     }
 }
 
@@ -314,7 +403,7 @@ __global__ __launch_bounds__(256) void whole_norm_store_kernel(
 }
 
 // out[t][h * dv + d] = x[t][h * dv + d] / rms(x[t][h * dv ..]) * weight[d] * act(g[t][gate_off + h * dv + d]): the
-// RMS norm of every head's output with a weight that the heads share, and a gate from columns of a product row (no
+// RMS norm of every head's output with a weight that the heads share (null: none), and a gate from columns of a product row (no
 // gate: the normed heads as they are).  x is float32 (one tensor, or partial sums that are added here) or, with xa
 // present, a product in the activation type; its rows are x_width values wide and the heads begin at place 0.  The
 // gate's activation: 0 silu, 1 sigmoid, 2 none (the columns hold the factor itself).  One wavefront per (token, head).
@@ -333,7 +422,7 @@ __global__ __launch_bounds__(kWave) void head_norm_gate_kernel(ProductView<float
     }
     const float inv = inv_rms(wave_sum(ss), 1.0f / static_cast<float>(dv), eps);
     for (int d = lane; d < dv; d += kWave) {
-        float y = (act_typed ? xa.at(xr + d) : x.at(xr + d)) * inv * to_float(weight[d]);
+        float y = (act_typed ? xa.at(xr + d) : x.at(xr + d)) * inv * (weight ? to_float(weight[d]) : 1.0f);
         if (g.present()) {
             const float gate = g.at(static_cast<size_t>(t) * gate_width + gate_off + h * dv + d);
             const float sig = 1.0f / (1.0f + expf(-gate));
@@ -368,7 +457,7 @@ __global__ __launch_bounds__(256) void head_norm_gate_wide_kernel(ProductView<fl
     }
     const float inv = inv_rms(block_sum(ss, scratch), 1.0f / static_cast<float>(dv), eps);
     auto put = [&](int d, float value) {
-        float y = value * inv * to_float(weight[d]);
+        float y = value * inv * (weight ? to_float(weight[d]) : 1.0f);
         if (g.present()) {
             const float gate = g.at(static_cast<size_t>(t) * gate_width + gate_off + h * dv + d);
             const float sig = 1.0f / (1.0f + expf(-gate));
@@ -424,7 +513,9 @@ extern "C" int egpt_head_norm_store(const void* proj, int n_splits, const float*
                                     float norm_eps, int row_width, void* q_out, const void* q_weight,
                                     const void* k_weight, float eps, int flags, const float* cos_sin, int rot_dims, float mag,
                                     const int32_t* slots, void* k_cache, void* v_cache, int n_tokens, int nq, int nkv, int dk,
-                                    int dv, int page_size, int dtype, void* stream) {
+                                    int dv, int page_size, float* values_out, const float* mix_with, float mix, int n_gates,
+                                    int gate_off, float* gates_out, int dtype, void* stream) {
+    if (n_gates < 0 || (n_gates > 0 && (!gates_out || gate_off < 0 || gate_off + n_gates > row_width))) return EGPT_BAD_ARGUMENT;
     if (!proj || !q_out || n_splits < 0 || n_tokens < 0 || nq <= 0 || nkv <= 0 || dk <= 0 || dv <= 0 || page_size <= 0 ||
         (dtype != 0 && dtype != 1) || flags < 0 || flags >= 32)
         return EGPT_BAD_ARGUMENT;
@@ -438,17 +529,39 @@ extern "C" int egpt_head_norm_store(const void* proj, int n_splits, const float*
     if (row_ss && (n_splits < 1 || ss_splits < 1 || hidden <= 0)) return EGPT_BAD_ARGUMENT;
     const RowFactor factor{row_ss, ss_splits, n_tokens, hidden, norm_eps};
     const size_t stride = static_cast<size_t>(n_tokens) * row_width;
-    dim3 grid(n_tokens, nq + 2 * nkv);
+    const HeadExtras ex{values_out, mix_with, mix, n_gates, gate_off, gates_out};
+    if (!q_weight && !k_weight && !(flags & (kNormPlain | kNormValues))) {
+        const int nt = n_tokens >= 256 ? 8 : 1;           // (a prompt: the tokens of a page side by side)
+        const int per_head = rot_dims / 2 + (dk - rot_dims + 1) / 2;
+        const long long items = static_cast<long long>(nt) * ((nq + nkv) * per_head + nkv * dv + n_gates);
+        if ((items + 255) / 256 > 65535) return EGPT_UNSUPPORTED_SIZE;
+        const dim3 turn_grid((n_tokens + nt - 1) / nt, static_cast<unsigned>((items + 255) / 256));
+#define EGPT_TURN(T_, NT_)                                                                                                       \
+    head_turn_store_kernel<T_, NT_><<<turn_grid, 256, 0, s>>>(                                                                   \
+        view_of<T_>(proj, n_splits, stride), factor, row_width, static_cast<T_*>(q_out), flags, cos_sin, rot_dims, mag, slots,   \
+        static_cast<T_*>(k_cache), static_cast<T_*>(v_cache), n_tokens, nq, nkv, dk, dv, page_size, ex)
+        if (dtype == 0) {
+            if (nt == 8) EGPT_TURN(float, 8);
+            else EGPT_TURN(float, 1);
+        } else {
+            if (nt == 8) EGPT_TURN(bf16_t, 8);
+            else EGPT_TURN(bf16_t, 1);
+        }
+#undef EGPT_TURN
+        EGPT_CHECK_LAUNCH();
+        return EGPT_OK;
+    }
+    dim3 grid(n_tokens, nq + 2 * nkv + (n_gates > 0 ? 1 : 0));
     if (dtype == 0)
         head_norm_store_kernel<float><<<grid, kWave, 0, s>>>(
             view_of<float>(proj, n_splits, stride), factor, row_width, static_cast<float*>(q_out), static_cast<const float*>(q_weight),
             static_cast<const float*>(k_weight), eps, flags, cos_sin, rot_dims, mag, slots, static_cast<float*>(k_cache),
-            static_cast<float*>(v_cache), nq, nkv, dk, dv, page_size);
+            static_cast<float*>(v_cache), nq, nkv, dk, dv, page_size, ex);
     else
         head_norm_store_kernel<bf16_t><<<grid, kWave, 0, s>>>(
             view_of<bf16_t>(proj, n_splits, stride), factor, row_width, static_cast<bf16_t*>(q_out), static_cast<const bf16_t*>(q_weight),
             static_cast<const bf16_t*>(k_weight), eps, flags, cos_sin, rot_dims, mag, slots, static_cast<bf16_t*>(k_cache),
-            static_cast<bf16_t*>(v_cache), nq, nkv, dk, dv, page_size);
+            static_cast<bf16_t*>(v_cache), nq, nkv, dk, dv, page_size, ex);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }
@@ -544,7 +657,7 @@ extern "C" int egpt_whole_norm_store(const void* proj, int n_splits, int row_wid
 extern "C" int egpt_head_norm_gate(const void* x, int x_splits, int x_is_act, int x_width, const void* weight, float eps,
                                    const void* gate, int gate_splits, int gate_width, int gate_off, int gate_act, void* out,
                                    int n_tokens, int heads, int dv, int dtype, void* stream) {
-    if (!x || x_splits < 0 || !weight || !out || n_tokens < 0 || heads <= 0 || dv <= 0 || gate_splits < 0 || (dtype != 0 && dtype != 1) ||
+    if (!x || x_splits < 0 || !out || n_tokens < 0 || heads <= 0 || dv <= 0 || gate_splits < 0 || (dtype != 0 && dtype != 1) ||
         gate_act < 0 || gate_act > 2 || x_width < heads * dv || (x_is_act && x_splits != 0))
         return EGPT_BAD_ARGUMENT;
     if (gate && (gate_off < 0 || gate_off + heads * dv > gate_width)) return EGPT_BAD_ARGUMENT;

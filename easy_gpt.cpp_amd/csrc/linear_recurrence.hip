@@ -8,7 +8,7 @@
 // egpt_bounded_gate makes decays with a learned lower bound, a = l + (1 - l) sigmoid(z + b), from columns of a product;
 // egpt_decayed_state_scan runs the recurrence; its queries, keys and values may each pass through SiLU on their way in,
 // its keys may be tied to the decays, k = 1 - a (a forget gate that also sets what is written), instead of columns of
-// the product, and its decay may be one constant per head.
+// the product, its decay may be one constant per head, and its queries and keys may be rotated on their way in.
 //
 // The delta rule, S <- diag(g_t) S; u_t = beta_t (v_t - S^T k_t); S <- S + k_t u_t^T; o_t = S^T q_t, mixes the key channels in
 // every token (S^T k), so its scan keeps a head's whole key range in one workgroup: egpt_delta_rule_scan.  Its operands
@@ -84,12 +84,13 @@ constexpr int kScanWaves = 4;       // wavefronts per workgroup, kScanKeys / kSc
 // what bounds a token is what LDS returns for them (every lane gets its copy), which is why a workgroup takes few key
 // channels.  The wavefronts' parts go through LDS and are added in the order of the wavefronts, a batch of kScanTokens
 // tokens at a time; the batch's operands are staged in LDS, the next batch's loads in flight in registers meanwhile.
-template <typename T>
+template <typename T, bool ROTATED>
 __global__ __launch_bounds__(64 * kScanWaves) void decayed_state_scan_kernel(
     ProductView<T> proj, int proj_width, int q_off, int k_off, int v_off, float q_scale, const float* __restrict__ decay,
     float* __restrict__ states, const int32_t* __restrict__ slots, const unsigned char* __restrict__ fresh,
     const int32_t* __restrict__ q_start, const int32_t* __restrict__ q_len, float* __restrict__ out, int n_tokens, int heads,
-    int dk, int dv, int key_splits, int q_silu, int tied_keys, int k_silu, int v_silu, const float* __restrict__ head_decay) {
+    int dk, int dv, int key_splits, int q_silu, int tied_keys, int k_silu, int v_silu, const float* __restrict__ head_decay,
+    const float* __restrict__ cos_sin, int rot_dims, float mag, int interleaved, float k_scale) {
     constexpr int NS = kScanWaves, DKR = kScanKeys / kScanWaves, THREADS = 64 * NS, DKP = kScanKeys;
     constexpr int QKA = kScanTokens * DKP / THREADS;          // values of q (or k, or decays) of a batch per thread
     constexpr int VL = kScanTokens * kScanCols / THREADS;     // values of v, and outputs, of a batch per thread
@@ -118,6 +119,17 @@ __global__ __launch_bounds__(64 * kScanWaves) void decayed_state_scan_kernel(
     }
     const int channels = heads * dk;
     float rq[QKA], rk[QKA], ra[QKA], rv[VL];
+    // the value at place r of a head whose columns begin at `at`, turned with its partner
+    auto turned = [&](size_t row, size_t at, int r) {
+        const float own = proj.at(at + r);
+        if (!ROTATED || r >= rot_dims) return own;
+        const int half = rot_dims / 2;
+        const int i = interleaved ? r / 2 : (r < half ? r : r - half);
+        const bool first = interleaved ? (r & 1) == 0 : r < half;
+        const float other = proj.at(at + (interleaved ? (r ^ 1) : (first ? r + half : r - half)));
+        const float c = cos_sin[row * rot_dims + 2 * i] * mag, s = cos_sin[row * rot_dims + 2 * i + 1] * mag;
+        return first ? __fmaf_rn(own, c, -__fmul_rn(other, s)) : __fmaf_rn(other, s, __fmul_rn(own, c));
+    };
     auto fetch = [&](int base) {
         const int count = min(kScanTokens, n - base);
 #pragma unroll
@@ -127,9 +139,9 @@ __global__ __launch_bounds__(64 * kScanWaves) void decayed_state_scan_kernel(
             rq[u] = rk[u] = ra[u] = 0.f;
             if (tt < count && r < dk) {
                 const size_t row = static_cast<size_t>(t0 + base + tt);
-                rq[u] = proj.at(row * proj_width + q_off + h * dk + r);      // (scaled when it is staged: nothing here waits for a load)
+                rq[u] = turned(row, row * proj_width + q_off + h * dk, r);      // (scaled when it is staged: nothing here waits for a load)
                 ra[u] = head_decay ? head_decay[h] : decay[row * channels + h * dk + r];
-                if (!tied_keys) rk[u] = proj.at(row * proj_width + k_off + h * dk + r);
+                if (!tied_keys) rk[u] = turned(row, row * proj_width + k_off + h * dk, r);
             }
         }
 #pragma unroll
@@ -150,7 +162,7 @@ __global__ __launch_bounds__(64 * kScanWaves) void decayed_state_scan_kernel(
             // (a tied key is 1 - a; a place that holds no token or no channel has a = 0 and would get k = 1, which meets a
             // query of zero and a state row that is never stored)
             q_s[tid + u * THREADS] = (q_silu ? rq[u] / (1.0f + expf(-rq[u])) : rq[u]) * q_scale;
-            k_s[tid + u * THREADS] = tied_keys ? 1.0f - ra[u] : (k_silu ? rk[u] / (1.0f + expf(-rk[u])) : rk[u]);
+            k_s[tid + u * THREADS] = tied_keys ? 1.0f - ra[u] : (k_silu ? rk[u] / (1.0f + expf(-rk[u])) : rk[u]) * k_scale;
             a_s[tid + u * THREADS] = ra[u];
         }
 #pragma unroll
@@ -241,13 +253,15 @@ template <typename T>
 static int launch_scan(const void* proj, int n_splits, int proj_width, int q_off, int k_off, int v_off, float q_scale,
                        const float* decay, float* states, const int32_t* slots, const unsigned char* fresh,
                        const int32_t* q_start, const int32_t* q_len, int n_seqs, int n_tokens, float* out, int heads, int dk,
-                       int dv, int q_silu, int tied_keys, int k_silu, int v_silu, const float* head_decay, hipStream_t s) {
+                       int dv, int q_silu, int tied_keys, int k_silu, int v_silu, const float* head_decay, const float* cos_sin,
+                       int rot_dims, float mag, int interleaved, float k_scale, hipStream_t s) {
     const ProductView<T> view = scan_view<T>(proj, n_splits, static_cast<size_t>(n_tokens) * proj_width);
     const int key_splits = (dk + kScanKeys - 1) / kScanKeys;
     dim3 grid(n_seqs, heads, (dv + kScanCols - 1) / kScanCols * key_splits);
-    decayed_state_scan_kernel<T><<<grid, 64 * kScanWaves, 0, s>>>(view, proj_width, q_off, k_off, v_off, q_scale, decay, states, slots,
-                                                                  fresh, q_start, q_len, out, n_tokens, heads, dk, dv, key_splits,
-                                                                  q_silu, tied_keys, k_silu, v_silu, head_decay);
+    auto kernel = rot_dims > 0 ? decayed_state_scan_kernel<T, true> : decayed_state_scan_kernel<T, false>;
+    kernel<<<grid, 64 * kScanWaves, 0, s>>>(view, proj_width, q_off, k_off, v_off, q_scale, decay, states, slots, fresh, q_start, q_len,
+                                            out, n_tokens, heads, dk, dv, key_splits, q_silu, tied_keys, k_silu, v_silu, head_decay,
+                                            cos_sin, rot_dims, mag, interleaved, k_scale);
     return EGPT_OK;
 }
 
@@ -257,7 +271,10 @@ extern "C" int egpt_decayed_state_scan(const void* proj, int n_splits, int proj_
                                        float q_scale, const float* decay, float* states, const int32_t* slots,
                                        const unsigned char* fresh, const int32_t* q_start, const int32_t* q_len, int n_seqs,
                                        int n_tokens, float* out, int heads, int dk, int dv, int q_silu, int tied_keys,
-                                       int k_silu, int v_silu, const float* head_decay, int dtype, void* stream) {
+                                       int k_silu, int v_silu, const float* head_decay, const float* cos_sin, int rot_dims,
+                                       float mag, int interleaved, float k_scale, int dtype, void* stream) {
+    if (rot_dims < 0 || rot_dims % 2 || rot_dims > dk || (rot_dims > 0 && (!cos_sin || q_silu || k_silu || tied_keys)))
+        return EGPT_BAD_ARGUMENT;
     // head_decay float32 [heads]: one constant decay per head in place of the decays per token and key channel
     if (!proj || (!decay && !head_decay) || (tied_keys && k_silu) || !states || !slots || !q_start || !q_len || !out || n_splits < 0 || n_seqs <= 0 || n_tokens < 0 ||
         heads <= 0 || dk <= 0 || dv <= 0 || q_off < 0 || (!tied_keys && k_off < 0) || v_off < 0 || (dtype != 0 && dtype != 1))
@@ -270,10 +287,12 @@ extern "C" int egpt_decayed_state_scan(const void* proj, int n_splits, int proj_
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (dtype == 0)
         launch_scan<float>(proj, n_splits, proj_width, q_off, k_off, v_off, q_scale, decay, states, slots, fresh, q_start,
-                           q_len, n_seqs, n_tokens, out, heads, dk, dv, q_silu, tied_keys, k_silu, v_silu, head_decay, s);
+                           q_len, n_seqs, n_tokens, out, heads, dk, dv, q_silu, tied_keys, k_silu, v_silu, head_decay, cos_sin, rot_dims,
+                           mag, interleaved, k_scale, s);
     else
         launch_scan<bf16_t>(proj, n_splits, proj_width, q_off, k_off, v_off, q_scale, decay, states, slots, fresh, q_start,
-                            q_len, n_seqs, n_tokens, out, heads, dk, dv, q_silu, tied_keys, k_silu, v_silu, head_decay, s);
+                            q_len, n_seqs, n_tokens, out, heads, dk, dv, q_silu, tied_keys, k_silu, v_silu, head_decay, cos_sin, rot_dims,
+                           mag, interleaved, k_scale, s);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }

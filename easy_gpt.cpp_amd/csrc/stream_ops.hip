@@ -1,6 +1,7 @@
 // Operations on the residual stream and on logits for designs that do not norm by the root mean square alone:
 // an embedding gather with a constant factor, the layer norm with weight and bias fused with the addition into the
-// stream, the mean of two RMS-normed branch outputs, and the tanh cap on logits.  Statistics and sums are float32;
+// stream, the mean of two RMS-normed branch outputs, parallel residual streams that a sublayer reads as a weighted sum and
+// rewrites as a mixture, and the tanh cap on logits.  Statistics and sums are float32;
 // values are rounded once, when they are written in the activation type.
 #include "api.h"
 #include "common.h"
@@ -174,6 +175,157 @@ __global__ __launch_bounds__(256) void post_norm_add_kernel(const float* h, Prod
         out[base + j] = from_float<T>((row_s[j] - mean) * inv * to_float(next_w[j]));
 }
 
+// VEC neighbouring values of a product (idx a multiple of VEC, rows a multiple of VEC wide)
+template <int VEC, typename T>
+__device__ __forceinline__ void product_values(const ProductView<T>& p, size_t idx, float* v) {
+    if constexpr (VEC == 1) {
+        v[0] = p.at(idx);
+    } else {
+        static_assert(VEC == 4, "four values or one");
+        if (p.n_splits == 0) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) v[i] = to_float(p.whole[idx + i]);
+            return;
+        }
+        float4 sum = *reinterpret_cast<const float4*>(p.partial + idx);
+        for (int s0 = 1; s0 < p.n_splits; s0 += 8) {              // up to eight loads in flight; added in the order of the splits
+            float4 t[8];
+#pragma unroll
+            for (int i = 0; i < 8; ++i)
+                t[i] = s0 + i < p.n_splits ? *reinterpret_cast<const float4*>(p.partial + (s0 + i) * p.split_stride + idx)
+                                           : float4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int i = 0; i < 8; ++i) sum.x += t[i].x, sum.y += t[i].y, sum.z += t[i].z, sum.w += t[i].w;
+        }
+        v[0] = sum.x, v[1] = sum.y, v[2] = sum.z, v[3] = sum.w;
+    }
+}
+
+template <int VEC>
+__device__ __forceinline__ void load_floats(const float* p, float* v) {
+    if constexpr (VEC == 1) {
+        v[0] = *p;
+    } else {
+        const float4 a = *reinterpret_cast<const float4*>(p);
+        v[0] = a.x, v[1] = a.y, v[2] = a.z, v[3] = a.w;
+    }
+}
+
+constexpr int kMostStreams = 8;       // streams whose values of one place a thread holds together; more are read again
+
+// n residual streams x [n][rows][hidden] (stream_stride values apart; 0: all n are the same one).  With a pending output y (a
+// product) they first become x'_t = sum_s mix[s][t] x_s + out_w[t] * scale * y (scale [hidden], null: 1), written to x_out
+// (null: not kept); then u = sum_s in_w[s] x'_s (in_w null: the plain sum) and out = u / sqrt(mean(u^2) + eps) * norm_w.  With
+// rows only those rows are read (and nothing is kept).  One workgroup per row; S: the number of streams, 0: any number
+// (x_out then must not be x).
+template <typename T, int S, int VEC>
+__global__ __launch_bounds__(1024) void connect_streams_kernel(const float* x, size_t stream_stride, int n_streams, ProductView<T> y,
+                                                               const float* __restrict__ scale, const float* __restrict__ mix,
+                                                               const float* __restrict__ out_w, const float* __restrict__ in_w,
+                                                               float* x_out, size_t out_stride, const int32_t* __restrict__ rows,
+                                                               const T* __restrict__ norm_w, float eps, T* __restrict__ out,
+                                                               int hidden) {
+    extern __shared__ __attribute__((aligned(16))) float row_s[];
+    __shared__ float scratch[16];
+    const size_t src = rows ? static_cast<size_t>(rows[blockIdx.x]) : static_cast<size_t>(blockIdx.x);
+    const size_t base = src * hidden;
+    const bool update = y.present();
+    const int n = S > 0 ? S : n_streams;
+    float ss = 0.f;
+    for (int j = threadIdx.x * VEC; j < hidden; j += blockDim.x * VEC) {
+        float u[VEC], yv[VEC];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) u[e] = 0.f;
+        if constexpr (S > 0) {
+            float xv[S][VEC];
+#pragma unroll
+            for (int s = 0; s < S; ++s) load_floats<VEC>(x + s * stream_stride + base + j, xv[s]);
+            if (update) {
+                product_values<VEC>(y, base + j, yv);
+                if (scale) {
+                    float sv[VEC];
+                    load_floats<VEC>(scale + j, sv);
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) yv[e] *= sv[e];
+                }
+                float nv[S][VEC];
+#pragma unroll
+                for (int t = 0; t < S; ++t) {
+                    const float ow = out_w[t];
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) nv[t][e] = ow * yv[e];
+#pragma unroll
+                    for (int s = 0; s < S; ++s) {
+                        const float m = mix[s * S + t];
+#pragma unroll
+                        for (int e = 0; e < VEC; ++e) nv[t][e] = fmaf(m, xv[s][e], nv[t][e]);
+                    }
+                }
+#pragma unroll
+                for (int t = 0; t < S; ++t) {
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) xv[t][e] = nv[t][e];
+                    if (x_out != nullptr) {
+                        float* dst = x_out + t * out_stride + base + j;
+                        if constexpr (VEC == 4) *reinterpret_cast<float4*>(dst) = float4{nv[t][0], nv[t][1], nv[t][2], nv[t][3]};
+                        else *dst = nv[t][0];
+                    }
+                }
+            }
+#pragma unroll
+            for (int s = 0; s < S; ++s) {
+                const float w = in_w ? in_w[s] : 1.0f;
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) u[e] = fmaf(w, xv[s][e], u[e]);
+            }
+        } else {
+            if (update) {
+                product_values<VEC>(y, base + j, yv);
+                if (scale) {
+#pragma unroll
+                    for (int e = 0; e < VEC; ++e) yv[e] *= scale[j + e];
+                }
+            }
+            for (int t = 0; t < n; ++t) {
+                const float w = in_w ? in_w[t] : 1.0f;
+#pragma unroll
+                for (int e = 0; e < VEC; ++e) {
+                    float v;
+                    if (update) {
+                        v = out_w[t] * yv[e];
+                        for (int s = 0; s < n; ++s) v = fmaf(mix[s * n + t], x[s * stream_stride + base + j + e], v);
+                        if (x_out != nullptr) x_out[t * out_stride + base + j + e] = v;
+                    } else {
+                        v = x[t * stream_stride + base + j + e];
+                    }
+                    u[e] = fmaf(w, v, u[e]);
+                }
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+            row_s[j + e] = u[e];
+            ss = fmaf(u[e], u[e], ss);
+        }
+    }
+    const float inv = inv_rms(block_sum(ss, scratch), 1.0f / static_cast<float>(hidden), eps);
+    T* orow = out + static_cast<size_t>(blockIdx.x) * hidden;
+    for (int j = threadIdx.x * VEC; j < hidden; j += blockDim.x * VEC) {      // (a thread reads back its own values)
+        float v[VEC];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) v[e] = row_s[j + e] * inv * to_float(norm_w[j + e]);
+        if constexpr (VEC == 4 && sizeof(T) == 2) {
+            uint2 packed;
+            packed.x = f32_to_bf16_bits(v[0]) | (static_cast<uint32_t>(f32_to_bf16_bits(v[1])) << 16);
+            packed.y = f32_to_bf16_bits(v[2]) | (static_cast<uint32_t>(f32_to_bf16_bits(v[3])) << 16);
+            *reinterpret_cast<uint2*>(orow + j) = packed;
+        } else {
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) orow[j + e] = from_float<T>(v[e]);
+        }
+    }
+}
+
 // x <- x * scale, then (cap > 0) x <- cap * tanh(x / cap)
 __global__ __launch_bounds__(256) void tanh_cap_kernel(float* __restrict__ x, float scale, float cap, size_t n) {
     const float inv = cap > 0.f ? 1.0f / cap : 0.f;
@@ -283,6 +435,56 @@ extern "C" int egpt_post_norm_add(const float* h, const void* y, int y_splits, c
                                                               stream_view<bf16_t>(y2, y2 ? y2_splits : 0, stride), fy, fy2,
                                                               static_cast<const bf16_t*>(post_w), eps, mult, hist, n_hist, stride, mix,
                                                               h_out, static_cast<const bf16_t*>(next_w), static_cast<bf16_t*>(out), hidden);
+    EGPT_CHECK_LAUNCH();
+    return EGPT_OK;
+}
+
+template <typename T, int VEC>
+static void launch_connect(const float* x, size_t stream_stride, int n_streams, const ProductView<T>& y, const float* scale,
+                           const float* mix, const float* out_w, const float* in_w, float* x_out, size_t out_stride,
+                           const int32_t* rows, const T* norm_w, float eps, T* out, int n_rows, int hidden, hipStream_t s) {
+    // few rows: a row's places all at once; many rows fill the GPU with narrower workgroups
+    const int most = n_rows <= 512 ? 1024 : 256;
+    int threads = ((hidden + VEC - 1) / VEC + kWave - 1) / kWave * kWave;
+    threads = threads > most ? most : threads;
+    const size_t lds = static_cast<size_t>(hidden) * sizeof(float);
+#define EGPT_CONNECT(S)                                                                                                        \
+    case S:                                                                                                                    \
+        connect_streams_kernel<T, S, VEC><<<n_rows, threads, lds, s>>>(x, stream_stride, n_streams, y, scale, mix, out_w, in_w, \
+                                                                       x_out, out_stride, rows, norm_w, eps, out, hidden);     \
+        break;
+    switch (n_streams <= kMostStreams ? n_streams : 0) {
+        EGPT_CONNECT(0) EGPT_CONNECT(1) EGPT_CONNECT(2) EGPT_CONNECT(3) EGPT_CONNECT(4) EGPT_CONNECT(5) EGPT_CONNECT(6)
+        EGPT_CONNECT(7) EGPT_CONNECT(8)
+    }
+#undef EGPT_CONNECT
+}
+
+extern "C" int egpt_connect_streams(const float* x, long long stream_stride, int n_streams, const void* y, int y_splits, int y_rows,
+                                    const float* scale, const float* mix, const float* out_w, const float* in_w, float* x_out,
+                                    long long out_stride, const int32_t* rows, const void* norm_w, float eps, void* out,
+                                    int n_rows, int hidden, int dtype, void* stream) {
+    if (!x || stream_stride < 0 || n_streams <= 0 || !norm_w || !out || n_rows < 0 || hidden <= 0 || y_splits < 0 || out_stride < 0 ||
+        (dtype != 0 && dtype != 1) || (y && (!mix || !out_w || y_rows <= 0)) || (!y && x_out) || (rows && x_out))
+        return EGPT_BAD_ARGUMENT;
+    if (x_out == x && (stream_stride != out_stride || n_streams > kMostStreams)) return EGPT_BAD_ARGUMENT;
+    if (hidden > 16384) return EGPT_UNSUPPORTED_SIZE;          // a row lies in LDS
+    if (n_rows == 0) return EGPT_OK;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    const size_t stride = static_cast<size_t>(y_rows) * hidden;
+    const bool fours = hidden % 4 == 0;
+#define EGPT_CONNECT_T(T_, VEC_)                                                                                              \
+    launch_connect<T_, VEC_>(x, static_cast<size_t>(stream_stride), n_streams, stream_view<T_>(y, y ? y_splits : 0, stride), scale, \
+                             mix, out_w, in_w, x_out, static_cast<size_t>(out_stride), rows, static_cast<const T_*>(norm_w), eps, \
+                             static_cast<T_*>(out), n_rows, hidden, s)
+    if (dtype == 0) {
+        if (fours) EGPT_CONNECT_T(float, 4);
+        else EGPT_CONNECT_T(float, 1);
+    } else {
+        if (fours) EGPT_CONNECT_T(bf16_t, 4);
+        else EGPT_CONNECT_T(bf16_t, 1);
+    }
+#undef EGPT_CONNECT_T
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }

@@ -28,7 +28,8 @@ Methods of a backend (T tokens, B requests, R rows, act = bfloat16 or float32):
         j <= p (and j > p - window if window > 0) of that request through its block table
         (hints: singles=False says that no request brings exactly one token; combine=False lets the
         caller combine the parts of a split key range, which are then returned)
-  swiglu(gate_up act[T,2I], out act[T,I])        out = silu(gate_up[:, :I]) * gate_up[:, I:]
+  swiglu(gate_up act[T,2I], out act[T,I], activation='silu')   out = f(gate_up[:, :I]) * gate_up[:, I:], f silu or 'gelu_tanh', the
+        tanh form of gelu (product_swiglu and gate_up_swiglu take the same)
   argmax(logits f32[R,V], out i32[R])            lowest index among equal maxima
   sample(logits f32[R,V], temperature f32[R], top_k i32[R], top_p f32[R], uniform f32[R], out i32[R])
 
@@ -60,6 +61,17 @@ Methods of a backend (T tokens, B requests, R rows, act = bfloat16 or float32):
         dist_bias[head, min(p - j, far)] added to its scaled score (a learned bias by head and distance, tabulated per
         distance up to the one from which it no longer changes)
 
+  window_attention(..., softcap, head_gate f32[T,nq]|None): with a cap c the scaled score s becomes c * tanh(s / c) (the sink is
+        not capped); with a head gate a head's output is multiplied by its number
+  (head_norm_store also takes values_out f32[T,nkv*dv], mix_with f32[T,nkv*dv] and mix: the value heads as they are, and what
+   is stored is (1 - mix) * value + mix * mix_with; gates_out f32[T,n] and gate_offset: the sigmoids of n further columns)
+  connect_streams(streams f32[T,H] | f32[n,T,H], update StreamUpdate|None, read f32[n]|None, n_streams, rows i32[R]|None, weight act[H],
+                  eps, keep=True) -> (act[T|R,H], f32 streams)
+        n residual streams ([T,H]: all n are that one).  With an update they first become
+        x'_t = sum_s mix[s,t] x_s + write[t] * scale * y; the first result is rmsnorm(sum_s read[s] x'_s) * weight (read None: the
+        plain sum), the second the streams as they are now (in place where that is possible; with rows, or keep False, the
+        ones given: nothing is kept)
+
   embed_scaled(token_ids i32[T], table act[V,H], factor, out f32[T,H])          out = table[id] * factor
   add_layernorm(h f32[T,H], delta act[T,H]|f32[S,T,H]|None, rows i32[R]|None, weight act[H], bias act[H]|None, eps, out)
         h += delta; out = (h - mean) / sqrt(mean((h - mean)^2) + eps) * weight + bias; with rows only those, h untouched
@@ -86,7 +98,8 @@ Methods of a backend (T tokens, B requests, R rows, act = bfloat16 or float32):
    norm_after_rotation, values_are_keys; latent_prep takes queries (the query heads as a product of their own) and lead_width;
    head_norm_gate takes gate_act 'silu' | 'sigmoid' | 'factor', x_width and x_act; normed_pair_mean without weights is
    factor * a + factor_b * b; channel_decay takes rates f32[C] and negate: sigmoid(-z)^rates = exp(-rates * softplus(z));
-   decayed_state_scan takes k_silu, v_silu and head_decay f32[heads] in place of decay)
+   decayed_state_scan takes k_silu, v_silu, head_decay f32[heads] in place of decay, a rotation of queries and keys (cos_sin,
+   rotary_dim, pairing, magnitude) and k_scale; head_norm_gate's weight may be None)
   short_conv(proj, act_dtype, col0, conv_w act[C,taps], taps, unit_heads, unit_dim, scaled_heads, scale, unit_eps, sig_offset,
              n_sig, states f32[slots,N], state_offset, slots i32[B], fresh bool[B]|None, q_start, q_len, max_q_len) -> f32[T,C+n_sig]
         columns col0.. of the product rows through C causal convolutions over time (the last tap is the current token's; the
@@ -121,6 +134,17 @@ class ProductSum:
 
     def __init__(self, a, factor_a, b, factor_b):
         self.a, self.factor_a, self.b, self.factor_b = a, float(factor_a), b, float(factor_b)
+
+
+class StreamUpdate:
+    """What a sublayer of parallel residual streams leaves for the next kernel to write: x'_t = sum_s mix[s, t] x_s + write[t] *
+    scale * y, with y a product (act [T, H] or float32 partial sums [S, T, H]), scale float32 [H] or None, mix float32 [n, n],
+    write float32 [n]."""
+
+    __slots__ = ("y", "scale", "mix", "write")
+
+    def __init__(self, y, scale, mix, write):
+        self.y, self.scale, self.mix, self.write = y, scale, mix, write
 
 
 class KernelBackend:
@@ -179,7 +203,7 @@ class KernelBackend:
         of squares [S2, T], h + delta as a new tensor), or None."""
         return None
 
-    def product_swiglu(self, gate_up, row_ss, hidden, eps, w, residual=None):
+    def product_swiglu(self, gate_up, row_ss, hidden, eps, w, residual=None, activation="silu"):
         """swiglu(scale * sum of the partial sums gate_up) w^T as float32 partial sums (or added into `residual`,
         which is then returned), or None."""
         return None
@@ -189,8 +213,14 @@ class KernelBackend:
         then returned), or None."""
         return None
 
-    def gate_up_swiglu(self, x, w):
+    def gate_up_swiglu(self, x, w, activation="silu"):
         """silu(x Wgate^T) * (x Wup^T) as act [T, I] in one kernel, or None."""
+        return None
+
+    def constant_decay_heads(self, *args, **kwargs):
+        """act [T, heads * dv]: a linear attention with one constant decay per head from the input product to the gated heads,
+        in place of decayed_state_scan and head_norm_gate (operands: `kernels.hip.HipKernels.constant_decay_heads`); None if
+        not covered (nothing was done)."""
         return None
 
     def attention_decode_fused(self, *args, **kwargs):

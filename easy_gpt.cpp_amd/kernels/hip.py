@@ -10,10 +10,11 @@ import ctypes
 
 import torch
 
-from . import KernelBackend, KernelsUnavailable, ProductSum
+from . import KernelBackend, KernelsUnavailable, ProductSum, StreamUpdate
 
 _F32, _BF16, _I32, _I64 = torch.float32, torch.bfloat16, torch.int32, torch.int64
 _DT = {_F32: 0, _BF16: 1}
+_GATES = {"silu": 0, "gelu_tanh": 1}          # activations of a gated feed-forward's gate (gate_activation in common.h)
 
 
 def _load_library() -> ctypes.CDLL:
@@ -28,7 +29,7 @@ def _load_library() -> ctypes.CDLL:
         lib = ctypes.CDLL(path)
     except (build.BuildError, OSError) as e:
         raise KernelsUnavailable(f"the HIP kernel library could not be built or loaded: {e}") from e
-    if lib.egpt_abi_version() != 24:
+    if lib.egpt_abi_version() != 25:
         raise KernelsUnavailable(f"{path} has an unexpected ABI version")
     return lib
 
@@ -78,11 +79,11 @@ class HipKernels(KernelBackend):
         sigs = {
             "egpt_embed": [vp, vp, vp, i, i, i, i, i, vp],
             "egpt_add_rmsnorm": [vp, i, vp, i, i, vp, vp, f, vp, i, i, i, vp],
-            "egpt_swiglu": [vp, i, vp, i, i, f, vp, i, i, i, vp],
+            "egpt_swiglu": [vp, i, vp, i, i, f, vp, i, i, i, i, vp],
             "egpt_qkv_rope_store": [vp, i, vp, i, i, f, vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, vp],
             "egpt_rope_table": [vp, vp, vp, i, i, vp],
             "egpt_gemm_skinny_norm": [vp, i, vp, vp, i, vp, vp, vp, vp, i, i, i, i, i, vp],
-            "egpt_gemm_skinny_swiglu": [vp, i, vp, i, i, f, vp, vp, vp, i, i, i, i, i, vp],
+            "egpt_gemm_skinny_swiglu": [vp, i, vp, i, i, f, vp, vp, vp, i, i, i, i, i, i, vp],
             "egpt_gemm_skinny_attn": [vp, vp, i, i, i, vp, vp, vp, i, i, i, i, vp],
             "egpt_attention_combine": [vp, vp, vp, i, i, i, vp],
             "egpt_paged_attention_tiled": [vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, f, i, i, i, vp, vp, i, i,
@@ -100,14 +101,15 @@ class HipKernels(KernelBackend):
             "egpt_argmax": [vp, vp, vp, i, i, vp],
             "egpt_sample": [vp, vp, vp, vp, vp, vp, vp, i, i, vp],
             "egpt_sample_wide": [vp, vp, vp, vp, vp, vp, vp, i, i, vp],
-            "egpt_gemm_gate_up_swiglu": [vp, vp, vp, i, i, i, i, vp],
+            "egpt_gemm_gate_up_swiglu": [vp, vp, vp, i, i, i, i, i, vp],
             "egpt_embed_rmsnorm": [vp, vp, vp, f, vp, i, i, i, i, i, vp],
-            "egpt_head_norm_store": [vp, i, vp, i, i, f, i, vp, vp, vp, f, i, vp, i, f, vp, vp, vp, i, i, i, i, i, i, i, vp],
+            "egpt_head_norm_store": [vp, i, vp, i, i, f, i, vp, vp, vp, f, i, vp, i, f, vp, vp, vp, i, i, i, i, i, i, vp, vp, f, i, i, vp, i,
+                                     vp],
             "egpt_latent_prep": [vp, i, vp, i, i, f, i, vp, i, i, vp, vp, vp, f, vp, f, i, vp, vp, vp, i, i, i, i, i, i, i, vp],
             "egpt_sigmoid_gate": [vp, i, vp, i, vp, i, i, f, i, i, vp, i, i, i, vp],
-            "egpt_window_attention": [vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, vp, vp, i, i, vp, i, vp],
+            "egpt_window_attention": [vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, vp, vp, i, i, vp, f, vp, i, vp],
             "egpt_window_attention_tiled": [vp, vp, vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, vp, vp, i,
-                                            i, vp, i, i, i, vp],
+                                            i, vp, f, vp, i, i, i, vp],
             "egpt_embed_positions": [vp, vp, vp, vp, vp, i, i, i, i, i, vp],
             "egpt_post_norm_add": [vp, vp, i, vp, i, f, f, vp, f, f, vp, i, vp, vp, vp, vp, i, i, i, vp],
             "egpt_bounded_gate": [vp, i, i, i, vp, vp, vp, i, i, i, vp],
@@ -120,7 +122,9 @@ class HipKernels(KernelBackend):
             "egpt_whole_norm_store": [vp, i, i, vp, vp, vp, vp, f, vp, f, i, vp, vp, vp, i, i, i, i, i, i, i, vp],
             "egpt_head_norm_gate": [vp, i, i, i, vp, f, vp, i, i, i, i, vp, i, i, i, i, vp],
             "egpt_channel_decay": [vp, i, i, i, i, vp, vp, f, vp, i, vp, i, i, i, vp],
-            "egpt_decayed_state_scan": [vp, i, i, i, i, i, f, vp, vp, vp, vp, vp, vp, i, i, vp, i, i, i, i, i, i, i, vp, i, vp],
+            "egpt_decayed_state_scan": [vp, i, i, i, i, i, f, vp, vp, vp, vp, vp, vp, i, i, vp, i, i, i, i, i, i, i, vp, vp, i, f, i, f, i, vp],
+            "egpt_constant_decay": [vp, i, i, i, i, i, i, f, vp, i, i, f, vp, vp, vp, vp, vp, vp, i, i, vp, i, vp, f, i, vp, i, i, i, i, vp],
+            "egpt_connect_streams": [vp, ctypes.c_longlong, i, vp, i, i, vp, vp, vp, vp, vp, ctypes.c_longlong, vp, vp, f, vp, i, i, i, vp],
             "egpt_short_conv": [vp, i, i, i, vp, i, i, i, i, i, f, f, i, i, vp, ctypes.c_longlong, vp, vp, vp, vp, i, i, i, vp, i, vp],
             "egpt_delta_rule_scan": [vp, i, i, i, i, i, vp, vp, ctypes.c_longlong, vp, vp, vp, vp, i, i, vp, i, i, i, i, vp],
             "egpt_moe_route": [vp, vp, vp, vp, vp, i, i, i, i, i, vp, f, i, vp],
@@ -131,6 +135,8 @@ class HipKernels(KernelBackend):
         }
         lib.egpt_scan_key_splits.restype = i
         lib.egpt_scan_key_splits.argtypes = [i]
+        lib.egpt_decay_chunk.restype = i
+        lib.egpt_decay_chunk.argtypes = [i, i]
         lib.egpt_sample_workspace.restype = ctypes.c_size_t
         lib.egpt_sample_workspace.argtypes = [i, i]
         for name, argtypes in sigs.items():
@@ -426,7 +432,7 @@ class HipKernels(KernelBackend):
                   self._stream())
         return out, ss, h_new
 
-    def product_swiglu(self, gate_up, row_ss, hidden, eps, w, max_splits=20, waves=None, residual=None):
+    def product_swiglu(self, gate_up, row_ss, hidden, eps, w, max_splits=20, waves=None, residual=None, activation="silu"):
         """swiglu(scale * sum gate_up) w^T for float32 partial sums gate_up [S, T, 2I]; scale is the rows' 1/rms
         from row_ss [S2, T] (or 1).  Returns float32 partial sums [S3, T, N] or None if not covered; with a residual
         stream in fixed point [T, N] the product is added into it instead and the stream is returned."""
@@ -457,7 +463,7 @@ class HipKernels(KernelBackend):
         target = self._residual_target(residual, t, n, s)
         out = None if target is not None else torch.empty((s, t, n), dtype=_F32, device=w.device)
         self._run("egpt_gemm_skinny_swiglu", gate_up.data_ptr(), int(g_splits), self._ptr(row_ss), ss_splits, int(hidden),
-                  float(eps), w.data_ptr(), self._ptr(out), self._ptr(target), t, n, k, s, waves, self._stream())
+                  float(eps), w.data_ptr(), self._ptr(out), self._ptr(target), t, n, k, s, waves, _GATES[activation], self._stream())
         return out if target is None else target
 
     def product_attention(self, part_o, part_ml, w, max_splits=None, waves=None, residual=None):
@@ -497,7 +503,7 @@ class HipKernels(KernelBackend):
                   w.data_ptr(), self._ptr(out), self._ptr(target), t, n, s, waves, self._stream())
         return out if target is None else target
 
-    def gate_up_swiglu(self, x, w, groups=None):
+    def gate_up_swiglu(self, x, w, groups=None, activation="silu"):
         """silu(x Wgate^T) * (x Wup^T) as act [T, I] for w = [Wgate; Wup] ([2I, k]), in one kernel: for 17 to 64
         rows in bfloat16.  Returns None where another way is faster or the case is not covered."""
         t, k = x.shape
@@ -516,7 +522,7 @@ class HipKernels(KernelBackend):
         self._need(w, "w", _BF16, (2 * inter, k))
         out = torch.empty((t, inter), dtype=_BF16, device=x.device)
         self._run("egpt_gemm_gate_up_swiglu", x.data_ptr(), w.data_ptr(), out.data_ptr(), t, inter, k, groups,
-                  self._stream())
+                  _GATES[activation], self._stream())
         return out
 
     def combine_attention(self, part_o, part_ml, out):
@@ -907,12 +913,15 @@ class HipKernels(KernelBackend):
 
     def head_norm_store(self, proj, q_out, q_weight, k_weight, eps, norm_values, slots, k_cache, v_cache, nq, nkv, dk, dv,
                         page_size, row_ss=None, hidden=0, norm_eps=0.0, row_width=None, cos_sin=None, rotary_dim=0,
-                        pairing="half", magnitude=1.0, norm_plain=False, norm_after_rotation=False, values_are_keys=False):
+                        pairing="half", magnitude=1.0, norm_plain=False, norm_after_rotation=False, values_are_keys=False,
+                        values_out=None, mix_with=None, mix=0.0, gates_out=None, gate_offset=0):
         """row_width: the width of proj's rows when more stands behind the heads; cos_sin float32 [T, rotary_dim / 2, 2]
         with rotary_dim > 0: query and key heads are rotated over their first rotary_dim places (pairing 'half': place i
         with i + rotary_dim / 2; 'interleaved': 2i with 2i + 1), behind the norm or, with norm_after_rotation, before
         it; norm_plain: the heads are divided by their root mean square without a weight; values_are_keys: no value
-        columns, a value head is its key head as projected."""
+        columns, a value head is its key head as projected; values_out float32 [T, nkv * dv] takes the value heads as they are, mix_with
+        (such a tensor of another layer) makes what is stored (1 - mix) * value + mix * mix_with; gates_out float32 [T, n] takes the
+        sigmoids of the n columns from gate_offset on."""
         t = proj.shape[-2]
         dt = self._act(q_out, "q_out")
         used = (nq + nkv) * dk + (0 if values_are_keys else nkv * dv)
@@ -938,11 +947,21 @@ class HipKernels(KernelBackend):
             self._key_value_pages(k_cache, v_cache, q_out.dtype, nkv, page_size, dk, dv)
         flags = ((1 if norm_values else 0) | (2 if norm_plain else 0) | (4 if norm_after_rotation else 0)
                  | (8 if values_are_keys else 0) | (16 if pairing == "interleaved" else 0))
+        for name, v in (("values_out", values_out), ("mix_with", mix_with)):
+            if v is not None:
+                self._need(v, name, _F32, (t, nkv * dv))
+        n_gates = 0
+        if gates_out is not None:
+            n_gates = int(gates_out.shape[-1])
+            self._need(gates_out, "gates_out", _F32, (t, n_gates))
+            if gate_offset < 0 or gate_offset + n_gates > width:
+                raise ValueError(f"gate columns {gate_offset}..{gate_offset + n_gates} lie outside rows of {width} values")
         self._run("egpt_head_norm_store", proj.data_ptr(), splits, *self._row_factor(row_ss, splits, t, hidden, norm_eps),
                   width, q_out.data_ptr(), self._ptr(q_weight), self._ptr(k_weight), float(eps), flags,
                   self._ptr(cos_sin) if rotary_dim else None, int(rotary_dim), float(magnitude), self._ptr(slots),
                   self._ptr(k_cache) if slots is not None else None, self._ptr(v_cache) if slots is not None else None,
-                  t, nq, nkv, dk, dv, page_size, dt, self._stream())
+                  t, nq, nkv, dk, dv, page_size, self._ptr(values_out), self._ptr(mix_with), float(mix), n_gates, int(gate_offset),
+                  self._ptr(gates_out), dt, self._stream())
 
     def latent_prep(self, proj, q_plain, q_full, c_weight, eps, cos_sin, magnitude, rotary_dim, slots, k_cache, v_cache,
                     nq, dim, rot, rank, page_size, row_ss=None, hidden=0, norm_eps=0.0, queries=None, lead_width=None):
@@ -990,7 +1009,8 @@ class HipKernels(KernelBackend):
                   out.data_ptr(), t, n, dt, self._stream())
 
     def window_attention(self, q, out, k_cache, v_cache, block_table, q_start, q_len, kv_len, nq, nkv, dk, dv, page_size,
-                         scale, window, keep_first, sink, max_q_len, max_kv_len, dist_bias=None, block=0, slopes=None):
+                         scale, window, keep_first, sink, max_q_len, max_kv_len, dist_bias=None, block=0, slopes=None, softcap=None,
+                         head_gate=None):
         t = q.shape[0]
         block = int(block or 0)
         if block < 0:
@@ -999,6 +1019,14 @@ class HipKernels(KernelBackend):
             self._need(slopes, "slopes", _F32, (nq,))
             if dist_bias is not None:
                 raise ValueError("the attention kernels take a bias table or slopes, not both")
+        if softcap is not None:
+            if not softcap > 0:
+                raise ValueError(f"a cap on scores ({softcap}) must be positive")
+            if dist_bias is not None or slopes is not None:
+                raise ValueError("the attention kernels take a cap on scores or a bias by distance, not both")
+        if head_gate is not None:
+            self._need(head_gate, "head_gate", _F32, (t, nq))
+        cap = 0.0 if softcap is None else float(softcap)
         b, width = block_table.shape
         dt = self._act(q, "q")
         self._need(q, "q", None, (t, nq * dk))
@@ -1032,14 +1060,14 @@ class HipKernels(KernelBackend):
             self._run("egpt_window_attention_tiled", q.data_ptr(), out.data_ptr(), self._ptr(part_o), self._ptr(part_ml),
                       k_cache.data_ptr(), v_cache.data_ptr(), block_table.data_ptr(), width, q_start.data_ptr(),
                       q_len.data_ptr(), kv_len.data_ptr(), b, t, nq, nkv, dk, dv, page_size, float(scale), int(window),
-                      int(keep_first), self._ptr(sink), self._ptr(dist_bias), dist_far, block, self._ptr(slopes), n_splits,
-                      row_tiles, dt, self._stream())
+                      int(keep_first), self._ptr(sink), self._ptr(dist_bias), dist_far, block, self._ptr(slopes), cap,
+                      self._ptr(head_gate), n_splits, row_tiles, dt, self._stream())
             return
         # sizes that the matrix-core kernel does not take: the general kernel
         self._run("egpt_window_attention", q.data_ptr(), out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                   block_table.data_ptr(), width, q_start.data_ptr(), q_len.data_ptr(), kv_len.data_ptr(), b, t, nq, nkv,
                   dk, dv, page_size, float(scale), int(window), int(keep_first), self._ptr(sink), self._ptr(dist_bias),
-                  dist_far, block, self._ptr(slopes), dt, self._stream())
+                  dist_far, block, self._ptr(slopes), cap, self._ptr(head_gate), dt, self._stream())
 
 
     # ------------------------------------------------------------------ stream operations beyond the RMS norm
@@ -1091,6 +1119,35 @@ class HipKernels(KernelBackend):
                   self._ptr(weight_a), self._ptr(weight_b), float(eps), float(factor),
                   float(factor if factor_b is None else factor_b), out.data_ptr(), t, hidden, dt, self._stream())
         return out
+
+    def connect_streams(self, streams, update, read, n_streams, rows, weight, eps, keep=True):
+        dt = self._act(weight, "weight")
+        hidden = streams.shape[-1]
+        t = streams.shape[-2]
+        self._need(streams, "streams", _F32, (t, hidden) if streams.dim() == 2 else (n_streams, t, hidden))
+        self._need(weight, "weight", None, (hidden,))
+        if read is not None:
+            self._need(read, "read", _F32, (n_streams,))
+        n = t if rows is None else rows.shape[0]
+        if rows is not None:
+            self._need(rows, "rows", _I32, (n,))
+        y, splits, kept, scale, mix, write = None, 0, None, None, None, None
+        if update is not None:
+            y, scale, mix, write = update.y, update.scale, update.mix, update.write
+            splits = self._product(y, "y", weight.dtype, t, hidden)
+            self._need(mix, "mix", _F32, (n_streams, n_streams))
+            self._need(write, "write", _F32, (n_streams,))
+            if scale is not None:
+                self._need(scale, "scale", _F32, (hidden,))
+            if keep and rows is None:
+                # in place, unless the streams are still one tensor or too many for a thread to hold
+                in_place = streams.dim() == 3 and n_streams <= 8
+                kept = streams if in_place else torch.empty((n_streams, t, hidden), dtype=_F32, device=streams.device)
+        out = torch.empty((n, hidden), dtype=weight.dtype, device=streams.device)
+        self._run("egpt_connect_streams", streams.data_ptr(), t * hidden if streams.dim() == 3 else 0, int(n_streams), self._ptr(y),
+                  splits, t, self._ptr(scale), self._ptr(mix), self._ptr(write), self._ptr(read), self._ptr(kept), t * hidden,
+                  self._ptr(rows), weight.data_ptr(), float(eps), out.data_ptr(), n, hidden, dt, self._stream())
+        return out, streams if kept is None else kept
 
     def embed_positions(self, token_ids, positions, table, pos_table, out):
         dt = self._act(table, "table")
@@ -1202,14 +1259,15 @@ class HipKernels(KernelBackend):
         is_act = x.dim() == 2 and x_act is not None and x.dtype != _F32
         x_splits = self._product(x, "x", x.dtype if is_act else _F32, t, xw)
         self._need(out, "out", None, (t, heads * dv))
-        self._need(weight, "weight", out.dtype, (dv,))
+        if weight is not None:
+            self._need(weight, "weight", out.dtype, (dv,))
         width, splits = 0, 0
         if gate is not None:
             width = gate.shape[-1]
             splits = self._product(gate, "gate", out.dtype, t, width)
             if gate_offset < 0 or gate_offset + heads * dv > width:
                 raise ValueError(f"gate columns {gate_offset}..{gate_offset + heads * dv} lie outside rows of {width} values")
-        self._run("egpt_head_norm_gate", x.data_ptr(), x_splits, 1 if is_act else 0, xw, weight.data_ptr(), float(eps),
+        self._run("egpt_head_norm_gate", x.data_ptr(), x_splits, 1 if is_act else 0, xw, self._ptr(weight), float(eps),
                   self._ptr(gate), splits, int(width), int(gate_offset), acts[gate_act], out.data_ptr(), t, heads, dv, dt,
                   self._stream())
 
@@ -1254,9 +1312,11 @@ class HipKernels(KernelBackend):
         return out
 
     def decayed_state_scan(self, proj, act_dtype, q_offset, k_offset, v_offset, q_scale, decay, states, slots, fresh, q_start,
-                           q_len, heads, dk, dv, q_silu=False, tied_keys=False, k_silu=False, v_silu=False, head_decay=None):
+                           q_len, heads, dk, dv, q_silu=False, tied_keys=False, k_silu=False, v_silu=False, head_decay=None, cos_sin=None,
+                           rotary_dim=0, pairing="half", magnitude=1.0, k_scale=1.0):
         """k_silu, v_silu: keys and values pass SiLU on their way in, as queries do with q_silu; head_decay float32 [heads]:
-        one constant decay per head (decay is then None)."""
+        one constant decay per head (decay is then None); cos_sin float32 [T, rotary_dim / 2, 2] with rotary_dim > 0: queries and
+        keys are rotated on their way in (not together with SiLU or tied keys); keys are multiplied by k_scale."""
         t, width = proj.shape[-2], proj.shape[-1]
         if act_dtype not in _DT:
             raise TypeError("act_dtype must be float32 or bfloat16")
@@ -1283,7 +1343,62 @@ class HipKernels(KernelBackend):
         self._run("egpt_decayed_state_scan", proj.data_ptr(), splits, int(width), int(q_offset), 0 if tied_keys else int(k_offset), int(v_offset),
                   float(q_scale), self._ptr(decay), states.data_ptr(), slots.data_ptr(), self._ptr(fresh), q_start.data_ptr(),
                   q_len.data_ptr(), b, t, out.data_ptr(), heads, dk, dv, int(bool(q_silu)), int(bool(tied_keys)),
-                  int(bool(k_silu)), int(bool(v_silu)), self._ptr(head_decay), _DT[act_dtype], self._stream())
+                  int(bool(k_silu)), int(bool(v_silu)), self._ptr(head_decay),
+                  *self._rotation(cos_sin, rotary_dim, pairing, magnitude, t, dk), float(k_scale), _DT[act_dtype], self._stream())
+        return out
+
+    def _rotation(self, cos_sin, rotary_dim, pairing, magnitude, t: int, dk: int):
+        """(table or None, rotated places, magnitude, interleaved) for kernels that rotate from the step's table."""
+        if pairing not in ("half", "interleaved"):
+            raise ValueError(f"unknown pairing '{pairing}' of the rotation (half, interleaved)")
+        if not rotary_dim:
+            return None, 0, 1.0, 0
+        if rotary_dim % 2 or not 0 < rotary_dim <= dk:
+            raise ValueError(f"rotary_dim {rotary_dim} must be even and at most the key size {dk}")
+        self._need(cos_sin, "cos_sin", _F32, (t, rotary_dim // 2, 2))
+        return cos_sin.data_ptr(), int(rotary_dim), float(magnitude), 1 if pairing == "interleaved" else 0
+
+    decay_step_tokens = 4       # a step's longest portion up to which the constant-decay attention walks its tokens one by one
+
+    def constant_decay_heads(self, proj, act_dtype, q_offset, k_offset, v_offset, gate_offset, k_scale, powers, states, slots,
+                             fresh, q_start, q_len, max_q_len, heads, dk, dv, weight, eps, gate_act="silu", cos_sin=None,
+                             rotary_dim=0, pairing="half", magnitude=1.0):
+        """act [T, heads * dv]: S_t = d_h S_(t-1) + (k_scale k_t) v_t^T, o_t = S_t^T q_t with rotated queries and keys, every head's
+        o divided by its root mean square, times weight (act [dv] or None) and act(gate columns), 'silu' or 'sigmoid'.  powers
+        float32 [heads, 65]: d_h^0 .. d_h^64.  Portions of more than a few tokens in chunks on the matrix cores, few tokens one
+        by one.  None if the sizes are not covered."""
+        chunk = int(self.lib.egpt_decay_chunk(dk, dv))
+        if not chunk or gate_act not in ("silu", "sigmoid"):
+            return None
+        t, width = proj.shape[-2], proj.shape[-1]
+        if act_dtype not in _DT:
+            raise TypeError("act_dtype must be float32 or bfloat16")
+        splits = self._product(proj, "proj", act_dtype, t, width)
+        b = q_start.shape[0]
+        self._need(powers, "powers", _F32, (heads, 65))
+        self._need(states, "states", _F32)
+        if states.dim() != 4 or tuple(states.shape[1:]) != (heads, dk, dv):
+            raise ValueError(f"states must be [slots, {heads}, {dk}, {dv}], got {tuple(states.shape)}")
+        for name, v in (("slots", slots), ("q_start", q_start), ("q_len", q_len)):
+            self._need(v, name, _I32, (b,))
+        if fresh is not None:
+            self._need(fresh, "fresh", torch.bool, (b,))
+        if weight is not None:
+            self._need(weight, "weight", act_dtype, (dv,))
+        for off, n in ((q_offset, heads * dk), (k_offset, heads * dk), (v_offset, heads * dv), (gate_offset, heads * dv)):
+            if off < 0 or off + n > width:
+                raise ValueError(f"columns {off}..{off + n} lie outside rows of {width} values")
+        table, rot, mag, interleaved = self._rotation(cos_sin, rotary_dim, pairing, magnitude, t, dk)
+        n_chunks, scratch = 0, None
+        if max_q_len > self.decay_step_tokens:
+            n_chunks = t // chunk + b                 # at least the number of all requests' chunks
+            scratch = torch.empty((n_chunks, heads, dk, dv), dtype=_F32, device=states.device)
+        out = torch.empty((t, heads * dv), dtype=act_dtype, device=states.device)
+        self._run("egpt_constant_decay", proj.data_ptr(), splits, int(width), int(q_offset), int(k_offset), int(v_offset),
+                  int(gate_offset), float(k_scale), table, rot, interleaved, mag, powers.data_ptr(), states.data_ptr(),
+                  slots.data_ptr(), self._ptr(fresh), q_start.data_ptr(), q_len.data_ptr(), b, t, self._ptr(scratch), n_chunks,
+                  self._ptr(weight), float(eps), 0 if gate_act == "silu" else 1, out.data_ptr(), heads, dk, dv, _DT[act_dtype],
+                  self._stream())
         return out
 
     def _records(self, states, offset: int, floats: int):
@@ -1444,8 +1559,8 @@ class HipKernels(KernelBackend):
             n_splits = max(1, min(chunks, -(-1024 // workgroups), 64))
         return row_tiles, n_splits
 
-    def swiglu(self, gate_up, out, row_ss=None, hidden=0, eps=0.0):
-        """out = up * silu(gate) for gate_up act [T, 2I] or float32 partial sums [S, T, 2I].  row_ss float32
+    def swiglu(self, gate_up, out, row_ss=None, hidden=0, eps=0.0, activation="silu"):
+        """out = up * silu(gate) (or another `activation` of the gate) for gate_up act [T, 2I] or float32 partial sums [S, T, 2I].  row_ss float32
         [S2, T]: the partial sums still lack each row's factor 1/sqrt(sum_s row_ss[s] / hidden + eps)."""
         t, inter = out.shape
         dt = self._act(out, "out")
@@ -1458,7 +1573,7 @@ class HipKernels(KernelBackend):
             ss_splits = int(row_ss.shape[0])
             self._need(row_ss, "row_ss", _F32, (ss_splits, t))
         self._run("egpt_swiglu", gate_up.data_ptr(), splits, self._ptr(row_ss), ss_splits, int(hidden), float(eps),
-                  out.data_ptr(), t, inter, dt, self._stream())
+                  out.data_ptr(), t, inter, _GATES[activation], dt, self._stream())
 
     def argmax(self, logits, out):
         r, v = logits.shape

@@ -277,6 +277,12 @@ class StreamJoin(Part):
     every result of the depth and goes on with a learned weighted sum of them (`parts/depth_average.py`)."""
 
 
+class StreamConnection(Part):
+    """How one branch of a layer is connected to several parallel residual streams (`parts/connected.py`):
+    read(h, delta, norm) -> (the branch's normed input act [T, H], h'): h the streams, delta the update that the branch before
+    left, h' the streams with it; written(y) -> this branch's own update, for whoever comes next."""
+
+
 class Block:
     """Arrangement of one layer's parts around the residual stream.
 
@@ -293,6 +299,7 @@ class Block:
     uses_mixer = True
     uses_feed_forward = True
     takes_stream_join = False            # True: the constructor takes `stream_join=` (a StreamJoin or None)
+    connection_slots: tuple[str, ...] = ()     # branches whose StreamConnection the constructor takes, as `connections={slot: ...}`
 
     def __init__(self, mixer: Mixer | None, feed_forward: FeedForward | None, norms: dict[str, Norm]):
         if set(norms) != set(self.norm_slots):
@@ -320,6 +327,7 @@ BLOCKS: dict[str, Callable[..., Block]] = {}
 EMBEDDINGS: dict[str, Callable[..., Part]] = {}
 OUTPUT_HEADS: dict[str, Callable[..., Part]] = {}
 STREAM_JOINS: dict[str, Callable[..., StreamJoin]] = {}
+STREAM_CONNECTIONS: dict[str, Callable[..., StreamConnection]] = {}
 
 _REGISTRIES = {
     "mixer": MIXERS,
@@ -330,12 +338,13 @@ _REGISTRIES = {
     "embedding": EMBEDDINGS,
     "output_head": OUTPUT_HEADS,
     "stream_join": STREAM_JOINS,
+    "stream_connection": STREAM_CONNECTIONS,
 }
 
 
 def register_part(family: str, kind: str, factory: Callable[..., Any], replace: bool = False) -> None:
     """Add a part under `kind` to one of the families: mixer, feed_forward, norm,
-    position_encoding, block, embedding, output_head, stream_join."""
+    position_encoding, block, embedding, output_head, stream_join, stream_connection."""
     reg = _REGISTRIES[family]
     if kind in reg and not replace:
         raise ValueError(f"{family} '{kind}' is already registered")

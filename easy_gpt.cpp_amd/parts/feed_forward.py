@@ -1,4 +1,4 @@
-"""Dense gated feed-forward (SwiGLU).
+"""Dense gated feed-forward (SwiGLU, or with another activation of the gate).
 
 As the reference computes it (/root/reference/src/models/mlp.cpp:41-49, CUDA form
 /root/reference/src/cuda/ops/mlp.cu:152-162): u = x Wup^T, g = x Wgate^T,
@@ -23,14 +23,16 @@ class SwiGLU(FeedForward):
                  names: tuple[str, str, str] = ("gate_proj.weight", "up_proj.weight", "down_proj.weight"),
                  unrounded: bool = False):
         """names: the tensors of the gate, up and down matrices behind `prefix`.  unrounded: the output is always
-        float32 partial sums (for an arrangement that adds it to another branch's before anything is rounded)."""
-        if activation != "silu":
+        float32 partial sums (for an arrangement that adds it to another branch's before anything is rounded).  activation: of
+        the gate, 'silu' or 'gelu_tanh' (the tanh form of gelu)."""
+        if activation not in ("silu", "gelu_tanh"):
             raise ValueError(f"activation '{activation}' is not supported by the swiglu feed-forward")
         self.prefix = prefix
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
         self.names = tuple(names)
         self.unrounded = bool(unrounded)
+        self.activation = activation
         self.w_gate_up = self.w_down = None
 
     def param_specs(self):
@@ -65,26 +67,26 @@ class SwiGLU(FeedForward):
                 gate_up, row_ss, h_new = fused
                 x.applied(h_new)
                 residual = pending.residual()
-                out = k.product_swiglu(gate_up, row_ss, self.hidden_size, rms[1], self.w_down, residual=residual)
+                out = k.product_swiglu(gate_up, row_ss, self.hidden_size, rms[1], self.w_down, residual=residual, activation=self.activation)
                 if out is not None:
                     return None if out is residual else out
                 # SwiGLU by itself; it applies the rows' pending 1/rms factor
                 act = torch.empty((h_new.shape[0], self.intermediate_size), dtype=self.w_down.dtype, device=h_new.device)
-                k.swiglu(gate_up, act, row_ss=row_ss, hidden=self.hidden_size, eps=rms[1])
+                k.swiglu(gate_up, act, row_ss=row_ss, hidden=self.hidden_size, eps=rms[1], activation=self.activation)
                 return down(act)
             x = x.materialize()
             residual = pending.residual()
         t = x.shape[0]
-        act = k.gate_up_swiglu(x, self.w_gate_up)        # a few dozen tokens: product and activation in one kernel
+        act = k.gate_up_swiglu(x, self.w_gate_up, activation=self.activation)        # a few dozen tokens: product and activation in one kernel
         if act is not None:
             return down(act)
         gate_up = k.product(x, self.w_gate_up)           # act [T, 2I] or float32 partial sums [S, T, 2I]
         if gate_up.dim() == 3:
-            out = k.product_swiglu(gate_up, None, self.hidden_size, 0.0, self.w_down, residual=residual)
+            out = k.product_swiglu(gate_up, None, self.hidden_size, 0.0, self.w_down, residual=residual, activation=self.activation)
             if out is not None:
                 return None if out is residual else out
         act = torch.empty((t, self.intermediate_size), dtype=x.dtype, device=x.device)
-        k.swiglu(gate_up, act)
+        k.swiglu(gate_up, act, activation=self.activation)
         return down(act)
 
 

@@ -1,5 +1,5 @@
 """Attention mixers that treat single heads before the scores: norms per head, a window that keeps the first tokens,
-latent keys and values, a sink in the softmax, an output gate.
+latent keys and values, a sink in the softmax, a tanh cap on the scores, values mixed with an earlier layer's, an output gate.
 
 Both mixers here run the same three steps through the backend: one product for everything that reads the mixer's
 input, a preparation kernel that norms, rotates and stores into the cache pages, and `window_attention`, the
@@ -7,7 +7,10 @@ attention kernel with separate key and value sizes, window, kept first tokens an
 
 `NormedAttention`: grouped-query attention whose queries and keys are RMS-normed per head with a weight that the
 heads share, whose values are divided by their root mean square before they are cached, and whose window keeps the
-request's first tokens visible: position i sees j <= i if i - j < window or j < keep_first.
+request's first tokens visible: position i sees j <= i if i - j < window or j < keep_first.  Each of these is an option;
+others are a rotation, a sink that is learned or constant, a cap on the scores, an output gate per value or per head, and a
+mixture of the layer's values with those that the first layer of the run order that mixes values made of the same tokens
+(`mixes_values`: they stay in the step's shared values, float32, and the mixed ones are cached).
 
 `LatentAttention`: every token leaves one latent vector c (RMS-normed, `latent_dim` wide) and one rotated key part
 that all heads share; a head's unrotated key is W_uk c and its value W_uv c.  Only c and the rotated part are cached.
@@ -23,6 +26,9 @@ import torch
 from .. import kernels
 from .base import CacheNeed, Mixer, PagedTensor, PendingNorm, make_part, register_part
 from .spec import ParamSpec, PartSpec
+
+
+_FIRST_VALUES = "attention.first_values"       # in a step's shared values: what layers that mix values mix in
 
 
 def _window(window) -> int | None:
@@ -77,14 +83,17 @@ class NormedAttention(_TwoPhases):
     def __init__(self, prefix: str, hidden_size: int, n_heads: int, n_kv_heads: int, key_dim: int, value_dim: int,
                  scale: float, eps: float, window: int | None = None, keep_first: int = 0, norm_queries_keys: bool = True,
                  norm_values: bool = False, norm_weighted: bool = True, norm_after_rotation: bool = False,
-                 position: PartSpec | None = None, values_are_keys: bool = False, sink: bool = False, gated: bool = False,
-                 names: dict | None = None):
+                 position: PartSpec | None = None, values_are_keys: bool = False, sink: bool | float = False,
+                 gated: bool | str = False, softcap: float | None = None, mixes_values: bool = False, names: dict | None = None):
         """norm_weighted False: queries and keys are divided by their root mean square and no more (no weight tensors);
         position: a rotary encoding of queries and keys (None: no rotation), applied behind the norm, or before it
         with norm_after_rotation; values_are_keys: there is no value projection, a value head is its key head as
-        projected (before norm and rotation); sink: one number per head joins the softmax's denominator; gated: the
-        heads' outputs are multiplied by sigmoid(W_g x).  names: tensor names behind `prefix` of q, k, v, o, the
-        weights q_norm, k_norm, and sink, gate."""
+        projected (before norm and rotation); sink: one number per head joins the softmax's denominator, learned (True) or the
+        same constant score for every head (a number); gated: the heads' outputs are multiplied by sigmoid(W_g x), one number
+        per value, or with 'heads' one per head; softcap c: a score s becomes c tanh(s / c); mixes_values: the cached values are
+        (1 - lambda) v + lambda v_first with lambda a tensor of one number, v_first the values of the run order's first layer
+        that mixes (whose own lambda is not used).  names: tensor names behind `prefix` of q, k, v, o, the weights q_norm,
+        k_norm, and sink, gate, value_mix."""
         if n_heads % n_kv_heads:
             raise ValueError(f"n_heads ({n_heads}) must be a multiple of n_kv_heads ({n_kv_heads})")
         widest = kernels.KernelBackend.max_window_attention_dim
@@ -102,10 +111,16 @@ class NormedAttention(_TwoPhases):
         self.keep_first = int(keep_first) if self.window else 0
         self.norm_queries_keys, self.norm_values = bool(norm_queries_keys), bool(norm_values)
         self.norm_weighted, self.norm_after_rotation = bool(norm_weighted), bool(norm_after_rotation)
-        self.values_are_keys, self.has_sink, self.gated = bool(values_are_keys), bool(sink), bool(gated)
+        if gated not in (False, True, "heads"):
+            raise ValueError(f"gated ({gated!r}) must be False, True (a gate per value) or 'heads' (a gate per head)")
+        self.values_are_keys, self.has_sink = bool(values_are_keys), sink is True
+        self.constant_sink = None if isinstance(sink, bool) else float(sink)
+        self.gated, self.gate_per_head = gated is True, gated == "heads"
+        self.softcap = None if softcap is None else float(softcap)
+        self.mixes_values, self.mix = bool(mixes_values), 0.0
         self.position = None if position is None else make_part("position_encoding", position, head_dim=self.key_dim)
         self.names = dict(q="q_proj.weight", k="k_proj.weight", v="v_proj.weight", o="o_proj.weight",
-                          q_norm="q_norm.weight", k_norm="k_norm.weight", sink="sink", gate="g_proj.weight")
+                          q_norm="q_norm.weight", k_norm="k_norm.weight", sink="sink", gate="g_proj.weight", value_mix="value_mix")
         self.names.update(names or {})
         self.q_width, self.k_width = self.n_heads * self.key_dim, self.n_kv_heads * self.key_dim
         self.v_width = 0 if self.values_are_keys else self.n_kv_heads * self.value_dim
@@ -126,15 +141,17 @@ class NormedAttention(_TwoPhases):
                       ParamSpec(p + n["k_norm"], (self.key_dim,), role="norm_scale")]
         if self.has_sink:
             specs.append(ParamSpec(p + n["sink"], (self.n_heads,), role="bias", dtype="float32"))
-        if self.gated:
-            specs.append(ParamSpec(p + n["gate"], (self.out_width, h)))
+        if self.gated or self.gate_per_head:
+            specs.append(ParamSpec(p + n["gate"], (self.out_width if self.gated else self.n_heads, h)))
+        if self.mixes_values:
+            specs.append(ParamSpec(p + n["value_mix"], (), role="bias", dtype="float32", alt_shapes=((1,),)))
         if self.position is not None:
             specs += self.position.param_specs()
         return specs
 
     def load(self, get, dtype, device):
         p, n = self.prefix, self.names
-        which = ["q", "k"] + ([] if self.values_are_keys else ["v"]) + (["gate"] if self.gated else [])
+        which = ["q", "k"] + ([] if self.values_are_keys else ["v"]) + (["gate"] if self.gated or self.gate_per_head else [])
         w = torch.cat([get(p + n[x]).to(dtype) for x in which], dim=0)      # one product serves all that reads x
         self.w_qkv = w.to(device).contiguous()
         self.w_o = self._to(get(p + n["o"]), "compute", dtype, device)
@@ -143,6 +160,10 @@ class NormedAttention(_TwoPhases):
             self.k_weight = self._to(get(p + n["k_norm"]), "compute", dtype, device)
         if self.has_sink:
             self.sink = get(p + n["sink"]).to(torch.float32).to(device).contiguous()
+        elif self.constant_sink is not None:
+            self.sink = torch.full((self.n_heads,), self.constant_sink, dtype=torch.float32).to(device)
+        if self.mixes_values:
+            self.mix = float(get(p + n["value_mix"]).to(torch.float32).reshape(()))
         if self.position is not None:
             self.position.load(get, dtype, device)
 
@@ -167,20 +188,36 @@ class NormedAttention(_TwoPhases):
             rotation = dict(cos_sin=self.position.table(ctx), rotary_dim=rotary[1], pairing=self.position.pairing,
                             magnitude=getattr(self.position, "magnitude", 1.0))
         plain = self.norm_queries_keys and not self.norm_weighted
-        if plain or self.norm_after_rotation or self.values_are_keys or self.gated:
+        if plain or self.norm_after_rotation or self.values_are_keys or self.gated or self.gate_per_head:
             rotation.update(norm_plain=plain, norm_after_rotation=self.norm_after_rotation,
                             values_are_keys=self.values_are_keys, row_width=self.w_qkv.shape[0])
+        gate_at = self.q_width + self.k_width + self.v_width
+        head_gate = None
+        if self.gate_per_head:
+            head_gate = torch.empty((t, self.n_heads), dtype=torch.float32, device=p.device)
+            rotation.update(gates_out=head_gate, gate_offset=gate_at)
+        if self.mixes_values:
+            first = ctx.shared.get(_FIRST_VALUES)
+            if first is None:
+                first = torch.empty((t, self.n_kv_heads * self.value_dim), dtype=torch.float32, device=p.device)
+                ctx.shared[_FIRST_VALUES] = first
+                rotation.update(values_out=first)
+            else:
+                rotation.update(mix_with=first, mix=self.mix)
+        scores = {}
+        if self.softcap is not None or head_gate is not None:
+            scores = dict(softcap=self.softcap, head_gate=head_gate)
         k.head_norm_store(p.proj, q, self.q_weight, self.k_weight, self.eps, self.norm_values,
                           cache.slots if cache.writes else None, cache.k, cache.v, self.n_heads, self.n_kv_heads,
                           self.key_dim, self.value_dim, cache.page_size, **p.factor, **rotation)
         attn = torch.empty((t, self.out_width), dtype=p.dtype, device=p.device)
         k.window_attention(q, attn, cache.k, cache.v, cache.block_table, ctx.q_start, ctx.q_len, ctx.kv_len,
                            self.n_heads, self.n_kv_heads, self.key_dim, self.value_dim, cache.page_size, self.scale,
-                           self.window or 0, self.keep_first, self.sink, ctx.max_q_len, ctx.max_kv_len)
+                           self.window or 0, self.keep_first, self.sink, ctx.max_q_len, ctx.max_kv_len, **scores)
         if not self.gated:
             return attn
         gated = torch.empty_like(attn)
-        k.sigmoid_gate(attn, 0, p.proj, self.q_width + self.k_width + self.v_width, gated, **p.factor)
+        k.sigmoid_gate(attn, 0, p.proj, gate_at, gated, **p.factor)
         return gated
 
 

@@ -41,6 +41,12 @@ class Model:
                 if not getattr(BLOCKS[ls.block], "takes_stream_join", False):
                     raise ValueError(f"the block arrangement '{ls.block}' takes no stream join")
                 extra["stream_join"] = make_part("stream_join", ls.stream_join, **ctx)
+            slots = getattr(BLOCKS[ls.block], "connection_slots", ())
+            if set(ls.connections) != set(slots):
+                raise ValueError(f"the block arrangement '{ls.block}' connects the branches {sorted(slots)}, the layer gives "
+                                 f"{sorted(ls.connections)}")
+            if slots:
+                extra["connections"] = {slot: make_part("stream_connection", cs, **ctx) for slot, cs in ls.connections.items()}
             self.layers.append(BLOCKS[ls.block](mixer, ff, norms, **extra))
         self.final_norm = make_part("norm", spec.final_norm, **ctx)
         self.output_head = make_part("output_head", spec.output_head, vocab_size=spec.vocab_size, **ctx)

@@ -17,18 +17,19 @@ from .spec import ParamSpec
 class RMSNorm(Norm):
     graph_safe = True
 
-    def __init__(self, prefix: str, hidden_size: int, eps: float):
+    def __init__(self, prefix: str, hidden_size: int, eps: float, name: str = "weight"):
         self.prefix = prefix
         self.hidden_size = int(hidden_size)
         self.eps = float(eps)
+        self.name = name                   # the weight is the tensor `prefix + name`
         self.weight: torch.Tensor | None = None
 
     def param_specs(self):
         h = self.hidden_size
-        return [ParamSpec(self.prefix + "weight", (h,), role="norm_scale", alt_shapes=((h, 1),))]
+        return [ParamSpec(self.prefix + self.name, (h,), role="norm_scale", alt_shapes=((h, 1),))]
 
     def load(self, get, dtype, device):
-        self.weight = self._to(get(self.prefix + "weight").reshape(self.hidden_size), "compute", dtype, device)
+        self.weight = self._to(get(self.prefix + self.name).reshape(self.hidden_size), "compute", dtype, device)
 
     def rms_params(self):
         return self.weight, self.eps
@@ -50,8 +51,7 @@ class ScalarRMSNorm(RMSNorm):
     weight per coordinate run it, and parts that fold a norm into their first kernel see an ordinary weight."""
 
     def __init__(self, prefix: str, hidden_size: int, eps: float, name: str = "weight"):
-        super().__init__(prefix, hidden_size, eps)
-        self.name = name
+        super().__init__(prefix, hidden_size, eps, name)
 
     def param_specs(self):
         return [ParamSpec(self.prefix + self.name, (), role="norm_scale", alt_shapes=((1,),))]
@@ -59,6 +59,25 @@ class ScalarRMSNorm(RMSNorm):
     def load(self, get, dtype, device):
         gain = get(self.prefix + self.name).reshape(1).to(dtype)
         self.weight = gain.expand(self.hidden_size).to(device).contiguous()
+
+
+class StreamSumRMSNorm(RMSNorm):
+    """The RMS norm of the sum of parallel residual streams: what closes a model whose layers are connected by several of
+    them.  `h` is the streams float32 [n, T, H] (or [T, H] while all n are equal), `delta` the last sublayer's pending
+    `kernels.StreamUpdate`, which is added on the way without being kept."""
+
+    def __init__(self, prefix: str, hidden_size: int, eps: float, streams: int, name: str = "weight"):
+        super().__init__(prefix, hidden_size, eps, name)
+        self.streams = int(streams)
+
+    def rms_params(self):
+        return None                        # (a sum comes before it: no part may fold it as a plain norm)
+
+    def forward(self, h, delta):
+        return kernels.backend().connect_streams(h, delta, None, self.streams, None, self.weight, self.eps, keep=False)[0]
+
+    def forward_rows(self, h, delta, rows):
+        return kernels.backend().connect_streams(h, delta, None, self.streams, rows, self.weight, self.eps)[0]
 
 
 class LayerNorm(Norm):
@@ -102,3 +121,4 @@ class LayerNorm(Norm):
 register_part("norm", "rmsnorm", RMSNorm)
 register_part("norm", "layernorm", LayerNorm)
 register_part("norm", "rmsnorm_scalar", ScalarRMSNorm)
+register_part("norm", "rmsnorm_stream_sum", StreamSumRMSNorm)

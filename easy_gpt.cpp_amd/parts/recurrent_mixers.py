@@ -1,9 +1,10 @@
-"""Mixers with a matrix state per head and request that stand beside an attention in one layer.
+"""Mixers with a matrix state per head and request, alone in a layer or beside an attention.
 
 `ConstantDecayAttention`: linear attention whose state decays by one constant per head,
-S_t = d_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t with q, k, v = silu of their projections and no other scale.  The heads'
-outputs are RMS-normed together (one statistic over all heads, a weight per value), multiplied by sigmoid(W_g x) and
-projected.
+S_t = d_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.  In one form q, k, v are silu of their projections with no other scale, the
+heads' outputs are RMS-normed together (one statistic over all heads, a weight per value) and multiplied by sigmoid(W_g x).
+In the other (retention) queries and keys are rotated by their position, keys have a constant factor, every head's output
+is divided by its own root mean square, without a weight, and multiplied by silu(W_g x).  Both are projected.
 
 `GatedDeltaRule`: queries, keys and values pass a short causal convolution over time per channel (zeros before the
 sequence's start) and silu; queries and keys are made unit vectors per head (x / sqrt(sum x^2 + unit_eps)), queries
@@ -22,9 +23,9 @@ from __future__ import annotations
 import torch
 
 from .. import kernels
-from .base import StateNeed, register_part
+from .base import StateNeed, make_part, register_part
 from .branch_mixers import _Branch
-from .spec import ParamSpec
+from .spec import ParamSpec, PartSpec
 
 
 def _sizes_ok(key_dim: int, value_dim: int) -> None:
@@ -37,8 +38,13 @@ class ConstantDecayAttention(_Branch):
     graph_safe = True
 
     def __init__(self, prefix: str, hidden_size: int, n_heads: int, key_dim: int, value_dim: int, decay, eps: float,
-                 names: dict | None = None):
-        """decay: one number per head.  names: tensor names behind `prefix` of q, k, v, g, norm, o."""
+                 activated: bool = True, position: PartSpec | None = None, key_scale: float = 1.0, norm_heads: bool = False,
+                 norm_weighted: bool = True, gate_act: str = "sigmoid", names: dict | None = None):
+        """decay: one number per head; activated: queries, keys and values pass silu; position: a rotary encoding of queries
+        and keys (None: no rotation; not together with `activated`); key_scale: a factor on the keys; norm_heads: every head
+        is normed by itself (else all together); norm_weighted: the norm has a weight per value ([heads * value size], or
+        [value size] for all heads with norm_heads); gate_act: 'sigmoid' or 'silu'.  names: tensor names behind `prefix` of
+        q, k, v, g, norm, o."""
         _sizes_ok(key_dim, value_dim)
         self.prefix, self.hidden_size = prefix, int(hidden_size)
         self.n_heads, self.key_dim, self.value_dim = int(n_heads), int(key_dim), int(value_dim)
@@ -46,10 +52,18 @@ class ConstantDecayAttention(_Branch):
         if len(self.decay_values) != self.n_heads:
             raise ValueError(f"{len(self.decay_values)} decays for {self.n_heads} heads")
         self.eps = float(eps)
+        if activated and position is not None and position.kind != "none":
+            raise ValueError("queries and keys are rotated as projected or pass silu, not both")
+        if gate_act not in ("sigmoid", "silu"):
+            raise ValueError(f"unknown gate activation '{gate_act}' (sigmoid, silu)")
+        self.activated, self.key_scale, self.gate_act = bool(activated), float(key_scale), gate_act
+        self.norm_heads, self.norm_weighted = bool(norm_heads), bool(norm_weighted)
+        self.position = None if position is None else make_part("position_encoding", position, head_dim=self.key_dim)
         self.names = dict(q="q", k="k", v="v", g="g", norm="norm", o="o")
         self.names.update(names or {})
         self.qk_width, self.v_width = self.n_heads * self.key_dim, self.n_heads * self.value_dim
-        self.w_in = self.w_o = self.norm_weight = self.decay = None
+        self.normed_width = self.value_dim if self.norm_heads else self.v_width
+        self.w_in = self.w_o = self.norm_weight = self.decay = self.powers = None
 
     def state_need(self):
         return StateNeed((self.n_heads, self.key_dim, self.value_dim), torch.float32)
@@ -59,29 +73,52 @@ class ConstantDecayAttention(_Branch):
         return [
             ParamSpec(p + n["q"], (self.qk_width, h)), ParamSpec(p + n["k"], (self.qk_width, h)),
             ParamSpec(p + n["v"], (self.v_width, h)), ParamSpec(p + n["g"], (self.v_width, h)),
-            ParamSpec(p + n["norm"], (self.v_width,), role="norm_scale"),
+            *([ParamSpec(p + n["norm"], (self.normed_width,), role="norm_scale")] if self.norm_weighted else []),
             ParamSpec(p + n["o"], (h, self.v_width)),
+            *(self.position.param_specs() if self.position is not None else []),
         ]
 
     def load(self, get, dtype, device):
         p, n = self.prefix, self.names
         w = torch.cat([get(p + n[x]).to(dtype) for x in ("q", "k", "v", "g")], dim=0)       # one product reads x
         self.w_in = w.to(device).contiguous()
-        self.norm_weight = self._to(get(p + n["norm"]), "compute", dtype, device)
+        if self.norm_weighted:
+            self.norm_weight = self._to(get(p + n["norm"]), "compute", dtype, device)
         self.w_o = self._to(get(p + n["o"]), "compute", dtype, device)
         self.decay = torch.tensor(self.decay_values, dtype=torch.float32).to(device)
+        # d^0 .. d^64 of every head, each power rounded once
+        base = self.decay.to("cpu", torch.float64)[:, None]
+        self.powers = torch.pow(base, torch.arange(65, dtype=torch.float64)[None, :]).to(torch.float32).to(device).contiguous()
+        if self.position is not None:
+            self.position.load(get, dtype, device)
 
     def branch(self, x, ctx, cache, state):
         k = kernels.backend()
         t = x.shape[0]
         qk, vw = self.qk_width, self.v_width
         proj = k.product(x, self.w_in, unrounded=True)                 # [q | k | v | g]
-        o = k.decayed_state_scan(proj, x.dtype, 0, qk, 2 * qk, 1.0, None, state.data, state.slots, state.fresh_device,
-                                 ctx.q_start, ctx.q_len, self.n_heads, self.key_dim, self.value_dim, q_silu=True,
-                                 k_silu=True, v_silu=True, head_decay=self.decay)
-        gated = torch.empty((t, vw), dtype=x.dtype, device=x.device)
-        # all heads are normed together: one "head" as wide as all of them
-        k.head_norm_gate(o, self.norm_weight, self.eps, proj, 2 * qk + vw, gated, 1, vw, gate_act="sigmoid")
+        rotation = {}
+        rotary = self.position.rotary(x.device) if self.position is not None else None
+        if rotary is not None:
+            rotation = dict(cos_sin=self.position.table(ctx), rotary_dim=rotary[1], pairing=self.position.pairing,
+                            magnitude=getattr(self.position, "magnitude", 1.0))
+        gated = None
+        if self.norm_heads and not self.activated:
+            gated = k.constant_decay_heads(proj, x.dtype, 0, qk, 2 * qk, 2 * qk + vw, self.key_scale, self.powers, state.data,
+                                           state.slots, state.fresh_device, ctx.q_start, ctx.q_len, ctx.max_q_len, self.n_heads,
+                                           self.key_dim, self.value_dim, self.norm_weight, self.eps, gate_act=self.gate_act,
+                                           **rotation)
+        if gated is None:
+            silu = dict(q_silu=True, k_silu=True, v_silu=True) if self.activated else {}
+            if self.key_scale != 1.0:
+                silu["k_scale"] = self.key_scale
+            o = k.decayed_state_scan(proj, x.dtype, 0, qk, 2 * qk, 1.0, None, state.data, state.slots, state.fresh_device,
+                                     ctx.q_start, ctx.q_len, self.n_heads, self.key_dim, self.value_dim, head_decay=self.decay,
+                                     **silu, **rotation)
+            gated = torch.empty((t, vw), dtype=x.dtype, device=x.device)
+            # (all heads normed together: one "head" as wide as all of them)
+            heads = self.n_heads if self.norm_heads else 1
+            k.head_norm_gate(o, self.norm_weight, self.eps, proj, 2 * qk + vw, gated, heads, vw // heads, gate_act=self.gate_act)
         return k.product(gated, self.w_o, unrounded=True), None
 
 

@@ -15,7 +15,7 @@ class ParamSpec:
     """One tensor of the weights file.
 
     role    how random weights draw it: 'matrix', 'embedding', 'bias' ~ N(0, 0.02);
-            'norm_scale' ~ 1 + N(0, 0.02); 'mean_weights' ~ (1 + N(0, 0.02)) / n; 'int_table' uniform integers; or any role that was added
+            'norm_scale' ~ 1 + N(0, 0.02); 'mean_weights' ~ (1 + N(0, 0.02)) / n; 'stream_mix' near the identity; 'int_table' uniform integers; or any role that was added
             with `weights.register_role` (a decay in (0, 1), a table of a special form, ...)
     dtype   'compute' (cast to the engine's dtype), 'float32' or 'int32' (kept as stored)
     alt_shapes  other shapes accepted on load (the reference accepts [H, 1] for a
@@ -54,6 +54,8 @@ class LayerSpec:
             to the arrangement's constructor by name
     stream_join   a part of the family 'stream_join' that decides what goes on to the next layer once the layer's own
             result is known (a weighted sum over the results of all layers so far, say); None: the result itself
+    connections   parts of the family 'stream_connection', one per branch of an arrangement that has several residual
+            streams (`Block.connection_slots`): how the branch reads them and how its output is written to them
     """
 
     block: str
@@ -62,6 +64,7 @@ class LayerSpec:
     norms: Mapping[str, PartSpec] = field(default_factory=dict)
     block_params: Mapping[str, Any] = field(default_factory=dict)
     stream_join: PartSpec | None = None
+    connections: Mapping[str, PartSpec] = field(default_factory=dict)
 
 
 @dataclass(frozen=True)

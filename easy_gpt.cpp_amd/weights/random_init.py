@@ -104,6 +104,14 @@ def _mean_weights(shape, g, device):
     return _counter_normal(shape, g.initial_seed(), device, _STD / max(n, 1), 1.0 / max(n, 1))
 
 
+def _stream_mix(shape, g, device):
+    """A mixture [n, n] of n parallel streams near the identity: 0.9 on the diagonal, 0.1 / n everywhere, N(0, 0.02) on top,
+    so that a stream keeps its size and its own content over many layers."""
+    n = int(shape[0])
+    m = _counter_normal(shape, g.initial_seed(), device, _STD, 0.1 / max(n, 1))
+    return m + 0.9 * torch.eye(n, dtype=torch.float32, device=device)
+
+
 def _int_table(shape, g, device):
     n = 1
     for d in shape:
@@ -120,6 +128,7 @@ ROLES: dict[str, Callable[..., torch.Tensor]] = {
     "bias": _normal,
     "norm_scale": _norm_scale,
     "mean_weights": _mean_weights,
+    "stream_mix": _stream_mix,
     "int_table": _int_table,
 }
 

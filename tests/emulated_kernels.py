@@ -138,7 +138,8 @@ class EmulatedKernels(KernelBackend):
 
     def head_norm_store(self, proj, q_out, q_weight, k_weight, eps, norm_values, slots, k_cache, v_cache, nq, nkv, dk, dv,
                         page_size, row_width=None, cos_sin=None, rotary_dim=0, pairing="half", magnitude=1.0, norm_plain=False,
-                        norm_after_rotation=False, values_are_keys=False):
+                        norm_after_rotation=False, values_are_keys=False, values_out=None, mix_with=None, mix=0.0,
+                        gates_out=None, gate_offset=0):
         x = _whole(proj).to(F64)
         t = x.shape[0]
         unit = lambda a: a / torch.sqrt((a * a).mean(-1, keepdim=True) + eps)
@@ -160,6 +161,12 @@ class EmulatedKernels(KernelBackend):
             q, k = turn(q), turn(k)
         if norm_values:
             v = unit(v)
+        if values_out is not None:
+            values_out.copy_(v.reshape(t, nkv * dv).to(values_out.dtype))
+        if mix_with is not None:
+            v = (1.0 - mix) * v + mix * mix_with.to(F64).view(t, nkv, dv)
+        if gates_out is not None:
+            gates_out.copy_(torch.sigmoid(x[:, gate_offset : gate_offset + gates_out.shape[1]]).to(gates_out.dtype))
         q_out.copy_(q.reshape(t, nq * dk).to(q_out.dtype))
         if slots is not None:
             self._store(k_cache, v_cache, slots, page_size, k, v)
@@ -205,7 +212,8 @@ class EmulatedKernels(KernelBackend):
         out.copy_((xx * torch.sigmoid(g)).to(out.dtype))
 
     def window_attention(self, q, out, k_cache, v_cache, block_table, q_start, q_len, kv_len, nq, nkv, dk, dv, page_size,
-                         scale, window, keep_first, sink, max_q_len, max_kv_len, dist_bias=None, block=0, slopes=None):
+                         scale, window, keep_first, sink, max_q_len, max_kv_len, dist_bias=None, block=0, slopes=None,
+                         softcap=None, head_gate=None):
         group = nq // nkv
         q_all = q.view(q.shape[0], nq, dk).to(F64)
         for b in range(q_start.shape[0]):
@@ -224,6 +232,8 @@ class EmulatedKernels(KernelBackend):
                     keys = k_cache[pages, kh, offs, :].to(F64)
                     vals = v_cache[pages, kh, :, offs].to(F64)
                     sc = (keys @ q_all[s + i, h]) * scale
+                    if softcap is not None:
+                        sc = softcap * torch.tanh(sc / softcap)
                     if dist_bias is not None:
                         sc = sc + dist_bias[h, (p - js).clamp(max=dist_bias.shape[1] - 1)].to(F64)
                     if slopes is not None:
@@ -231,7 +241,8 @@ class EmulatedKernels(KernelBackend):
                     m = sc.max() if sink is None else torch.maximum(sc.max(), sink[h].to(F64))
                     e = torch.exp(sc - m)
                     denom = e.sum() + (torch.exp(sink[h].to(F64) - m) if sink is not None else 0.0)
-                    out[s + i, h * dv : (h + 1) * dv] = ((e / denom) @ vals).to(out.dtype)
+                    gate = 1.0 if head_gate is None else head_gate[s + i, h].to(F64)
+                    out[s + i, h * dv : (h + 1) * dv] = ((e / denom) @ vals * gate).to(out.dtype)
 
     # ---- operations of designs with layer norms, side-by-side mixers, a decaying state and experts
     def embed_scaled(self, token_ids, table, factor, out):
@@ -288,7 +299,7 @@ class EmulatedKernels(KernelBackend):
     def head_norm_gate(self, x, weight, eps, gate, gate_offset, out, heads, dv, gate_act="silu", x_width=None, x_act=None):
         t = out.shape[0]
         xx = _whole(x).to(F64)[:, : heads * dv].reshape(t, heads, dv)
-        xx = xx / torch.sqrt((xx * xx).mean(-1, keepdim=True) + eps) * weight.to(F64)
+        xx = xx / torch.sqrt((xx * xx).mean(-1, keepdim=True) + eps) * (1.0 if weight is None else weight.to(F64))
         if gate is None:
             out.copy_(xx.reshape(t, heads * dv).to(out.dtype))
             return
@@ -312,9 +323,13 @@ class EmulatedKernels(KernelBackend):
         return (low + (1.0 - low) * torch.sigmoid(v)).to(torch.float32)
 
     def decayed_state_scan(self, proj, act_dtype, q_offset, k_offset, v_offset, q_scale, decay, states, slots, fresh, q_start,
-                           q_len, heads, dk, dv, q_silu=False, tied_keys=False, k_silu=False, v_silu=False, head_decay=None):
-        x = _whole(proj).to(F64)
+                           q_len, heads, dk, dv, q_silu=False, tied_keys=False, k_silu=False, v_silu=False, head_decay=None, cos_sin=None,
+                           rotary_dim=0, pairing="half", magnitude=1.0, k_scale=1.0):
+        x = _whole(proj).to(F64).clone()
         t = x.shape[0]
+        for off in (q_offset, k_offset) if rotary_dim else ():
+            x[:, off : off + heads * dk] = self._turn(x[:, off : off + heads * dk].view(t, heads, dk), cos_sin, magnitude, rotary_dim,
+                                                      pairing).reshape(t, heads * dk)
         if head_decay is not None:
             decay = head_decay.to(F64)[None, :, None].expand(t, heads, dk).reshape(t, heads * dk)
         out = torch.zeros((t, heads * dv), dtype=torch.float32)
@@ -332,6 +347,7 @@ class EmulatedKernels(KernelBackend):
                     k = k * torch.sigmoid(k)
                 if v_silu:
                     v = v * torch.sigmoid(v)
+                k = k * k_scale
                 st = decay[i].to(F64).view(heads, dk)[:, :, None] * st + k[:, :, None] * v[:, None, :]
                 out[i] = torch.einsum("hkv,hk->hv", st, q).reshape(-1).to(torch.float32)
             states[slot] = st.to(states.dtype)
@@ -414,6 +430,22 @@ class EmulatedKernels(KernelBackend):
                 out[t] += wt[t, c] * (w_down[e].to(F64) @ act)
         return out.to(torch.float32)
 
+    def connect_streams(self, streams, update, read, n_streams, rows, weight, eps, keep=True):
+        x = streams.to(F64)
+        x = x[None].expand(n_streams, -1, -1) if x.dim() == 2 else x
+        kept = streams
+        if update is not None:
+            y = _whole(update.y).to(F64)
+            if update.scale is not None:
+                y = y * update.scale.to(F64)
+            x = torch.einsum("st,srw->trw", update.mix.to(F64), x) + update.write.to(F64)[:, None, None] * y[None]
+            if keep and rows is None:
+                kept = x.to(streams.dtype)
+        u = x.sum(0) if read is None else torch.einsum("s,srw->rw", read.to(F64), x)
+        u = u if rows is None else u[rows.long()]
+        out = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * weight.to(F64)
+        return out.to(weight.dtype), kept
+
     def embed_positions(self, token_ids, positions, table, pos_table, out):
         out.copy_((table[token_ids.long()].to(F64) + pos_table[positions.long()].to(F64)).to(out.dtype))
 
@@ -448,10 +480,13 @@ class EmulatedKernels(KernelBackend):
             y = y * torch.sigmoid(full[:, gate_col : gate_col + 1])
         out.copy_(y.to(out.dtype))
 
-    def swiglu(self, gate_up, out):
+    def swiglu(self, gate_up, out, activation="silu"):
         gate_up = _whole(gate_up)
         i = out.shape[1]
         g, u = gate_up[:, :i].to(F64), gate_up[:, i:].to(F64)
+        if activation == "gelu_tanh":
+            out.copy_((u * torch.nn.functional.gelu(g, approximate="tanh")).to(out.dtype))
+            return
         out.copy_((u * g / (1.0 + torch.exp(-g))).to(out.dtype))
 
     def argmax(self, logits, out):
