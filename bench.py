@@ -470,6 +470,30 @@ def bubetar_config(width, heads, kv_heads, hd, s_heads, s_dim, s_vdim, inner, ra
             "logit_softcap": 30.0, "layers": layers}
 
 
+# `--design tipezen`: the Tipezen design (retention and capped window attention in turn, values mixed across layers, a gate per
+# head, a dense feed-forward with a gelu gate, four parallel residual streams) beside the Bubetar model of the same sizes,
+# whose layers also hold a window attention with a sink and a linear attention with a constant decay, and beside the Qwen2
+# model of the same width, heads and inner width.  The sizes are those of the Bubetar comparison.
+def tipezen_config(width, heads, kv_heads, hd, s_heads, s_dim, s_vdim, inner, window, streams) -> dict:
+    ff = {"kind": "dense", "ff": inner}
+    retention = {"type": "retention", "mlp": ff,
+                 "mixer": {"heads": s_heads, "dim": s_dim, "vdim": s_vdim, "rot": {"base": 10000.0, "dims": s_dim},
+                           "decay": [1.0 - 2.0 ** (-3 - 5 * h / s_heads) for h in range(s_heads)]}}
+    attention = {"type": "attention", "mlp": ff,
+                 "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "softcap": 50.0,
+                           "mask": {"size": window}, "v_mix": True,
+                           "rot": {"base": 500000.0, "dims": hd, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    return {"architecture": "Tipezen", "vocab": DESIGN_VOCAB, "width": width, "norm": {"eps": 1e-6}, "streams": streams,
+            "layers": [retention, attention] * (DESIGN_LAYERS // 2)}
+
+
+def bubetar_sizes():
+    """(label, sizes of the Bubetar model of the comparison)"""
+    for s, d in zip(NEBANEX_SIZES, DESIGN_SIZES):
+        label, width, heads, kv_heads, hd, s_heads, s_dim, s_vdim = s[:8]
+        yield label, (width, heads, kv_heads, hd, s_heads, s_dim, s_vdim, s[9] * s[10] + s[11], d[6], d[7], d[8])
+
+
 def design_models(design):
     """(label, {name: config}) for every size of the comparison, and how the sizes are named in the record."""
     if design == "pekasun":
@@ -479,11 +503,15 @@ def design_models(design):
             yield label, dict(zip(keys, s[1:])), pekasun_config(*s[1:]), (width, inner, heads, kv_heads, hd)
     elif design == "bubetar":
         keys = ("width", "heads", "kv_heads", "head", "state_heads", "state_key", "state_value", "inner", "latent", "rotated", "window")
-        for s, d in zip(NEBANEX_SIZES, DESIGN_SIZES):
-            label, width, heads, kv_heads, hd, s_heads, s_dim, s_vdim = s[:8]
-            inner = s[9] * s[10] + s[11]
-            sizes = (width, heads, kv_heads, hd, s_heads, s_dim, s_vdim, inner, d[6], d[7], d[8])
+        for label, sizes in bubetar_sizes():
+            width, heads, kv_heads, hd, inner = *sizes[:4], sizes[7]
             yield label, dict(zip(keys, sizes)), bubetar_config(*sizes), (width, inner, heads, kv_heads, hd)
+    elif design == "tipezen":
+        keys = ("width", "heads", "kv_heads", "head", "state_heads", "state_key", "state_value", "inner", "window", "streams")
+        for label, of in bubetar_sizes():
+            sizes = (*of[:8], of[10], 4)
+            width, heads, kv_heads, hd, inner = *sizes[:4], sizes[7]
+            yield label, dict(zip(keys, sizes)), tipezen_config(*sizes), (width, inner, heads, kv_heads, hd)
     else:
         keys = ("width", "heads", "kv_heads", "head", "state_heads", "state_key", "state_value", "experts", "chosen",
                 "expert_inner", "shared_inner")
@@ -508,6 +536,7 @@ def design_comparison(args) -> dict:
         models = {
             design: design_cfg,
             **({"nebanex": nebanex_config(*next(s for s in NEBANEX_SIZES if s[0] == label)[1:])} if design in ("kezolix", "bubetar") else {}),
+            **({"bubetar": bubetar_config(*dict(bubetar_sizes())[label])} if design == "tipezen" else {}),
             "qwen2": dict(QWEN25_05B, hidden_size=width, intermediate_size=inner, num_attention_heads=heads,
                           num_key_value_heads=kv_heads, head_dim=hd, num_hidden_layers=DESIGN_LAYERS, vocab_size=DESIGN_VOCAB,
                           tie_word_embeddings=False),
@@ -573,9 +602,9 @@ def main() -> int:
     ap.add_argument("--no-lookahead", action="store_true",
                     help="wait for a step's tokens on the host before the next step is launched (the scheduler with --serve, "
                          "the decode loop otherwise)")
-    ap.add_argument("--design", default=None, choices=["pekasun", "nebanex", "kezolix", "bubetar"],
+    ap.add_argument("--design", default=None, choices=["pekasun", "nebanex", "kezolix", "bubetar", "tipezen"],
                     help="instead of the record: prefill and decode of that design at a few layer sizes beside the Qwen2 "
-                         "model of equal sizes (kezolix, bubetar: also beside the Nebanex model of equal sizes)")
+                         "model of equal sizes (kezolix, bubetar: also beside the Nebanex model of equal sizes, tipezen: beside the Bubetar model)")
     ap.add_argument("--direct-loop", action="store_true",
                     help="decode with the engine's step function in a loop of the benchmark's own instead of Scheduler.step")
     args = ap.parse_args()

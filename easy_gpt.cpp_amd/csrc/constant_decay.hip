@@ -24,6 +24,8 @@ constexpr int kDecayPowers = 65;           // d^0 .. d^64 per head
 template <typename T>
 struct DecayArgs {
     ProductView<T> proj;
+    const float* flat;                     // proj as one float32 tensor whose heads start on 16 bytes, or null
+    int head_fours;                        // with flat: queries and keys may be rotated four places at a time too
     int proj_width, q_off, k_off, v_off, g_off;
     float k_scale;
     const float* cos_sin;                  // [tokens][rot_dims / 2][2]
@@ -65,11 +67,13 @@ __device__ __forceinline__ bool pair_places(int s, int rot_dims, int interleaved
 }
 __device__ __forceinline__ int pair_slots(int dk, int rot_dims) { return rot_dims / 2 + (dk - rot_dims + 1) / 2; }
 
+__device__ __forceinline__ float gate_value(float z, int act) {
+    const float sig = 1.0f / (1.0f + expf(-z));
+    return act == 0 ? z * sig : sig;
+}
 template <typename T>
 __device__ __forceinline__ float gate_of(const DecayArgs<T>& a, size_t t, int column) {
-    const float z = a.proj.at(t * a.proj_width + a.g_off + column);
-    const float sig = 1.0f / (1.0f + expf(-z));
-    return a.gate_act == 0 ? z * sig : sig;
+    return gate_value(a.proj.at(t * a.proj_width + a.g_off + column), a.gate_act);
 }
 
 // which request and which of its chunks a workgroup has; false: none
@@ -88,6 +92,37 @@ __device__ __forceinline__ bool find_chunk(const DecayArgs<T>& a, int index, int
 template <typename T, int C, int THREADS, typename F>
 __device__ __forceinline__ void stage_heads(const DecayArgs<T>& a, int offset, int h, int t0, int n, int padded, int row, float* dst,
                                             F factor) {
+    const int pads = padded - a.dk;
+    for (int idx = threadIdx.x; idx < C * pads; idx += THREADS) dst[(idx / pads) * row + a.dk + idx % pads] = 0.f;
+    if (a.head_fours) {                                   // halves that turn together, four places of each at a time
+        const int half = a.rot_dims / 2, turns = half / 4, items = turns + (a.dk - a.rot_dims) / 4;
+#pragma unroll 4
+        for (int idx = threadIdx.x; idx < C * items; idx += THREADS) {
+            const int tt = idx / items, s = idx % items;
+            const bool turned = s < turns;
+            const int pa = turned ? 4 * s : a.rot_dims + 4 * (s - turns);
+            float4 x = float4{0.f, 0.f, 0.f, 0.f}, y = x;
+            if (tt < n) {
+                const size_t t = static_cast<size_t>(t0 + tt), at = t * a.proj_width + offset + h * a.dk;
+                const float f = factor(tt);
+                x = *reinterpret_cast<const float4*>(a.flat + at + pa);
+                if (turned) {
+                    y = *reinterpret_cast<const float4*>(a.flat + at + pa + half);
+                    const float4 c0 = *reinterpret_cast<const float4*>(a.cos_sin + t * a.rot_dims + 8 * s);
+                    const float4 c1 = *reinterpret_cast<const float4*>(a.cos_sin + t * a.rot_dims + 8 * s + 4);
+                    rotate_pair(x.x, y.x, c0.x * a.mag, c0.y * a.mag, x.x, y.x);
+                    rotate_pair(x.y, y.y, c0.z * a.mag, c0.w * a.mag, x.y, y.y);
+                    rotate_pair(x.z, y.z, c1.x * a.mag, c1.y * a.mag, x.z, y.z);
+                    rotate_pair(x.w, y.w, c1.z * a.mag, c1.w * a.mag, x.w, y.w);
+                    y.x *= f, y.y *= f, y.z *= f, y.w *= f;
+                }
+                x.x *= f, x.y *= f, x.z *= f, x.w *= f;
+            }
+            *reinterpret_cast<float4*>(dst + tt * row + pa) = x;
+            if (turned) *reinterpret_cast<float4*>(dst + tt * row + pa + half) = y;
+        }
+        return;
+    }
     const int slots = pair_slots(a.dk, a.rot_dims);
 #pragma unroll 4
     for (int idx = threadIdx.x; idx < C * slots; idx += THREADS) {
@@ -109,12 +144,21 @@ __device__ __forceinline__ void stage_heads(const DecayArgs<T>& a, int offset, i
         dst[tt * row + pa] = x;
         if (pb < a.dk) dst[tt * row + pb] = y;
     }
-    const int pads = padded - a.dk;
-    for (int idx = threadIdx.x; idx < C * pads; idx += THREADS) dst[(idx / pads) * row + a.dk + idx % pads] = 0.f;
 }
 
 template <typename T, int C, int WIDTH, int THREADS>
 __device__ __forceinline__ void stage_values(const DecayArgs<T>& a, int h, int t0, int n, int row, float* dst) {
+    if (a.flat != nullptr) {                              // four features at a time (dv is a multiple of four)
+#pragma unroll 8
+        for (int idx = threadIdx.x; idx < C * (WIDTH / 4); idx += THREADS) {
+            const int tt = idx / (WIDTH / 4), f = idx % (WIDTH / 4) * 4;
+            float4 v = float4{0.f, 0.f, 0.f, 0.f};
+            if (tt < n && f < a.dv)
+                v = *reinterpret_cast<const float4*>(a.flat + static_cast<size_t>(t0 + tt) * a.proj_width + a.v_off + h * a.dv + f);
+            *reinterpret_cast<float4*>(dst + tt * row + f) = v;
+        }
+        return;
+    }
 #pragma unroll 4
     for (int idx = threadIdx.x; idx < C * WIDTH; idx += THREADS) {
         const int tt = idx / WIDTH, f = idx % WIDTH;
@@ -179,9 +223,18 @@ __global__ __launch_bounds__(64 * RT) void chunk_sums_kernel(DecayArgs<T> a) {
         for (int v = 0; v < 4; ++v) {
             const int row = r * 16 + lg * 4 + v;
             if (row >= a.dk) continue;
+            float* at = dst + static_cast<size_t>(row) * a.dv + lj * DT;
+            if constexpr (DT % 4 == 0) {
+                if (a.dv == 16 * DT) {
+#pragma unroll
+                    for (int d = 0; d < DT; d += 4)
+                        *reinterpret_cast<float4*>(at + d) = float4{acc[d][v], acc[d + 1][v], acc[d + 2][v], acc[d + 3][v]};
+                    continue;
+                }
+            }
 #pragma unroll
             for (int d = 0; d < DT; ++d)
-                if (lj * DT + d < a.dv) dst[static_cast<size_t>(row) * a.dv + lj * DT + d] = acc[d][v];
+                if (lj * DT + d < a.dv) at[d] = acc[d][v];
         }
     }
 }
@@ -256,35 +309,52 @@ __global__ __launch_bounds__(64 * RT) void chunk_outputs_kernel(DecayArgs<T> a) 
     d_f32x4 o[DT];
 #pragma unroll
     for (int d = 0; d < DT; ++d) o[d] = d_f32x4{0.f, 0.f, 0.f, 0.f};
-    // the state before the chunk (a new request's first chunk has none)
+    const bool whole_runs = a.dv == 16 * DT;              // every lane's run of features lies inside the head
+    // the gates of this lane's results (in flight from here on)
+    constexpr bool KEEP_GATES = DT <= 8;
+    float gates[4][KEEP_GATES ? DT : 1];
+    const bool gates_here = KEEP_GATES && a.flat != nullptr && whole_runs;
+    if constexpr (KEEP_GATES) if (gates_here) {
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const int tt = min(wave * 16 + lg * 4 + v, n - 1);
+            load_run<DT>(a.flat + static_cast<size_t>(t0 + tt) * a.proj_width + a.g_off + h * a.dv + lj * DT, gates[v]);
+        }
+    }
+    // the state before the chunk (a new request's first chunk has none), its rows read a piece ahead
     if (c > 0 || !(a.fresh != nullptr && a.fresh[b] != 0)) {
         const float* state = a.chunk_states + (static_cast<size_t>(blockIdx.x) * a.heads + h) * a.dk * a.dv;
         const float through = pw_s[row + 1];
-        const bool whole_runs = a.dv == 16 * DT;          // every lane's run lies inside the row
-        for (int kk = 0; kk < pieces; ++kk) {
-            const float4 q4 = *reinterpret_cast<const float4*>(q_row + kk * 16);
-            const float qv[4] = {q4.x * through, q4.y * through, q4.z * through, q4.w * through};
-            float sv[4][DT];
+        auto state_piece = [&](int kk, float (&sv)[4][DT]) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int key = kk * 16 + lg * 4 + i;
                 const float* src = state + static_cast<size_t>(key) * a.dv + lj * DT;
+                if (whole_runs && a.dk % 16 == 0) {
+                    load_run<DT>(src, sv[i]);
+                } else {
 #pragma unroll
-                for (int d = 0; d < DT; ++d) sv[i][d] = 0.f;
-                if (key < a.dk) {
-                    if (whole_runs) {
-                        load_run<DT>(src, sv[i]);
-                    } else {
-#pragma unroll
-                        for (int d = 0; d < DT; ++d)
-                            if (lj * DT + d < a.dv) sv[i][d] = src[d];
-                    }
+                    for (int d = 0; d < DT; ++d) sv[i][d] = key < a.dk && lj * DT + d < a.dv ? src[d] : 0.f;
                 }
             }
+        };
+        auto state_product = [&](int kk, const float (&sv)[4][DT]) {
+            const float4 q4 = *reinterpret_cast<const float4*>(q_row + kk * 16);
+            const float qv[4] = {q4.x * through, q4.y * through, q4.z * through, q4.w * through};
 #pragma unroll
             for (int i = 0; i < 4; ++i)
 #pragma unroll
                 for (int d = 0; d < DT; ++d) o[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv[i], sv[i][d], o[d], 0, 0, 0);
+        };
+        float sa[4][DT], sb[4][DT];                       // (two sets in turn)
+        state_piece(0, sa);
+        for (int kk = 0; kk < pieces; kk += 2) {
+            if (kk + 1 < pieces) state_piece(kk + 1, sb);
+            state_product(kk, sa);
+            if (kk + 1 < pieces) {
+                if (kk + 2 < pieces) state_piece(kk + 2, sa);
+                state_product(kk + 1, sb);
+            }
         }
     }
     // the chunk's own tokens up to each row's: scores transposed, so that a lane holds four keys of its row, which are the
@@ -324,14 +394,32 @@ __global__ __launch_bounds__(64 * RT) void chunk_outputs_kernel(DecayArgs<T> a) 
         const float inv = inv_rms(ss, 1.0f / static_cast<float>(a.dv), a.eps);
         const size_t t = static_cast<size_t>(t0 + tt);
         T* dst = a.out + t * a.heads * a.dv + static_cast<size_t>(h) * a.dv;
+        float y[DT];
 #pragma unroll
         for (int d = 0; d < DT; ++d) {
             const int f = lj * DT + d;
-            if (f >= a.dv) break;
-            float y = o[d][v] * inv;
-            if (a.norm_w != nullptr) y *= to_float(a.norm_w[f]);
-            dst[f] = from_float<T>(y * gate_of(a, t, h * a.dv + f));
+            y[d] = 0.f;
+            if (f >= a.dv) continue;
+            y[d] = o[d][v] * inv;
+            if (a.norm_w != nullptr) y[d] *= to_float(a.norm_w[f]);
+            y[d] *= gates_here ? gate_value(gates[v][KEEP_GATES ? d : 0], a.gate_act) : gate_of(a, t, h * a.dv + f);
         }
+        if constexpr (sizeof(T) == 2 && DT % 8 == 0) {
+            if (whole_runs) {
+#pragma unroll
+                for (int d = 0; d < DT; d += 8) {
+                    uint32_t w[4];
+#pragma unroll
+                    for (int i = 0; i < 4; ++i)
+                        w[i] = f32_to_bf16_bits(y[d + 2 * i]) | (static_cast<uint32_t>(f32_to_bf16_bits(y[d + 2 * i + 1])) << 16);
+                    *reinterpret_cast<uint4*>(dst + lj * DT + d) = uint4{w[0], w[1], w[2], w[3]};
+                }
+                continue;
+            }
+        }
+#pragma unroll
+        for (int d = 0; d < DT; ++d)
+            if (lj * DT + d < a.dv) dst[lj * DT + d] = from_float<T>(y[d]);
     }
 }
 
@@ -351,7 +439,8 @@ __global__ __launch_bounds__(1024) void decay_steps_kernel(DecayArgs<T> a) {
     float* q_s = decay_smem;
     float* k_s = q_s + dk;
     float* v_s = k_s + dk + ((2 * dk) & 3 ? 4 - ((2 * dk) & 3) : 0);      // (on 16 bytes)
-    float* part_s = v_s + (dv + 3) / 4 * 4;
+    float* g_s = v_s + (dv + 3) / 4 * 4;
+    float* part_s = g_s + dv;
     float* record = a.states + (static_cast<size_t>(a.slots[b]) * a.heads + h) * dk * dv;
     const bool anew = a.fresh != nullptr && a.fresh[b] != 0;
     float s[NV][VEC];
@@ -367,9 +456,11 @@ __global__ __launch_bounds__(1024) void decay_steps_kernel(DecayArgs<T> a) {
     for (int i0 = 0; i0 < n; ++i0) {
         const size_t t = static_cast<size_t>(t0 + i0), row = t * a.proj_width;
         __syncthreads();                              // the token before is written out
-        for (int idx = threadIdx.x; idx < 2 * slots + dv; idx += blockDim.x) {
+        for (int idx = threadIdx.x; idx < 2 * slots + 2 * dv; idx += blockDim.x) {
             if (idx >= 2 * slots) {
-                v_s[idx - 2 * slots] = a.proj.at(row + a.v_off + h * dv + (idx - 2 * slots));
+                const int f = idx - 2 * slots;
+                if (f < dv) v_s[f] = a.proj.at(row + a.v_off + h * dv + f);
+                else g_s[f - dv] = gate_of(a, t, h * dv + (f - dv));
                 continue;
             }
             const bool key = idx >= slots;
@@ -387,9 +478,6 @@ __global__ __launch_bounds__(1024) void decay_steps_kernel(DecayArgs<T> a) {
             dst[pa] = x * f;
             if (pb < dk) dst[pb] = y * f;
         }
-        // (a thread of the output stage reads its gate while the state is updated)
-        float gate = 0.f;
-        if (threadIdx.x < dv) gate = gate_of(a, t, h * dv + threadIdx.x);
         __syncthreads();
         if (active) {
             float vv[VEC], o[VEC];
@@ -417,7 +505,7 @@ __global__ __launch_bounds__(1024) void decay_steps_kernel(DecayArgs<T> a) {
         if (threadIdx.x < dv) {
             float y = o * inv;
             if (a.norm_w != nullptr) y *= to_float(a.norm_w[threadIdx.x]);
-            a.out[(t * a.heads + h) * dv + threadIdx.x] = from_float<T>(y * gate);
+            a.out[(t * a.heads + h) * dv + threadIdx.x] = from_float<T>(y * g_s[threadIdx.x]);
         }
     }
     if (active) {
@@ -487,14 +575,16 @@ static int launch_chunks_for(const DecayArgs<T>& a, int n_chunks, hipStream_t s)
 template <typename T, int VEC>
 static int launch_steps(const DecayArgs<T>& a, hipStream_t s) {
     const int columns = (a.dv + VEC - 1) / VEC;
-    // the narrowest workgroup whose threads keep at most 32 values of the state each, else the widest
+    // the narrowest workgroup whose threads keep at most 32 values of the state each and that reads a token's values and
+    // gates in one round, else the widest
+    const int items = 2 * (a.rot_dims / 2 + (a.dk - a.rot_dims + 1) / 2) + 2 * a.dv;
     int threads = 256, rows = 0;
     for (;; threads *= 2) {
         rows = (a.dk + threads / columns - 1) / (threads / columns);
-        if (rows * VEC <= 32 || threads == 1024) break;
+        if ((rows * VEC <= 32 && items <= threads) || threads == 1024) break;
     }
     const int groups = threads / columns;
-    const size_t lds = (static_cast<size_t>(2 * a.dk + 4) + (a.dv + 3) / 4 * 4 + static_cast<size_t>(groups) * columns * VEC) * sizeof(float);
+    const size_t lds = (static_cast<size_t>(2 * a.dk + 4) + (a.dv + 3) / 4 * 4 + a.dv + static_cast<size_t>(groups) * columns * VEC) * sizeof(float);
     if (lds > 48 * 1024) return EGPT_UNSUPPORTED_SIZE;
     const dim3 grid(a.n_seqs, a.heads);
 #define EGPT_STEPS(NV)                                                          \
@@ -516,6 +606,11 @@ static int launch_decay(DecayArgs<T>& a, const void* proj, int n_splits, int n_t
     a.proj.partial = n_splits > 0 ? static_cast<const float*>(proj) : nullptr;
     a.proj.n_splits = n_splits;
     a.proj.split_stride = static_cast<size_t>(n_tokens) * a.proj_width;
+    a.flat = n_splits == 1 ? static_cast<const float*>(proj) : (n_splits == 0 && sizeof(T) == 4 ? static_cast<const float*>(proj) : nullptr);
+    const bool fours = a.proj_width % 4 == 0 && a.dv % 4 == 0 && a.v_off % 4 == 0 && a.g_off % 4 == 0 &&
+                       reinterpret_cast<uintptr_t>(proj) % 16 == 0;
+    if (!fours) a.flat = nullptr;
+    a.head_fours = a.flat != nullptr && !a.interleaved && a.rot_dims % 8 == 0 && a.dk % 4 == 0 && a.q_off % 4 == 0 && a.k_off % 4 == 0;
     if (n_chunks > 0) return decay_chunk(a.dk, a.dv) == 64 ? launch_chunks_for<T, 4>(a, n_chunks, s) : launch_chunks_for<T, 2>(a, n_chunks, s);
     if (a.dv % 4 == 0) return launch_steps<T, 4>(a, s);
     return launch_steps<T, 1>(a, s);
