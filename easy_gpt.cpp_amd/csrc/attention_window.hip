@@ -261,7 +261,8 @@ __device__ __forceinline__ int place_in_page(int key, int page_size, int page_sh
     return page_shift >= 0 ? key & (page_size - 1) : key % page_size;
 }
 
-template <typename T, int DT, int RT, int RW>
+// CAPPED: scores pass the tanh cap (and get neither a bias table nor slopes).
+template <typename T, int DT, int RT, int RW, bool CAPPED>
 __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attention_tiled_kernel(WindowArgs a) {
     constexpr int E = 16 / sizeof(T);             // elements in 16 bytes
     constexpr int KT = sizeof(T) == 2 ? 64 : 32;  // keys per chunk
@@ -530,7 +531,19 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
             // a chunk that every row of the tile sees whole (below the diagonal and inside the window, or all kept
             // tokens) needs no mask
             const bool whole = key0 + KT - 1 <= tile_p_min[w] && (key0 >= tile_lo_max[w] || key0 + KT <= a.keep_first);
-            if (a.dist_bias != nullptr) {
+            if constexpr (CAPPED) {
+                const float inner = scale / a.softcap;
+#pragma unroll
+                for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+                    for (int v = 0; v < 4; ++v) {
+                        const int key = key0 + kt * 16 + lg * 4 + v;
+                        const bool seen = whole || (key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first));
+                        const float sc = seen ? a.softcap * bounded_tanh<T>(acc[w][kt][v] * inner) : -INFINITY;
+                        acc[w][kt][v] = sc;
+                        mx = fmaxf(mx, sc);
+                    }
+            } else if (a.dist_bias != nullptr) {
                 // the bias of the row's head by distance; a chunk that lies `far` or more behind every row of the tile
                 // gets the table's last entry throughout
                 const float* brow = a.dist_bias + static_cast<size_t>(head[w]) * (a.dist_far + 1);
@@ -558,18 +571,6 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
                         const int key = key0 + kt * 16 + lg * 4 + v;
                         const bool seen = whole || (key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first));
                         const float sc = seen ? fmaf(acc[w][kt][v], scale, -slope * static_cast<float>(p_row[w] - key)) : -INFINITY;
-                        acc[w][kt][v] = sc;
-                        mx = fmaxf(mx, sc);
-                    }
-            } else if (a.softcap > 0.f) {
-                const float inner = scale / a.softcap;
-#pragma unroll
-                for (int kt = 0; kt < NKT; ++kt)
-#pragma unroll
-                    for (int v = 0; v < 4; ++v) {
-                        const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = whole || (key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first));
-                        const float sc = seen ? a.softcap * bounded_tanh<T>(acc[w][kt][v] * inner) : -INFINITY;
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
                     }
@@ -711,13 +712,13 @@ __global__ __launch_bounds__(kWave) void window_attention_fold_kernel(const floa
     }
 }
 
-template <typename T, int DT, int RT, int RW>
+template <typename T, int DT, int RT, int RW, bool CAPPED>
 static int launch_tiled(const WindowArgs& a, int max_rows, hipStream_t s) {
     constexpr int E = 16 / sizeof(T), KT = sizeof(T) == 2 ? 64 : 32, PF = 4 * E, ROWS = 16 * RT * RW;
     const int krow = (a.dk + PF - 1) / PF * PF + E;
     const size_t lds = (static_cast<size_t>(ROWS + KT) * krow + static_cast<size_t>(DT) * 16 * (KT + E)) * sizeof(T);
     if (lds > 160 * 1024) return EGPT_UNSUPPORTED_SIZE;
-    auto kernel = window_attention_tiled_kernel<T, DT, RT, RW>;
+    auto kernel = window_attention_tiled_kernel<T, DT, RT, RW, CAPPED>;
     if (lds > 48 * 1024) {
         static bool raised = false;       // per instance of this template: the limit is asked for once
         if (!raised) {
@@ -737,8 +738,12 @@ static int launch_tiled(const WindowArgs& a, int max_rows, hipStream_t s) {
 // row_tiles: 4 (four wavefronts with 16 rows each) or 8 (with 32 rows each)
 template <typename T, int DT>
 static int launch_tiled_for_rows(const WindowArgs& a, int max_rows, int row_tiles, hipStream_t s) {
-    if (row_tiles == 8) return launch_tiled<T, DT, 4, 2>(a, max_rows, s);
-    return launch_tiled<T, DT, 4, 1>(a, max_rows, s);
+    if (a.softcap > 0.f) {
+        if (row_tiles == 8) return launch_tiled<T, DT, 4, 2, true>(a, max_rows, s);
+        return launch_tiled<T, DT, 4, 1, true>(a, max_rows, s);
+    }
+    if (row_tiles == 8) return launch_tiled<T, DT, 4, 2, false>(a, max_rows, s);
+    return launch_tiled<T, DT, 4, 1, false>(a, max_rows, s);
 }
 
 template <typename T>
