@@ -158,7 +158,7 @@ def _edge_cuts(reqs, rid, edges):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("window, dim, vdim", [(5, 16, 16), (64, 16, 16), (100, 12, 20), (33, 64, 32)])
+@pytest.mark.parametrize("window, dim, vdim", [(5, 16, 16), (64, 16, 16), (100, 12, 20), (33, 64, 48)])
 def test_a_loud_key_is_seen_to_the_windows_last_position_and_not_beyond(tmp_path, dtype, window, dim, vdim):
     """One key stands out at position `window`.  Asking tokens at the last position whose window holds it and at the next
     one: as a whole prompt, in portions cut just before and just after the edge, and decoded one by one; against the plain
