@@ -1,2 +1,2 @@
 """Built-in architectures; importing this package registers them."""
-from . import bubetar, kezolix, nebanex, pekasun, qwen2, tipezen  # noqa: F401
+from . import bubetar, karesun, kezolix, nebanex, pekasun, qwen2, tipezen  # noqa: F401

@@ -1,5 +1,6 @@
 from .base import ConfigError, KeyReader, read_json
 from .bubetar import BubetarConfig
+from .karesun import KaresunConfig
 from .kezolix import KezolixConfig
 from .nebanex import NebanexConfig
 from .pekasun import PekasunConfig
@@ -20,6 +21,7 @@ __all__ = [
     "BubetarConfig",
     "ConfigError",
     "KeyReader",
+    "KaresunConfig",
     "KezolixConfig",
     "NebanexConfig",
     "PekasunConfig",

@@ -1,7 +1,8 @@
 // Activations of feed-forward layers that have no gate product: the square of relu, and a polynomial of the inner
 // values whose three powers are each divided by their root mean square over the token's inner values.  Optionally the
 // whole row is multiplied by the sigmoid of one more column of the same product (a gate of one number per token, whose
-// weights ride as one more row of the up matrix).  Statistics and the activation are float32; the result is rounded
+// weights ride as one more row of the up matrix).  The product may still lack each row's factor of a norm that was folded
+// into it.  Statistics and the activation are float32; the result is rounded
 // once, when it is written in the activation type for the product that follows.
 #include "api.h"
 #include "common.h"
@@ -54,7 +55,7 @@ __device__ __forceinline__ void load_values(const bf16_t* p, float* v) {
 // any width); else its element type (the activation type of a whole product, float for a product written out in
 // float32), read and written in pieces of 16 bytes of the result: rows start on 16 bytes then.
 template <typename T, int MODE, typename S>
-__global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, int z_width, int cols, const float* __restrict__ coef,
+__global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, RowFactor factor, int z_width, int cols, const float* __restrict__ coef,
                                                             float eps, int gate_col, T* __restrict__ out) {
     __shared__ float scratch[16];
     constexpr int E = 16 / sizeof(T);
@@ -67,8 +68,9 @@ __global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, in
     }
     const size_t row = static_cast<size_t>(blockIdx.x) * z_width;
     T* o = out + static_cast<size_t>(blockIdx.x) * cols;
+    const float rf = factor.of(blockIdx.x);
     float gate = 1.0f;
-    if (gate_col >= 0) gate = 1.0f / (1.0f + expf(-z.at(row + gate_col)));
+    if (gate_col >= 0) gate = 1.0f / (1.0f + expf(-z.at(row + gate_col) * rf));
     if constexpr (MODE == 0) {
         if constexpr (PIECES) {
             for (int j = threadIdx.x * E; j < cols; j += 256 * E) {
@@ -76,14 +78,14 @@ __global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, in
                 load_values<E>(src + row + j, v);
 #pragma unroll
                 for (int e = 0; e < E; ++e) {
-                    const float r = fmaxf(v[e], 0.f);
+                    const float r = fmaxf(v[e] * rf, 0.f);
                     v[e] = r * r * gate;
                 }
                 store_piece(o + j, v);
             }
         } else {
             for (int j = threadIdx.x; j < cols; j += blockDim.x) {
-                const float v = fmaxf(z.at(row + j), 0.f);
+                const float v = fmaxf(z.at(row + j) * rf, 0.f);
                 o[j] = from_float<T>(v * v * gate);
             }
         }
@@ -106,19 +108,22 @@ __global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, in
                     if (j < cols) {
                         load_values<E>(src + row + j, v + i * E);
 #pragma unroll
-                        for (int e = 0; e < E; ++e) take(v[i * E + e]);
+                        for (int e = 0; e < E; ++e) {
+                            v[i * E + e] *= rf;
+                            take(v[i * E + e]);
+                        }
                     }
                 }
             } else {
 #pragma unroll
                 for (int i = 0; i < kKeep; ++i) {
                     const int j = threadIdx.x + i * 256;
-                    v[i] = j < cols ? z.at(row + j) : 0.f;
+                    v[i] = j < cols ? z.at(row + j) * rf : 0.f;
                     take(v[i]);
                 }
             }
         } else {
-            for (int j = threadIdx.x; j < cols; j += blockDim.x) take(z.at(row + j));
+            for (int j = threadIdx.x; j < cols; j += blockDim.x) take(z.at(row + j) * rf);
         }
         const float inv_n = 1.0f / static_cast<float>(cols);
         const float n1 = coef[0] / sqrtf(block_sum(s1, scratch) * inv_n + eps);
@@ -148,7 +153,7 @@ __global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, in
                 }
             }
         } else {
-            for (int j = threadIdx.x; j < cols; j += blockDim.x) o[j] = from_float<T>(poly(z.at(row + j)));
+            for (int j = threadIdx.x; j < cols; j += blockDim.x) o[j] = from_float<T>(poly(z.at(row + j) * rf));
         }
     }
 }
@@ -158,7 +163,7 @@ __global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, in
 using namespace egpt;
 
 template <typename T>
-static void launch_activation(const void* z, int z_splits, int z_width, int cols, int mode, const float* coef, float eps,
+static void launch_activation(const void* z, int z_splits, const RowFactor& factor, int z_width, int cols, int mode, const float* coef, float eps,
                               int gate_col, void* out, int n_tokens, hipStream_t s) {
     ProductView<T> v;
     v.whole = z_splits == 0 ? static_cast<const T*>(z) : nullptr;
@@ -172,7 +177,7 @@ static void launch_activation(const void* z, int z_splits, int z_width, int cols
                          reinterpret_cast<uintptr_t>(out) % 16 == 0;
     const int src = !aligned || z_splits > 1 ? 0 : (z_splits == 0 ? 1 : 2);      // as it comes; of T; of float
     T* o = static_cast<T*>(out);
-#define EGPT_ACTIVATION(MODE, S) ff_activation_kernel<T, MODE, S><<<n_tokens, 256, 0, s>>>(v, z_width, cols, coef, eps, gate_col, o)
+#define EGPT_ACTIVATION(MODE, S) ff_activation_kernel<T, MODE, S><<<n_tokens, 256, 0, s>>>(v, factor, z_width, cols, coef, eps, gate_col, o)
     if (mode == 0) {
         if (src == 0) EGPT_ACTIVATION(0, void);
         else if (src == 1) EGPT_ACTIVATION(0, T);
@@ -185,17 +190,19 @@ static void launch_activation(const void* z, int z_splits, int z_width, int cols
 #undef EGPT_ACTIVATION
 }
 
-extern "C" int egpt_ff_activation(const void* z, int z_splits, int z_width, int cols, int mode, const float* coef, float eps,
+extern "C" int egpt_ff_activation(const void* z, int z_splits, const float* row_ss, int ss_splits, int hidden, float norm_eps, int z_width, int cols, int mode, const float* coef, float eps,
                                   int gate_col, void* out, int n_tokens, int dtype, void* stream) {
     if (!z || !out || z_splits < 0 || cols <= 0 || cols > z_width || n_tokens < 0 || (mode != 0 && mode != 1) ||
-        (mode == 1 && !coef) || gate_col >= z_width || (dtype != 0 && dtype != 1))
+        (mode == 1 && !coef) || gate_col >= z_width || (dtype != 0 && dtype != 1) ||
+        (row_ss && (z_splits < 1 || ss_splits < 1 || hidden <= 0)))
         return EGPT_BAD_ARGUMENT;
     if (n_tokens == 0) return EGPT_OK;
     hipStream_t s = static_cast<hipStream_t>(stream);
+    const RowFactor factor{row_ss, ss_splits, n_tokens, hidden, norm_eps};
     if (dtype == 0)
-        launch_activation<float>(z, z_splits, z_width, cols, mode, coef, eps, gate_col, out, n_tokens, s);
+        launch_activation<float>(z, z_splits, factor, z_width, cols, mode, coef, eps, gate_col, out, n_tokens, s);
     else
-        launch_activation<bf16_t>(z, z_splits, z_width, cols, mode, coef, eps, gate_col, out, n_tokens, s);
+        launch_activation<bf16_t>(z, z_splits, factor, z_width, cols, mode, coef, eps, gate_col, out, n_tokens, s);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }

@@ -15,12 +15,13 @@ int egpt_abi_version(void);
 // units of 2^-32 (see common.h), which the products of steps of few tokens add their partial results into.
 int egpt_embed(const int32_t* ids, const void* table, void* out, int fixed, int n_tokens, int hidden, int vocab,
                int dtype, void* stream);
-// h += delta (delta may be null); out = rmsnorm(h) * weight.  rows == null: every row, h written back.
+// h += delta (delta may be null); out = rmsnorm(h) * (weight_offset + weight).  rows == null: every row, h written back.
 // rows != null: only the listed rows, gathered into out[n_rows], h untouched.
 // A product may arrive as float32 partial sums of a split-k product, [n_splits][rows][cols]: then the
 // *_splits argument is > 0 and the consumer adds the splits up; 0 means one tensor of the activation type.
 int egpt_add_rmsnorm(void* h, int fixed, const void* delta, int delta_splits, int delta_rows, const int32_t* rows,
-                     const void* weight, float eps, void* out, int n_rows, int hidden, int dtype, void* stream);
+                     const void* weight, float weight_offset, float eps, void* out, int n_rows, int hidden, int dtype,
+                     void* stream);
 // row_ss (may be null) float32 [ss_splits, n_tokens]: gate_up are float32 partial sums that still lack each row's factor
 // 1/sqrt(sum_s row_ss[s][t] / hidden + eps)
 // act (here and in the products below that end or begin with it): the gate's activation, 0 silu, 1 the tanh form of gelu
@@ -112,8 +113,9 @@ int egpt_attention_combine(const float* part_o, const float* part_ml, void* out,
 // Products for m <= 16 rows whose x operand is computed while it is staged (see gemm_skinny.hip).
 // h_fixed != 0: h_in is a fixed-point residual stream that is complete as it is (no delta, h_out unused).
 int egpt_gemm_skinny_norm(const void* h_in, int h_fixed, float* h_out, const float* delta, int delta_splits,
-                          const void* norm_w, const void* w, float* out, float* ss_out, int m, int n, int k,
-                          int n_splits, int waves, void* stream);
+                          const void* norm_w, float norm_offset, const void* w, float* out, float* ss_out, int m, int n,
+                          int k, int n_splits, int waves, void* stream);
+// act 2: gate_up is up alone, [gu_splits][m][k], and the operand relu(up)^2.
 int egpt_gemm_skinny_swiglu(const float* gate_up, int gu_splits, const float* ss_in, int ss_splits, int hidden,
                             float eps, const void* w, float* out, void* acc_fixed, int m, int n, int k, int n_splits,
                             int waves, int act, void* stream);
@@ -140,7 +142,7 @@ int egpt_embed_rmsnorm(const int32_t* ids, const void* table, const void* weight
 // the angles in cos_sin float32 [n_tokens][rot_dims / 2][2] (cos, sin; both times mag).
 // values_out (may be null): the value heads as float32 [n_tokens][nkv * dv]; mix_with (may be null) float32 of that shape: what is
 // stored is (1 - mix) * value + mix * mix_with (values_out is not mixed); gates_out float32 [n_tokens][n_gates]: sigmoids of the
-// n_gates columns from gate_off on (n_gates 0: none).
+// n_gates columns from gate_off on (n_gates 0: none).  nkv 0: rows of queries alone, nothing is stored (slots null).
 int egpt_head_norm_store(const void* proj, int n_splits, const float* row_ss, int ss_splits, int hidden, float norm_eps,
                          int row_width, void* q_out, const void* q_weight, const void* k_weight, float eps, int flags,
                          const float* cos_sin, int rot_dims, float mag, const int32_t* slots, void* k_cache, void* v_cache,
@@ -170,24 +172,29 @@ int egpt_sigmoid_gate(const void* x, int heads, const void* gate, int gate_split
 // query's block of positions, floor(j / block) == floor(p / block).  slopes float32 [nq] (null: none): the scaled score
 // of key j loses slopes[head] * (p - j) (the matrix-core kernel takes a bias table or slopes, not both).  softcap c > 0: the
 // scaled score s becomes c tanh(s / c) (neither bias nor slopes then; the sink is not capped).  head_gate float32 [n_tokens][nq]
-// (null: none): a factor on each head's output.  q [n_tokens][nq][dk],
+// (null: none): a factor on each head's output.  maps 2 (else 1; no sink, bias, slopes or gate then): queries and keys are two
+// maps side by side, [map 1 | map 2] of dk / 2 each, over the same values; with a1, a2 their outputs a head's output is
+// a / sqrt(mean(a^2) + out_eps) * out_scale, a = a1 - map_weight * a2.  q [n_tokens][nq][dk],
 // out [n_tokens][nq][dv]; the other operands as egpt_paged_attention.
 int egpt_window_attention(const void* q, void* out, const void* k_cache, const void* v_cache, const int32_t* block_table,
                           int table_width, const int32_t* q_start, const int32_t* q_len, const int32_t* kv_len,
                           int n_seqs, int n_tokens, int nq, int nkv, int dk, int dv, int page_size, float scale,
                           int window, int keep_first, const float* sink, const float* dist_bias, int dist_far, int block,
-                          const float* slopes, float softcap, const float* head_gate, int dtype, void* stream);
+                          const float* slopes, float softcap, const float* head_gate, int maps, float map_weight,
+                          float out_scale, float out_eps, int dtype, void* stream);
 // The same on the matrix cores: dk a multiple of 4 (float32) or 8 (bfloat16) up to 256, dv a multiple of 16 up to 256,
 // page_size a multiple of 16.  row_tiles: tiles of 16 rows to a workgroup of four wavefronts: 8 (32 rows to a wavefront)
 // or 4 (16).  With
 // n_splits > 1 the chunks of keys of a workgroup's rows are dealt over as many workgroups, whose results part_o
-// [n_splits][n_tokens][nq][dv] and part_ml [n_splits][n_tokens][nq][2] (float32) a second kernel folds.
+// [n_splits][n_tokens][nq][dv] and part_ml [n_splits][n_tokens][nq][2] (float32; maps 2: [n_splits][n_tokens][nq][map]..) a
+// second kernel folds.  With maps 2 dk / 2 must be such a multiple, and row_tiles is 4.
 int egpt_window_attention_tiled(const void* q, void* out, float* part_o, float* part_ml, const void* k_cache,
                                 const void* v_cache, const int32_t* block_table, int table_width, const int32_t* q_start,
                                 const int32_t* q_len, const int32_t* kv_len, int n_seqs, int n_tokens, int nq, int nkv,
                                 int dk, int dv, int page_size, float scale, int window, int keep_first, const float* sink,
                                 const float* dist_bias, int dist_far, int block, const float* slopes, float softcap,
-                                const float* head_gate, int n_splits, int row_tiles, int dtype, void* stream);
+                                const float* head_gate, int maps, float map_weight, float out_scale, float out_eps,
+                                int n_splits, int row_tiles, int dtype, void* stream);
 // ---- residual stream and logits (stream_ops.hip)
 // out[t] = table[ids[t]] * factor as the float32 residual stream.
 int egpt_embed_scaled(const int32_t* ids, const void* table, float factor, float* out, int n_tokens, int hidden, int vocab,
@@ -202,9 +209,9 @@ int egpt_add_layernorm(float* h, const void* delta, int delta_splits, int delta_
 int egpt_normed_pair_mean(const void* a, int a_splits, const void* b, int b_splits, const void* bias_a, const void* bias_b,
                           const void* wa, const void* wb, float eps, float factor, float factor_b, float* out, int n_rows,
                           int hidden, int dtype, void* stream);
-// out[t] = table[ids[t]] + pos_table[positions[t]] as the float32 residual stream.
-int egpt_embed_positions(const int32_t* ids, const int32_t* positions, const void* table, const void* pos_table, float* out,
-                         int n_tokens, int hidden, int vocab, int max_pos, int dtype, void* stream);
+// out[t] = factor * table[ids[t]] + pos_table[positions[t]] as the residual stream (float32, or fixed point with fixed != 0).
+int egpt_embed_positions(const int32_t* ids, const int32_t* positions, const void* table, const void* pos_table, float factor,
+                         void* out, int fixed, int n_tokens, int hidden, int vocab, int max_pos, int dtype, void* stream);
 // x = h + mult * LN(y) * post_w (LN without bias; y a product: one tensor or float32 partial sums).  With hist (float32
 // [n_hist + 1][n_rows][hidden]) x is stored as hist[n_hist] and v = sum_(j <= n_hist) mix[j] * hist[j], else v = x.
 // h_out = v (h_out may be h).  With next_w, out = LN(v) * next_w in the activation type.
@@ -287,12 +294,14 @@ int egpt_delta_rule_scan(const float* ops, int ops_width, int q_off, int k_off, 
 // logits = x router^T + bias in float32; the `top` largest per token (lowest index among equals) to chosen[t][top], the
 // softmax over the chosen logits to weight[t][top].
 // score_all: scores = softmax over all experts; the `top` experts with the largest score + correction (float32 [experts],
-// null: none) are chosen, and weigh score / (sum of the chosen scores + 1e-20) * weight_scale.
+// null: none) are chosen, and weigh score / (sum of the chosen scores + 1e-20) * weight_scale, or with normalized == 0
+// score * weight_scale.  groups > 1 (with score_all): the outputs are `groups` equal groups of neighbours, a group's score is
+// the largest score + correction in it, and only outputs of the best keep_groups groups can be chosen.
 int egpt_moe_route(const void* x, const void* router, const void* bias, int32_t* chosen, float* weight, int n_tokens,
-                   int hidden, int experts, int top, int score_all, const float* correction, float weight_scale, int dtype,
-                   void* stream);
+                   int hidden, int experts, int top, int score_all, const float* correction, float weight_scale, int groups,
+                   int keep_groups, int normalized, int dtype, void* stream);
 // Rows (token, choice) grouped by expert: row_token[n_tokens * top] the token of every grouped row, place[t][top] the
-// grouped row of every (token, choice), tiles[0] the number of row tiles, then per tile (expert, first row, rows).
+// grouped row of every (token, choice) (-1 for a choice of `experts` or above, which has no row), tiles[0] the number of row tiles, then per tile (expert, first row, rows).
 // tile_rows: rows to a tile.  tiles holds 1 + 3 * (n_tokens * top / tile_rows + experts + 1) int32.
 int egpt_moe_group(const int32_t* chosen, int32_t* row_token, int32_t* place, int32_t* tiles, int32_t* counts, int n_tokens,
                    int top, int experts, int tile_rows, void* stream);
@@ -306,15 +315,18 @@ int egpt_moe_up(const void* x, const void* w_up, const int32_t* row_token, const
 // y[row] = act[row] Wd_e^T, float32 [n_tokens * top][hidden]; w_down [experts][hidden][ff].
 int egpt_moe_down(const void* act, const void* w_down, const int32_t* tiles, float* y, int n_rows, int hidden, int ff,
                   int experts, int tile_rows, int dtype, void* stream);
-// out[t] = sum_c weight[t][c] * y[place[t][c]] in the order of the choices, float32 [n_tokens][hidden].
-int egpt_moe_combine(const float* y, const int32_t* place, const float* weight, float* out, int n_tokens, int top, int hidden,
-                     void* stream);
+// out[t] = sum_c weight[t][c] * v_c in the order of the choices with v_c = y[place[t][c]], or x[t] where the place is -1;
+// float32 [n_tokens][hidden], or (out null) added to the fixed-point residual stream.
+int egpt_moe_combine(const float* y, const void* x, const int32_t* place, const float* weight, float* out, void* residual,
+                     int n_tokens, int top, int hidden, int dtype, void* stream);
 // ---- activations.hip: what stands between the two products of a feed-forward without a gate
 // out[t][j] = f(z[t][j]) for the first `cols` columns of a product row of z_width values (one tensor or float32 partial sums):
 // mode 0: relu(z)^2; mode 1: the normed polynomial c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 with N(u) = u / sqrt(mean_j(u_j^2) + eps)
-// over the row's cols values (coef float32 [4]).  gate_col >= 0: times sigmoid(z[t][gate_col]), one number per row.
-int egpt_ff_activation(const void* z, int z_splits, int z_width, int cols, int mode, const float* coef, float eps, int gate_col,
-                       void* out, int n_tokens, int dtype, void* stream);
+// over the row's cols values (coef float32 [4]).  gate_col >= 0: times sigmoid(z[t][gate_col]), one number per row.  row_ss (may
+// be null), ss_splits, hidden, norm_eps: the factor that the product's rows still lack, as in egpt_swiglu.
+int egpt_ff_activation(const void* z, int z_splits, const float* row_ss, int ss_splits, int hidden, float norm_eps, int z_width,
+                       int cols, int mode, const float* coef, float eps, int gate_col, void* out, int n_tokens, int dtype,
+                       void* stream);
 // scratch: n_rows * 32 floats followed by n_rows * 32 int32 (two-stage search for wide vocabularies), or null.
 int egpt_argmax(const float* logits, int32_t* out, void* scratch, int n_rows, int vocab, void* stream);
 // egpt_argmax for callers that cannot allocate device memory and have no workspace to pass (code under graph

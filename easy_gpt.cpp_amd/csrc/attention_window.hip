@@ -1,6 +1,7 @@
 // Softmax attention over the paged cache with separate key and value sizes, a window that keeps the first tokens,
 // a sink in the softmax, a learned bias per head and distance, keys visible only within the query's own block of
-// positions, a penalty per head that grows with the distance, a tanh cap on the scores and a gate per head on the output; ragged batches (prompt portions and single decoded tokens in one launch).
+// positions, a penalty per head that grows with the distance, a tanh cap on the scores, a gate per head on the output, and heads
+// that take the difference of two maps; ragged batches (prompt portions and single decoded tokens in one launch).
 //
 // Query i of request b stands at position p = kv_len[b] - q_len[b] + i and sees key j if j <= p and
 // (window == 0 or p - j < window or j < keep_first).  score = (q . k) * scale over the key size dk; the softmax is
@@ -11,7 +12,10 @@
 // the scaled score s becomes c tanh(s / c) (the sink is not capped); with a head gate [T][nq] a head's output is multiplied by it;
 // the output is the weighted sum of the values of size dv.  Query head h reads key/value head
 // h / (nq / nkv).  Queries q [T][nq][dk]; keys in pages [page][kv head][offset][dk], values in pages
-// [page][kv head][dv][offset]; nothing that is not visible is read, so pages need no clearing and pages that a window
+// [page][kv head][dv][offset].  With maps == 2 a query and a key of size dk are two maps side by side, [map 1 | map 2] of dk / 2
+// each, over the same values: each map is a softmax of its own (a1, a2), the difference a = a1 - map_weight * a2 is divided by its
+// root mean square sqrt(mean(a^2) + out_eps) over the dv features and multiplied by out_scale (no sink, bias, slopes or gate then);
+// every key and value is read once for both maps.  Nothing that is not visible is read, so pages need no clearing and pages that a window
 // gave back are never touched.  Scores, softmax statistics and the output sum are float32.
 #include "api.h"
 #include "common.h"
@@ -84,7 +88,7 @@ __global__ __launch_bounds__(64 * kSimpleWaves) void window_attention_simple_ker
     const int32_t* __restrict__ q_len, const int32_t* __restrict__ kv_len, int n_seqs, int nq, int nkv, int dk, int dv,
     int page_size, float scale, int window, int keep_first, const float* __restrict__ sink,
     const float* __restrict__ dist_bias, int dist_far, int block, const float* __restrict__ slopes, float softcap,
-    const float* __restrict__ head_gate) {
+    const float* __restrict__ head_gate, int maps, float map_weight, float out_scale, float out_eps) {
     constexpr int kMaxOwn = kWidest / kWave;
     __shared__ __attribute__((aligned(16))) float q_s[kWidest];
     __shared__ float part_ml[kSimpleWaves][2];
@@ -101,68 +105,91 @@ __global__ __launch_bounds__(64 * kSimpleWaves) void window_attention_simple_ker
     for (int d = threadIdx.x; d < dk; d += kWave * kSimpleWaves) q_s[d] = to_float(qp[d]);
     __syncthreads();
     const int32_t* table = block_table + static_cast<size_t>(b) * table_width;
-    float acc[kMaxOwn] = {};
-    float m_run = -INFINITY, l_run = 0.f;
-    for (int c = wave * kWave; c < n_visible; c += kWave * kSimpleWaves) {
-        const int vi = c + lane;
-        float s = -INFINITY;
-        if (vi < n_visible) {
-            const int j = vi < n_first ? vi : lo + (vi - n_first);
-            const long page = table[j / page_size];
-            const T* kr = k_cache + ((page * nkv + kvh) * page_size + j % page_size) * dk;
-            s = dot_row(q_s, kr, dk) * scale;
-            if (softcap > 0.f) s = softcap * tanhf(s / softcap);
-            if (dist_bias) s += dist_bias[static_cast<size_t>(h) * (dist_far + 1) + min(p - j, dist_far)];
-            if (slopes) s -= slopes[h] * static_cast<float>(p - j);
-        }
-        const float m_new = fmaxf(m_run, wave_max(s));       // finite: the chunk's first key is visible
-        const float pj = vi < n_visible ? expf(s - m_new) : 0.f;
-        const float alpha = expf(m_run - m_new);             // exp(-inf) = 0 on the wavefront's first chunk
-        l_run = l_run * alpha + wave_sum(pj);
-        m_run = m_new;
+    const int dm = dk / maps;                                // the size of one map's query and key
+    float first_map[kMaxOwn] = {};                           // wavefront 0: the first map's output
+    for (int map = 0; map < maps; ++map) {
+        float acc[kMaxOwn] = {};
+        float m_run = -INFINITY, l_run = 0.f;
+        for (int c = wave * kWave; c < n_visible; c += kWave * kSimpleWaves) {
+            const int vi = c + lane;
+            float s = -INFINITY;
+            if (vi < n_visible) {
+                const int j = vi < n_first ? vi : lo + (vi - n_first);
+                const long page = table[j / page_size];
+                const T* kr = k_cache + ((page * nkv + kvh) * page_size + j % page_size) * dk + map * dm;
+                s = dot_row(q_s + map * dm, kr, dm) * scale;
+                if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+                if (dist_bias) s += dist_bias[static_cast<size_t>(h) * (dist_far + 1) + min(p - j, dist_far)];
+                if (slopes) s -= slopes[h] * static_cast<float>(p - j);
+            }
+            const float m_new = fmaxf(m_run, wave_max(s));       // finite: the chunk's first key is visible
+            const float pj = vi < n_visible ? expf(s - m_new) : 0.f;
+            const float alpha = expf(m_run - m_new);             // exp(-inf) = 0 on the wavefront's first chunk
+            l_run = l_run * alpha + wave_sum(pj);
+            m_run = m_new;
 #pragma unroll
-        for (int r = 0; r < kMaxOwn; ++r) acc[r] *= alpha;
-        const int n_valid = min(kWave, n_visible - c);
-        for (int jj = 0; jj < n_valid; ++jj) {
-            const float pw = lane_value(pj, jj);
-            const int vj = c + jj;
-            const int j = vj < n_first ? vj : lo + (vj - n_first);
-            const long page = table[j / page_size];
-            const T* vr = v_cache + (page * nkv + kvh) * dv * page_size + j % page_size;
+            for (int r = 0; r < kMaxOwn; ++r) acc[r] *= alpha;
+            const int n_valid = min(kWave, n_visible - c);
+            for (int jj = 0; jj < n_valid; ++jj) {
+                const float pw = lane_value(pj, jj);
+                const int vj = c + jj;
+                const int j = vj < n_first ? vj : lo + (vj - n_first);
+                const long page = table[j / page_size];
+                const T* vr = v_cache + (page * nkv + kvh) * dv * page_size + j % page_size;
+#pragma unroll
+                for (int r = 0; r < kMaxOwn; ++r) {
+                    const int d = lane + r * kWave;
+                    if (d < dv) acc[r] = fmaf(pw, to_float(vr[static_cast<long>(d) * page_size]), acc[r]);
+                }
+            }
+        }
+        if (lane == 0) {
+            part_ml[wave][0] = m_run;
+            part_ml[wave][1] = l_run;
+        }
+#pragma unroll
+        for (int r = 0; r < kMaxOwn; ++r) {
+            const int d = lane + r * kWave;
+            if (d < dv) part_o[wave][d] = acc[r];
+        }
+        __syncthreads();
+        if (wave != 0) {
+            __syncthreads();                                     // (wavefront 0 has read the parts)
+            continue;
+        }
+        // wavefront 0 holds the first chunk, so the overall maximum is finite; a wavefront without keys has maximum -inf
+        // and weight exp(-inf) = 0
+        float m_all = sink ? sink[h] : -INFINITY;
+        for (int w = 0; w < kSimpleWaves; ++w) m_all = fmaxf(m_all, part_ml[w][0]);
+        float l_all = sink ? expf(sink[h] - m_all) : 0.f;
+        for (int w = 0; w < kSimpleWaves; ++w) l_all = fmaf(part_ml[w][1], expf(part_ml[w][0] - m_all), l_all);
+        const float inv_l = (head_gate ? head_gate[static_cast<size_t>(t) * nq + h] : 1.0f) / l_all;
+        T* o = out + (static_cast<size_t>(t) * nq + h) * dv;
+        float ss = 0.f;
+#pragma unroll
+        for (int r = 0; r < kMaxOwn; ++r) {
+            const int d = lane + r * kWave;
+            if (d < dv) {
+                float a = 0.f;
+                for (int w = 0; w < kSimpleWaves; ++w) a = fmaf(part_o[w][d], expf(part_ml[w][0] - m_all), a);
+                a *= inv_l;
+                if (maps == 1) {
+                    o[d] = from_float<T>(a);
+                } else {
+                    first_map[r] = map == 0 ? a : first_map[r] - map_weight * a;
+                    ss = fmaf(first_map[r], first_map[r], ss);
+                }
+            }
+        }
+        if (maps == 2 && map == 1) {
+            const float f = out_scale * inv_rms(wave_sum(ss), 1.0f / static_cast<float>(dv), out_eps);
 #pragma unroll
             for (int r = 0; r < kMaxOwn; ++r) {
                 const int d = lane + r * kWave;
-                if (d < dv) acc[r] = fmaf(pw, to_float(vr[static_cast<long>(d) * page_size]), acc[r]);
+                if (d < dv) o[d] = from_float<T>(first_map[r] * f);
             }
         }
-    }
-    if (lane == 0) {
-        part_ml[wave][0] = m_run;
-        part_ml[wave][1] = l_run;
-    }
-#pragma unroll
-    for (int r = 0; r < kMaxOwn; ++r) {
-        const int d = lane + r * kWave;
-        if (d < dv) part_o[wave][d] = acc[r];
-    }
-    __syncthreads();
-    if (wave != 0) return;
-    // wavefront 0 holds the first chunk, so the overall maximum is finite; a wavefront without keys has maximum -inf
-    // and weight exp(-inf) = 0
-    float m_all = sink ? sink[h] : -INFINITY;
-    for (int w = 0; w < kSimpleWaves; ++w) m_all = fmaxf(m_all, part_ml[w][0]);
-    float l_all = sink ? expf(sink[h] - m_all) : 0.f;
-    for (int w = 0; w < kSimpleWaves; ++w) l_all = fmaf(part_ml[w][1], expf(part_ml[w][0] - m_all), l_all);
-    const float inv_l = (head_gate ? head_gate[static_cast<size_t>(t) * nq + h] : 1.0f) / l_all;
-    T* o = out + (static_cast<size_t>(t) * nq + h) * dv;
-#pragma unroll
-    for (int r = 0; r < kMaxOwn; ++r) {
-        const int d = lane + r * kWave;
-        if (d < dv) {
-            float a = 0.f;
-            for (int w = 0; w < kSimpleWaves; ++w) a = fmaf(part_o[w][d], expf(part_ml[w][0] - m_all), a);
-            o[d] = from_float<T>(a * inv_l);
-        }
+        __syncthreads();
     }
 }
 
@@ -184,6 +211,9 @@ __global__ __launch_bounds__(64 * kSimpleWaves) void window_attention_simple_ker
 // chunks of a workgroup's rows are dealt over as many workgroups (grid z), which leave unnormalised results
 // part_o [split][token][head][dv] and (maximum, sum) part_ml [split][token][head][2] that window_attention_fold_kernel
 // combines; that kernel also adds the sink.  With one split the kernel finishes the rows itself.
+// With two maps to a head (MAPS) a wavefront's tiles come in pairs: tile 2 u is the first map of the 16 rows of pair u, tile
+// 2 u + 1 their second.  A map reads its own half of the query and key rows, which start on whole pieces in LDS; the values'
+// operands serve both.  The parts of a split are then [split][token][head][map].
 typedef __attribute__((ext_vector_type(8))) __bf16 w_bf16x8;
 typedef __attribute__((ext_vector_type(4))) float w_f32x4;
 typedef __attribute__((ext_vector_type(4))) unsigned int w_u32x4;
@@ -249,6 +279,8 @@ struct WindowArgs {
     const float* head_gate;  // [n_tokens][nq] or null: factors on the heads' outputs
     float softcap;           // > 0: scores become softcap * tanh(score / softcap)
     int block;               // keys are seen within the query's block of this many positions (0: no blocks)
+    int maps;                // softmax maps to a head: 1, or 2 whose difference is the head's output
+    float map_weight, out_scale, out_eps;
     int table_width, n_seqs, n_tokens, nq, nkv, dk, dv, page_size, window, keep_first, n_splits;
     int page_shift;          // log2 of the page size if that is a power of two, else -1
     float scale;
@@ -261,15 +293,16 @@ __device__ __forceinline__ int place_in_page(int key, int page_size, int page_sh
     return page_shift >= 0 ? key & (page_size - 1) : key % page_size;
 }
 
-// CAPPED: scores pass the tanh cap (and get neither a bias table nor slopes).
-template <typename T, int DT, int RT, int RW, bool CAPPED>
+// CAPPED: scores pass the tanh cap (and get neither a bias table nor slopes).  MAPS: softmax maps to a head (1 or 2).
+template <typename T, int DT, int RT, int RW, int MAPS, bool CAPPED>
 __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attention_tiled_kernel(WindowArgs a) {
     constexpr int E = 16 / sizeof(T);             // elements in 16 bytes
     constexpr int KT = sizeof(T) == 2 ? 64 : 32;  // keys per chunk
     constexpr int NKT = KT / 16;                  // tiles of 16 keys in a chunk
     constexpr int PF = 4 * E;                     // features (or keys) that one matrix_piece sums over
     constexpr int NP = KT / PF;                   // pieces of a chunk's keys
-    constexpr int ROWS = 16 * RT * RW, THREADS = 64 * RT;     // a wavefront takes RW tiles of 16 rows
+    constexpr int TILES = RW / MAPS;              // tiles of 16 rows to a wavefront; RW tiles of scores, one per map
+    constexpr int ROWS = 16 * RT * TILES, THREADS = 64 * RT;
     constexpr int VROW = KT + E;                  // padded LDS row of values (elements)
     constexpr int U = 8;                          // loads that a thread has in flight while the queries are staged
     constexpr int KU = 8;                         // 16-byte pieces of a chunk's keys per thread: 64 keys of 256 features
@@ -280,8 +313,10 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     const T* __restrict__ v_cache = static_cast<const T*>(a.v_cache);
     const int dk = a.dk, dv = a.dv, nq = a.nq, nkv = a.nkv, page_size = a.page_size, window = a.window;
     const int page_shift = a.page_shift;
-    const int n_pieces = (dk + PF - 1) / PF;
-    const int krow = n_pieces * PF + E;           // padded LDS row of keys and of queries
+    const int dm = dk / MAPS;                     // the size of one map's query and key
+    const int n_pieces = (dm + PF - 1) / PF;
+    const int mrow = n_pieces * PF;               // its padded place in an LDS row
+    const int krow = MAPS * mrow + E;             // padded LDS row of keys and of queries
     const int k_pieces = dk / E;                  // 16-byte pieces of a key
     T* q_s = reinterpret_cast<T*>(window_smem);
     T* k_s = q_s + ROWS * krow;
@@ -316,11 +351,11 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     const int c_begin = blockIdx.z * per_split, c_end = min(n_chunks, c_begin + per_split);
 
     // this wavefront's tiles of 16 rows, this lane's row in each
-    bool valid[RW];
-    int tok[RW], head[RW], p_row[RW], lo_row[RW];
+    bool valid[TILES];
+    int tok[TILES], head[TILES], p_row[TILES], lo_row[TILES];
 #pragma unroll
-    for (int w = 0; w < RW; ++w) {
-        const int r = blk_first + (wave * RW + w) * 16 + lj;
+    for (int w = 0; w < TILES; ++w) {
+        const int r = blk_first + (wave * TILES + w) * 16 + lj;
         valid[w] = r < rows;
         const int i_tok = valid[w] ? r / group_size : 0;
         tok[w] = qs + i_tok;
@@ -330,9 +365,9 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     }
 
     // the smallest position and the largest window start among a tile's rows (rows of no token aside)
-    int tile_p_min[RW], tile_lo_max[RW];
+    int tile_p_min[TILES], tile_lo_max[TILES];
 #pragma unroll
-    for (int w = 0; w < RW; ++w) {
+    for (int w = 0; w < TILES; ++w) {
         int pm = valid[w] ? p_row[w] : 0x7fffffff, lm = valid[w] ? lo_row[w] : 0;
 #pragma unroll
         for (int off = kWave / 2; off > 0; off >>= 1) {
@@ -347,6 +382,15 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     // value rows beyond the value size are zeroed once, the chunks never write there
     {
         const int pieces = krow / E;
+        // which element of a query or key lies at `place` of an LDS row (-1: a pad)
+        auto row_source = [&](int place) {
+            if constexpr (MAPS == 1) {
+                return place < dk ? place : -1;
+            } else {
+                const int m = place >= mrow ? 1 : 0, within = place - m * mrow;
+                return within < dm ? m * dm + within : -1;
+            }
+        };
         for (int base = tid; base < ROWS * pieces; base += THREADS * U) {
             w_u32x4 regs[U];
 #pragma unroll
@@ -355,9 +399,10 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
                 const int row = idx / pieces, c = idx % pieces;
                 const int rr = blk_first + row;
                 regs[u] = w_u32x4{0u, 0u, 0u, 0u};
-                if (idx < ROWS * pieces && rr < rows && c * E < dk) {
+                const int from = row_source(c * E);
+                if (idx < ROWS * pieces && rr < rows && from >= 0) {
                     const int t2 = qs + rr / group_size, h2 = kh * group_size + rr % group_size;
-                    regs[u] = *reinterpret_cast<const w_u32x4*>(q + (static_cast<size_t>(t2) * nq + h2) * dk + c * E);
+                    regs[u] = *reinterpret_cast<const w_u32x4*>(q + (static_cast<size_t>(t2) * nq + h2) * dk + from);
                 }
             }
 #pragma unroll
@@ -366,9 +411,15 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
                 if (idx < ROWS * pieces) *reinterpret_cast<w_u32x4*>(q_s + (idx / pieces) * krow + (idx % pieces) * E) = regs[u];
             }
         }
-        for (int idx = tid; idx < KT * (pieces - k_pieces); idx += THREADS)
-            *reinterpret_cast<w_u32x4*>(k_s + (idx / (pieces - k_pieces)) * krow + (k_pieces + idx % (pieces - k_pieces)) * E) =
-                w_u32x4{0u, 0u, 0u, 0u};
+        if constexpr (MAPS == 1) {
+            for (int idx = tid; idx < KT * (pieces - k_pieces); idx += THREADS)
+                *reinterpret_cast<w_u32x4*>(k_s + (idx / (pieces - k_pieces)) * krow + (k_pieces + idx % (pieces - k_pieces)) * E) =
+                    w_u32x4{0u, 0u, 0u, 0u};
+        } else {
+            for (int idx = tid; idx < KT * pieces; idx += THREADS)
+                if (row_source((idx % pieces) * E) < 0)
+                    *reinterpret_cast<w_u32x4*>(k_s + (idx / pieces) * krow + (idx % pieces) * E) = w_u32x4{0u, 0u, 0u, 0u};
+        }
         constexpr int VPIECES = VROW / E;
         for (int idx = tid; idx < DT * 16 * VPIECES; idx += THREADS)
             if (idx / VPIECES >= dv) *reinterpret_cast<w_u32x4*>(v_s + (idx / VPIECES) * VROW + (idx % VPIECES) * E) = w_u32x4{0u, 0u, 0u, 0u};
@@ -385,7 +436,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     }
     const float scale = a.scale;
     constexpr float kLog2e = 1.4426950408889634f;
-    const bool wave_active = blk_first + wave * RW * 16 < rows;      // a wavefront without rows only helps to stage
+    const bool wave_active = blk_first + wave * TILES * 16 < rows;      // a wavefront without rows only helps to stage
 
     // A chunk's keys [KT][dk] and values, transposed [dv][KT], travel through registers: the loads of the chunk after
     // this one are issued before this one's products and stored to LDS behind them.  What no row of the workgroup sees
@@ -403,7 +454,8 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
         const int idx = tid + u * THREADS;
         const bool used = idx < k_total;
         k_row[u] = used ? idx / k_pieces : -(1 << 28);          // (a key no chunk holds)
-        k_lds[u] = used ? (idx / k_pieces) * krow + (idx % k_pieces) * E : 0;
+        const int place = (idx % k_pieces) * E;
+        k_lds[u] = used ? (idx / k_pieces) * krow + (MAPS == 2 && place >= dm ? mrow + place - dm : place) : 0;
         k_off[u] = kh * page_size * dk + (used ? (idx % k_pieces) * E : 0);
     }
     int v_key[VU], v_lds[VU];
@@ -506,7 +558,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
         // ---- scores of this wavefront's rows against the chunk's keys: a key operand serves all of its row tiles
         w_f32x4 acc[RW][NKT];
         const T* ks = k_s + lj * krow + lg * E;
-        const T* qrow = q_s + (wave * RW * 16 + lj) * krow + lg * E;
+        const T* qrow = q_s + (wave * TILES * 16 + lj) * krow + lg * E;
 #pragma unroll
         for (int w = 0; w < RW; ++w)
 #pragma unroll
@@ -514,12 +566,16 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
         for (int j = 0; j < n_pieces; ++j) {
             w_u32x4 qv[RW];
 #pragma unroll
-            for (int w = 0; w < RW; ++w) qv[w] = *reinterpret_cast<const w_u32x4*>(qrow + w * 16 * krow + j * PF);
+            for (int w = 0; w < RW; ++w)
+                qv[w] = *reinterpret_cast<const w_u32x4*>(qrow + (w / MAPS) * 16 * krow + (w % MAPS) * mrow + j * PF);
 #pragma unroll
             for (int kt = 0; kt < NKT; ++kt) {
-                const w_u32x4 kvv = *reinterpret_cast<const w_u32x4*>(ks + kt * 16 * krow + j * PF);
 #pragma unroll
-                for (int w = 0; w < RW; ++w) acc[w][kt] = matrix_piece<T>(kvv, qv[w], acc[w][kt]);
+                for (int m = 0; m < MAPS; ++m) {
+                    const w_u32x4 kvv = *reinterpret_cast<const w_u32x4*>(ks + kt * 16 * krow + m * mrow + j * PF);
+#pragma unroll
+                    for (int w = m; w < RW; w += MAPS) acc[w][kt] = matrix_piece<T>(kvv, qv[w], acc[w][kt]);
+                }
             }
         }
         matrix_results_ready();
@@ -530,7 +586,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
             float mx = -INFINITY;
             // a chunk that every row of the tile sees whole (below the diagonal and inside the window, or all kept
             // tokens) needs no mask
-            const bool whole = key0 + KT - 1 <= tile_p_min[w] && (key0 >= tile_lo_max[w] || key0 + KT <= a.keep_first);
+            const bool whole = key0 + KT - 1 <= tile_p_min[w / MAPS] && (key0 >= tile_lo_max[w / MAPS] || key0 + KT <= a.keep_first);
             if constexpr (CAPPED) {
                 const float inner = scale / a.softcap;
 #pragma unroll
@@ -538,7 +594,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
 #pragma unroll
                     for (int v = 0; v < 4; ++v) {
                         const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = whole || (key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first));
+                        const bool seen = whole || (key <= p_row[w / MAPS] && (key >= lo_row[w / MAPS] || key < a.keep_first));
                         const float sc = seen ? a.softcap * bounded_tanh<T>(acc[w][kt][v] * inner) : -INFINITY;
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
@@ -546,31 +602,31 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
             } else if (a.dist_bias != nullptr) {
                 // the bias of the row's head by distance; a chunk that lies `far` or more behind every row of the tile
                 // gets the table's last entry throughout
-                const float* brow = a.dist_bias + static_cast<size_t>(head[w]) * (a.dist_far + 1);
-                const bool all_far = whole && tile_p_min[w] - (key0 + KT - 1) >= a.dist_far;
+                const float* brow = a.dist_bias + static_cast<size_t>(head[w / MAPS]) * (a.dist_far + 1);
+                const bool all_far = whole && tile_p_min[w / MAPS] - (key0 + KT - 1) >= a.dist_far;
                 const float b_far = brow[a.dist_far];
 #pragma unroll
                 for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
                     for (int v = 0; v < 4; ++v) {
                         const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first);
+                        const bool seen = key <= p_row[w / MAPS] && (key >= lo_row[w / MAPS] || key < a.keep_first);
                         float sc = -INFINITY;
                         if (all_far) sc = fmaf(acc[w][kt][v], scale, b_far);
-                        else if (seen) sc = fmaf(acc[w][kt][v], scale, brow[min(p_row[w] - key, a.dist_far)]);
+                        else if (seen) sc = fmaf(acc[w][kt][v], scale, brow[min(p_row[w / MAPS] - key, a.dist_far)]);
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
                     }
             } else if (a.slopes != nullptr) {
                 // the penalty of the row's head times the distance
-                const float slope = a.slopes[head[w]];
+                const float slope = a.slopes[head[w / MAPS]];
 #pragma unroll
                 for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
                     for (int v = 0; v < 4; ++v) {
                         const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = whole || (key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first));
-                        const float sc = seen ? fmaf(acc[w][kt][v], scale, -slope * static_cast<float>(p_row[w] - key)) : -INFINITY;
+                        const bool seen = whole || (key <= p_row[w / MAPS] && (key >= lo_row[w / MAPS] || key < a.keep_first));
+                        const float sc = seen ? fmaf(acc[w][kt][v], scale, -slope * static_cast<float>(p_row[w / MAPS] - key)) : -INFINITY;
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
                     }
@@ -588,7 +644,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
 #pragma unroll
                     for (int v = 0; v < 4; ++v) {
                         const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first);
+                        const bool seen = key <= p_row[w / MAPS] && (key >= lo_row[w / MAPS] || key < a.keep_first);
                         const float sc = seen ? acc[w][kt][v] * scale : -INFINITY;
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
@@ -645,34 +701,71 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
             }
     }
     matrix_results_ready();
+    float l_sum[RW];
 #pragma unroll
     for (int w = 0; w < RW; ++w) {
-        float l = l_run[w];
-        l += __shfl_xor(l, 16, kWave);
-        l += __shfl_xor(l, 32, kWave);
-        if (!valid[w]) continue;
-        if (a.n_splits > 1) {
-            const size_t row_at = (static_cast<size_t>(blockIdx.z) * a.n_tokens + tok[w]) * nq + head[w];
+        l_sum[w] = l_run[w];
+        l_sum[w] += __shfl_xor(l_sum[w], 16, kWave);
+        l_sum[w] += __shfl_xor(l_sum[w], 32, kWave);
+    }
+    if (a.n_splits > 1) {
+#pragma unroll
+        for (int w = 0; w < RW; ++w) {
+            const int u = w / MAPS;
+            if (!valid[u]) continue;
+            const size_t row_at = ((static_cast<size_t>(blockIdx.z) * a.n_tokens + tok[u]) * nq + head[u]) * MAPS + w % MAPS;
             float* po = a.part_o + row_at * dv + lg * 4;
 #pragma unroll
             for (int d = 0; d < DT; ++d)
                 if (d * 16 < dv) *reinterpret_cast<float4*>(po + d * 16) = float4{o[w][d][0], o[w][d][1], o[w][d][2], o[w][d][3]};
             if (lg == 0) {
                 a.part_ml[row_at * 2] = m_run[w];
-                a.part_ml[row_at * 2 + 1] = l;
+                a.part_ml[row_at * 2 + 1] = l_sum[w];
             }
-            continue;
         }
+        return;
+    }
+    if constexpr (MAPS == 2) {
+        // the difference of the two maps, divided by its root mean square (a row's four lanes hold its features; those
+        // beyond dv are zero)
+#pragma unroll
+        for (int u = 0; u < TILES; ++u) {
+            const float f1 = valid[u] ? 1.0f / l_sum[2 * u] : 0.f, f2 = valid[u] ? a.map_weight / l_sum[2 * u + 1] : 0.f;
+            float ss = 0.f;
+#pragma unroll
+            for (int d = 0; d < DT; ++d)
+#pragma unroll
+                for (int v = 0; v < 4; ++v) {
+                    const float x = o[2 * u][d][v] * f1 - o[2 * u + 1][d][v] * f2;
+                    o[2 * u][d][v] = x;
+                    ss = fmaf(x, x, ss);
+                }
+            ss += __shfl_xor(ss, 16, kWave);
+            ss += __shfl_xor(ss, 32, kWave);
+            const float f = a.out_scale * inv_rms(ss, 1.0f / static_cast<float>(dv), a.out_eps);
+            if (!valid[u]) continue;
+            T* op = static_cast<T*>(a.out) + (static_cast<size_t>(tok[u]) * nq + head[u]) * dv + lg * 4;
+#pragma unroll
+            for (int d = 0; d < DT; ++d)
+                if (d * 16 < dv)
+                    store_four<T>(op + d * 16, o[2 * u][d][0] * f, o[2 * u][d][1] * f, o[2 * u][d][2] * f, o[2 * u][d][3] * f);
+        }
+        return;
+    }
+#pragma unroll
+    for (int w = 0; w < RW; ++w) {
+        if (!valid[w / MAPS]) continue;
+        float l = l_sum[w];
         float weight = 1.0f;
         if (a.sink != nullptr) {
-            const float sk = a.sink[head[w]];
+            const float sk = a.sink[head[w / MAPS]];
             const float m_all = fmaxf(m_run[w], sk);
             weight = __builtin_amdgcn_exp2f((m_run[w] - m_all) * kLog2e);
             l = l * weight + __builtin_amdgcn_exp2f((sk - m_all) * kLog2e);
         }
         float inv = weight / l;
-        if (a.head_gate != nullptr) inv *= a.head_gate[static_cast<size_t>(tok[w]) * nq + head[w]];
-        T* op = static_cast<T*>(a.out) + (static_cast<size_t>(tok[w]) * nq + head[w]) * dv + lg * 4;
+        if (a.head_gate != nullptr) inv *= a.head_gate[static_cast<size_t>(tok[w / MAPS]) * nq + head[w / MAPS]];
+        T* op = static_cast<T*>(a.out) + (static_cast<size_t>(tok[w / MAPS]) * nq + head[w / MAPS]) * dv + lg * 4;
 #pragma unroll
         for (int d = 0; d < DT; ++d)
             if (d * 16 < dv)
@@ -712,13 +805,56 @@ __global__ __launch_bounds__(kWave) void window_attention_fold_kernel(const floa
     }
 }
 
-template <typename T, int DT, int RT, int RW, bool CAPPED>
+// The same for heads of two maps: both maps' parts are folded, and their difference is divided by its root mean square.
+template <typename T>
+__global__ __launch_bounds__(kWave) void window_attention_fold_maps_kernel(const float* __restrict__ part_o,
+                                                                         const float* __restrict__ part_ml, float map_weight,
+                                                                         float out_scale, float out_eps, T* __restrict__ out,
+                                                                         int n_rows, int dv, int n_splits) {
+    constexpr int kOwn = 256 / kWave;          // features of a row that a lane holds (dv <= 256)
+    __shared__ float weights[2][kWave];        // at most 64 splits
+    const int row = blockIdx.x, lane = threadIdx.x;
+#pragma unroll
+    for (int map = 0; map < 2; ++map) {
+        float m = -INFINITY, l = 0.f;
+        if (lane < n_splits) {
+            const float* ml = part_ml + ((static_cast<size_t>(lane) * n_rows + row) * 2 + map) * 2;
+            m = ml[0];
+            l = ml[1];
+        }
+        const float m_all = wave_max(m);
+        const float w = lane < n_splits ? expf(m - m_all) : 0.f;     // exp(-inf) = 0 for a split that saw nothing
+        weights[map][lane] = w / wave_sum(l * w) * (map == 0 ? 1.0f : -map_weight);
+    }
+    __syncthreads();
+    float acc[kOwn] = {};
+    for (int s = 0; s < n_splits; ++s) {
+        const float* po = part_o + (static_cast<size_t>(s) * n_rows + row) * 2 * dv;
+        const float w1 = weights[0][s], w2 = weights[1][s];
+#pragma unroll
+        for (int r = 0; r < kOwn; ++r) {
+            const int d = lane + r * kWave;
+            if (d < dv) acc[r] = fmaf(po[dv + d], w2, fmaf(po[d], w1, acc[r]));
+        }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int r = 0; r < kOwn; ++r) ss = fmaf(acc[r], acc[r], ss);
+    const float f = out_scale * inv_rms(wave_sum(ss), 1.0f / static_cast<float>(dv), out_eps);
+#pragma unroll
+    for (int r = 0; r < kOwn; ++r) {
+        const int d = lane + r * kWave;
+        if (d < dv) out[static_cast<size_t>(row) * dv + d] = from_float<T>(acc[r] * f);
+    }
+}
+
+template <typename T, int DT, int RT, int RW, int MAPS, bool CAPPED>
 static int launch_tiled(const WindowArgs& a, int max_rows, hipStream_t s) {
-    constexpr int E = 16 / sizeof(T), KT = sizeof(T) == 2 ? 64 : 32, PF = 4 * E, ROWS = 16 * RT * RW;
-    const int krow = (a.dk + PF - 1) / PF * PF + E;
+    constexpr int E = 16 / sizeof(T), KT = sizeof(T) == 2 ? 64 : 32, PF = 4 * E, ROWS = 16 * RT * (RW / MAPS);
+    const int krow = MAPS * ((a.dk / MAPS + PF - 1) / PF * PF) + E;
     const size_t lds = (static_cast<size_t>(ROWS + KT) * krow + static_cast<size_t>(DT) * 16 * (KT + E)) * sizeof(T);
     if (lds > 160 * 1024) return EGPT_UNSUPPORTED_SIZE;
-    auto kernel = window_attention_tiled_kernel<T, DT, RT, RW, CAPPED>;
+    auto kernel = window_attention_tiled_kernel<T, DT, RT, RW, MAPS, CAPPED>;
     if (lds > 48 * 1024) {
         static bool raised = false;       // per instance of this template: the limit is asked for once
         if (!raised) {
@@ -738,12 +874,22 @@ static int launch_tiled(const WindowArgs& a, int max_rows, hipStream_t s) {
 // row_tiles: 4 (four wavefronts with 16 rows each) or 8 (with 32 rows each)
 template <typename T, int DT>
 static int launch_tiled_for_rows(const WindowArgs& a, int max_rows, int row_tiles, hipStream_t s) {
-    if (a.softcap > 0.f) {
-        if (row_tiles == 8) return launch_tiled<T, DT, 4, 2, true>(a, max_rows, s);
-        return launch_tiled<T, DT, 4, 1, true>(a, max_rows, s);
+    if (a.maps == 2) {
+        if (row_tiles == 8) return EGPT_UNSUPPORTED_SIZE;
+        if (a.softcap > 0.f) return launch_tiled<T, DT, 4, 2, 2, true>(a, max_rows, s);
+        return launch_tiled<T, DT, 4, 2, 2, false>(a, max_rows, s);
     }
-    if (row_tiles == 8) return launch_tiled<T, DT, 4, 2, false>(a, max_rows, s);
-    return launch_tiled<T, DT, 4, 1, false>(a, max_rows, s);
+    if (a.softcap > 0.f) {
+        if (row_tiles == 8) return launch_tiled<T, DT, 4, 2, 1, true>(a, max_rows, s);
+        return launch_tiled<T, DT, 4, 1, 1, true>(a, max_rows, s);
+    }
+    if (row_tiles == 8) return launch_tiled<T, DT, 4, 2, 1, false>(a, max_rows, s);
+    return launch_tiled<T, DT, 4, 1, 1, false>(a, max_rows, s);
+}
+
+// what heads of two maps go together with
+static bool maps_fit(int maps, int dk, const float* sink, const float* dist_bias, const float* slopes, const float* head_gate) {
+    return maps == 1 || (maps == 2 && dk % 2 == 0 && !sink && !dist_bias && !slopes && !head_gate);
 }
 
 template <typename T>
@@ -767,11 +913,12 @@ extern "C" int egpt_window_attention(const void* q, void* out, const void* k_cac
                                      const int32_t* q_len, const int32_t* kv_len, int n_seqs, int n_tokens, int nq,
                                      int nkv, int dk, int dv, int page_size, float scale, int window, int keep_first,
                                      const float* sink, const float* dist_bias, int dist_far, int block, const float* slopes,
-                                     float softcap, const float* head_gate, int dtype, void* stream) {
+                                     float softcap, const float* head_gate, int maps, float map_weight, float out_scale,
+                                     float out_eps, int dtype, void* stream) {
     if (!q || !out || !k_cache || !v_cache || !block_table || !q_start || !q_len || !kv_len) return EGPT_BAD_ARGUMENT;
     if (n_seqs <= 0 || n_tokens < 0 || nq <= 0 || nkv <= 0 || nq % nkv != 0 || dk <= 0 || dv <= 0 || page_size <= 0 ||
         table_width <= 0 || window < 0 || keep_first < 0 || (dtype != 0 && dtype != 1) || (dist_bias && dist_far < 0) || block < 0 ||
-        !(softcap >= 0.f) || (softcap > 0.f && (dist_bias || slopes)))
+        !(softcap >= 0.f) || (softcap > 0.f && (dist_bias || slopes)) || !maps_fit(maps, dk, sink, dist_bias, slopes, head_gate))
         return EGPT_BAD_ARGUMENT;
     if (dk > kWidest || dv > kWidest || nq > 65535) return EGPT_UNSUPPORTED_SIZE;
     if (n_tokens == 0) return EGPT_OK;
@@ -781,12 +928,14 @@ extern "C" int egpt_window_attention(const void* q, void* out, const void* k_cac
         window_attention_simple_kernel<float><<<grid, kWave * kSimpleWaves, 0, s>>>(
             static_cast<const float*>(q), static_cast<float*>(out), static_cast<const float*>(k_cache),
             static_cast<const float*>(v_cache), block_table, table_width, q_start, q_len, kv_len, n_seqs, nq, nkv, dk,
-            dv, page_size, scale, window, keep_first, sink, dist_bias, dist_far, block, slopes, softcap, head_gate);
+            dv, page_size, scale, window, keep_first, sink, dist_bias, dist_far, block, slopes, softcap, head_gate, maps, map_weight,
+            out_scale, out_eps);
     else
         window_attention_simple_kernel<bf16_t><<<grid, kWave * kSimpleWaves, 0, s>>>(
             static_cast<const bf16_t*>(q), static_cast<bf16_t*>(out), static_cast<const bf16_t*>(k_cache),
             static_cast<const bf16_t*>(v_cache), block_table, table_width, q_start, q_len, kv_len, n_seqs, nq, nkv, dk,
-            dv, page_size, scale, window, keep_first, sink, dist_bias, dist_far, block, slopes, softcap, head_gate);
+            dv, page_size, scale, window, keep_first, sink, dist_bias, dist_far, block, slopes, softcap, head_gate, maps, map_weight,
+            out_scale, out_eps);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }
@@ -797,16 +946,17 @@ extern "C" int egpt_window_attention_tiled(const void* q, void* out, float* part
                                            int n_tokens, int nq, int nkv, int dk, int dv, int page_size, float scale,
                                            int window, int keep_first, const float* sink, const float* dist_bias,
                                            int dist_far, int block, const float* slopes, float softcap, const float* head_gate,
-                                           int n_splits, int row_tiles, int dtype, void* stream) {
+                                           int maps, float map_weight, float out_scale, float out_eps, int n_splits,
+                                           int row_tiles, int dtype, void* stream) {
     if (!q || !out || !k_cache || !v_cache || !block_table || !q_start || !q_len || !kv_len) return EGPT_BAD_ARGUMENT;
     if (n_seqs <= 0 || n_tokens < 0 || nq <= 0 || nkv <= 0 || nq % nkv != 0 || dk <= 0 || dv <= 0 || page_size <= 0 ||
         table_width <= 0 || window < 0 || keep_first < 0 || n_splits < 1 || (dtype != 0 && dtype != 1) ||
         (row_tiles != 4 && row_tiles != 8) || (dist_bias && dist_far < 0) || block < 0 || (dist_bias && slopes) ||
-        !(softcap >= 0.f) || (softcap > 0.f && (dist_bias || slopes)))
+        !(softcap >= 0.f) || (softcap > 0.f && (dist_bias || slopes)) || !maps_fit(maps, dk, sink, dist_bias, slopes, head_gate))
         return EGPT_BAD_ARGUMENT;
     if (n_splits > 1 && (!part_o || !part_ml)) return EGPT_BAD_ARGUMENT;
     const int e = dtype == 0 ? 4 : 8;
-    if (dk % e || dk > 256 || dv % 16 || dv > 256 || page_size % 16 || nkv > 65535 || n_splits > 64) return EGPT_UNSUPPORTED_SIZE;
+    if (dk % (e * maps) || dk > 256 || dv % 16 || dv > 256 || page_size % 16 || nkv > 65535 || n_splits > 64) return EGPT_UNSUPPORTED_SIZE;
     if (n_tokens == 0) return EGPT_OK;
     hipStream_t s = static_cast<hipStream_t>(stream);
     WindowArgs a;
@@ -814,6 +964,7 @@ extern "C" int egpt_window_attention_tiled(const void* q, void* out, float* part
     a.block_table = block_table; a.q_start = q_start; a.q_len = q_len; a.kv_len = kv_len; a.sink = sink;
     a.dist_bias = dist_bias; a.dist_far = dist_far; a.slopes = slopes; a.block = block;
     a.softcap = softcap; a.head_gate = head_gate;
+    a.maps = maps; a.map_weight = map_weight; a.out_scale = out_scale; a.out_eps = out_eps;
     a.table_width = table_width; a.n_seqs = n_seqs; a.n_tokens = n_tokens; a.nq = nq; a.nkv = nkv; a.dk = dk; a.dv = dv;
     a.page_size = page_size; a.window = window; a.keep_first = keep_first; a.n_splits = n_splits; a.scale = scale;
     a.page_shift = -1;
@@ -826,7 +977,15 @@ extern "C" int egpt_window_attention_tiled(const void* q, void* out, float* part
         code = launch_tiled_for_dv<bf16_t>(a, n_tokens, row_tiles, s);
     if (code != EGPT_OK) return code;
     EGPT_CHECK_LAUNCH();
-    if (n_splits > 1) {
+    if (n_splits > 1 && maps == 2) {
+        if (dtype == 0)
+            window_attention_fold_maps_kernel<float><<<n_tokens * nq, kWave, 0, s>>>(
+                part_o, part_ml, map_weight, out_scale, out_eps, static_cast<float*>(out), n_tokens * nq, dv, n_splits);
+        else
+            window_attention_fold_maps_kernel<bf16_t><<<n_tokens * nq, kWave, 0, s>>>(
+                part_o, part_ml, map_weight, out_scale, out_eps, static_cast<bf16_t*>(out), n_tokens * nq, dv, n_splits);
+        EGPT_CHECK_LAUNCH();
+    } else if (n_splits > 1) {
         if (dtype == 0)
             window_attention_fold_kernel<float><<<n_tokens * nq, kWave, 0, s>>>(part_o, part_ml, sink, head_gate, static_cast<float*>(out),
                                                                                n_tokens * nq, nq, dv, n_splits);

@@ -45,6 +45,7 @@ __device__ __forceinline__ void rotate_pair(float a, float b, float c, float s, 
 // The activation of a gated feed-forward's gate: 0 silu, z / (1 + exp(-z)); 1 the tanh form of gelu,
 // z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), which is z / (1 + exp(-2 sqrt(2 / pi) (z + 0.044715 z^3))).
 constexpr int kGateSilu = 0, kGateGeluTanh = 1;
+constexpr int kUngatedRelu2 = 2;         // no gate: the square of relu (where a product can begin with either)
 __device__ __forceinline__ float gate_exponent(float z, int act) {
     return act == kGateSilu ? z : 1.5957691216057308f * fmaf(0.044715f * z * z, z, z);
 }
@@ -99,6 +100,20 @@ struct ProductView {
             for (int i = 0; i < 16; ++i) v += t[i];
         }
         return v;
+    }
+};
+
+// A product whose x operand was (h * norm weight) still lacks each row's factor 1 / sqrt(sum_s ss[s][row] / hidden + eps):
+// the sums of squares arrive beside it (null: the product is complete).
+struct RowFactor {
+    const float* ss;
+    int splits, n_rows, hidden;
+    float eps;
+    __device__ __forceinline__ float of(int row) const {
+        if (ss == nullptr) return 1.0f;
+        float total = 0.f;
+        for (int s = 0; s < splits; ++s) total += ss[static_cast<size_t>(s) * n_rows + row];
+        return inv_rms(total, 1.0f / static_cast<float>(hidden), eps);
     }
 };
 

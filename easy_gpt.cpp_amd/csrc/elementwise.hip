@@ -20,12 +20,13 @@ __global__ void embed_kernel(const int32_t* __restrict__ ids, const T* __restric
 }
 
 // ----------------------------------------------------------------------------- add + RMSNorm
-// ss = sum x^2 (float32), inv = 1/sqrt(ss/H + eps), y = x * inv * w
+// ss = sum x^2 (float32), inv = 1/sqrt(ss/H + eps), y = x * inv * (w_off + w): w_off is 0, or what a weight is stored as its
+// distance from (1, say), added in float32
 // (/root/reference/src/models/norm.cpp:47-59, /root/reference/src/cuda/ops/self_attn_detail.cuh:385-418).
 // The residual addition h += delta happens here too, in float32.
 template <typename T, typename R, int KEEP>
 __global__ void add_rmsnorm_kernel(R* __restrict__ h, ProductView<T> delta,
-                                   const int32_t* __restrict__ rows, const T* __restrict__ weight, float eps,
+                                   const int32_t* __restrict__ rows, const T* __restrict__ weight, float w_off, float eps,
                                    T* __restrict__ out, int hidden) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
@@ -48,7 +49,7 @@ __global__ void add_rmsnorm_kernel(R* __restrict__ h, ProductView<T> delta,
             w[i] = 0.f;
             if (j < hidden) {
                 v[i] = residual_load(hrow + j);
-                w[i] = to_float(weight[j]);
+                w[i] = w_off + to_float(weight[j]);
             }
         }
         if (has_delta) {
@@ -88,7 +89,7 @@ __global__ void add_rmsnorm_kernel(R* __restrict__ h, ProductView<T> delta,
     for (int j = threadIdx.x; j < hidden; j += blockDim.x) {
         float v = residual_load(hrow + j);       // already updated when written back
         if (has_delta && !write_back) v += delta.at(dbase + j);
-        orow[j] = from_float<T>(v * inv * to_float(weight[j]));
+        orow[j] = from_float<T>(v * inv * (w_off + to_float(weight[j])));
     }
 }
 
@@ -110,7 +111,7 @@ __device__ __forceinline__ void load8_as_float(const float* p, float* v) {
 template <typename DT>   // delta as bfloat16, or as float32 (a product that was written out in float32)
 __global__ __launch_bounds__(256) void add_rmsnorm_vec8_kernel(float* __restrict__ h, const DT* __restrict__ delta,
                                                                const int32_t* __restrict__ rows,
-                                                               const bf16_t* __restrict__ weight, float eps,
+                                                               const bf16_t* __restrict__ weight, float w_off, float eps,
                                                                bf16_t* __restrict__ out, int hidden) {
     __shared__ float scratch[16];
     const int r = blockIdx.x;
@@ -163,6 +164,8 @@ __global__ __launch_bounds__(256) void add_rmsnorm_vec8_kernel(float* __restrict
             }
             load8_as_float(weight + j, w);
         }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) w[i] += w_off;
         uint4 o;
         o.x = f32_to_bf16_bits(v[0] * inv * w[0]) | (static_cast<uint32_t>(f32_to_bf16_bits(v[1] * inv * w[1])) << 16);
         o.y = f32_to_bf16_bits(v[2] * inv * w[2]) | (static_cast<uint32_t>(f32_to_bf16_bits(v[3] * inv * w[3])) << 16);
@@ -426,8 +429,8 @@ static ProductView<T> make_view(const void* p, int n_splits, size_t split_stride
 }
 
 extern "C" int egpt_add_rmsnorm(void* h, int fixed, const void* delta, int delta_splits, int delta_rows,
-                                const int32_t* rows, const void* weight, float eps, void* out, int n_rows, int hidden,
-                                int dtype, void* stream) {
+                                const int32_t* rows, const void* weight, float weight_offset, float eps, void* out,
+                                int n_rows, int hidden, int dtype, void* stream) {
     if (!h || !weight || !out || n_rows < 0 || hidden <= 0 || delta_splits < 0) return EGPT_BAD_ARGUMENT;
     if (delta && delta_rows <= 0) return EGPT_BAD_ARGUMENT;
     if (n_rows == 0) return EGPT_OK;
@@ -441,20 +444,20 @@ extern "C" int egpt_add_rmsnorm(void* h, int fixed, const void* delta, int delta
         float* hf = static_cast<float*>(h);
         if (delta_splits == 0)
             add_rmsnorm_vec8_kernel<bf16_t><<<n_rows, threads, 0, s>>>(
-                hf, static_cast<const bf16_t*>(delta), rows, static_cast<const bf16_t*>(weight), eps,
-                static_cast<bf16_t*>(out), hidden);
+                hf, static_cast<const bf16_t*>(delta), rows, static_cast<const bf16_t*>(weight), weight_offset,
+                eps, static_cast<bf16_t*>(out), hidden);
         else   // one float32 "partial sum": a product written out in float32
             add_rmsnorm_vec8_kernel<float><<<n_rows, threads, 0, s>>>(
-                hf, static_cast<const float*>(delta), rows, static_cast<const bf16_t*>(weight), eps,
-                static_cast<bf16_t*>(out), hidden);
+                hf, static_cast<const float*>(delta), rows, static_cast<const bf16_t*>(weight), weight_offset,
+                eps, static_cast<bf16_t*>(out), hidden);
         EGPT_CHECK_LAUNCH();
         return EGPT_OK;
     }
     if (dtype != 0 && dtype != 1) return EGPT_BAD_ARGUMENT;
 #define EGPT_NORM_KEEP(T_, R_, KEEP_)                                                                      \
     add_rmsnorm_kernel<T_, R_, KEEP_><<<n_rows, threads, 0, s>>>(                                          \
-        static_cast<R_*>(h), make_view<T_>(delta, delta_splits, stride), rows, static_cast<const T_*>(weight), eps, \
-        static_cast<T_*>(out), hidden)
+        static_cast<R_*>(h), make_view<T_>(delta, delta_splits, stride), rows, static_cast<const T_*>(weight), \
+        weight_offset, eps, static_cast<T_*>(out), hidden)
 #define EGPT_NORM(T_, R_)                                        \
     do {                                                         \
         /* (a wide row behind partial sums is faster in the loop: 7.7 against 8.7 us at 64 rows of 5,120) */ \
@@ -600,4 +603,4 @@ extern "C" const char* egpt_error_string(int code) {
     }
 }
 
-extern "C" int egpt_abi_version(void) { return 25; }
+extern "C" int egpt_abi_version(void) { return 26; }

@@ -15,11 +15,12 @@
 // A decode step is a chain of small dependent kernels, and each link costs a few microseconds whatever it
 // computes.  So for m <= 16 the staging of x can also compute x from what the previous kernels left
 // ("prologues"), which removes the separate norm, SwiGLU and attention-combine kernels from the chain:
-//   NORM    x = (h + sum_s delta_s) * norm_weight, not yet divided by the row's RMS: that factor is the same
+//   NORM    x = (h + sum_s delta_s) * (offset + norm_weight), not yet divided by the row's RMS: that factor is the same
 //           for the whole row, so it is applied to the product afterwards by the consumer.  Workgroups of
 //           the first column also write h + delta (the new residual stream, into a second buffer) and the
 //           row's sum of squares of their k range.
 //   SWIGLU  x = silu(g) * u with [g | u] = inv_rms * sum_s gate_up_s (partial sums of a NORM product).
+//   RELU2   x = relu(u)^2 with u = inv_rms * sum_s up_s, a feed-forward without a gate.
 //   ATTN    x = sum_s wgt_s * o_s: the combination of the partial attention results over key splits.
 #include "api.h"
 #include "common.h"
@@ -35,7 +36,7 @@ constexpr int kLdsRow = kStep + 8;  // bf16 elements per staged row of x (16 byt
 constexpr int kMaxLocalHeads = 8;   // ATTN prologue: heads that one workgroup's k range may touch
 constexpr int kMaxAttnSplits = 64;
 
-enum Prologue { kPlain = 0, kNorm = 1, kSwiglu = 2, kAttn = 3 };
+enum Prologue { kPlain = 0, kNorm = 1, kSwiglu = 2, kAttn = 3, kRelu2 = 4 };
 
 struct SkinnyArgs {
     const bf16_t* w;
@@ -53,8 +54,9 @@ struct SkinnyArgs {
     const float* delta;        // [delta_splits][m][k] or null
     int delta_splits;
     const bf16_t* norm_w;      // [k]
+    float norm_off;            // added to the norm weight
     float* ss_out;             // [n_splits][m]
-    // kSwiglu: x[m][k] from gate_up [gu_splits][m][2k]
+    // kSwiglu: x[m][k] from gate_up [gu_splits][m][2k]; kRelu2: from up [gu_splits][m][k]
     const float* gu;
     int gu_splits;
     int act;                   // the gate's activation (gate_activation in common.h)
@@ -245,21 +247,23 @@ __global__ __launch_bounds__(64 * NW) void gemm_skinny_kernel(SkinnyArgs a) {
                 for (int j = 0; j < 8; ++j) {
                     ssq += f[j] * f[j];
                     const uint32_t bits = (j & 1) ? (wb[j / 2] & 0xffff0000u) : (wb[j / 2] << 16);
-                    f[j] *= __uint_as_float(bits);
+                    f[j] *= a.norm_off + __uint_as_float(bits);
                 }
-            } else if constexpr (PRO == kSwiglu) {
-                // gate, up and the row's sums of squares: every load is issued before the first is waited
+            } else if constexpr (PRO == kSwiglu || PRO == kRelu2) {
+                // gate, up (RELU2: up alone) and the row's sums of squares: every load is issued before the first is waited
                 // for (the counter of outstanding loads is in order, so a wait for any of them is a wait for
                 // the stream of w as well: one round trip in all)
+                constexpr bool GATED = PRO == kSwiglu;
                 constexpr int GU = 4, SS = 8;     // splits per batch of loads
-                const size_t idx = static_cast<size_t>(r) * 2 * k + kc;
-                const size_t stride = static_cast<size_t>(m) * 2 * k;
+                const size_t width = GATED ? 2 * static_cast<size_t>(k) : k;
+                const size_t idx = r * width + kc;
+                const size_t stride = m * width;
                 float tg[GU][8], tu[GU][8], sst[SS];
 #pragma unroll
                 for (int i = 0; i < GU; ++i) {
                     const float* p = a.gu + idx + min(i, a.gu_splits - 1) * stride;
                     load8f(p, tg[i]);
-                    load8f(p + k, tu[i]);
+                    if constexpr (GATED) load8f(p + k, tu[i]);
                 }
                 const float* ssp = a.ss_in ? a.ss_in + r : a.gu;       // without a scale: any readable address
                 const int ss_n = a.ss_in ? a.ss_splits : 1;
@@ -272,12 +276,12 @@ __global__ __launch_bounds__(64 * NW) void gemm_skinny_kernel(SkinnyArgs a) {
 #pragma unroll
                     for (int j = 0; j < 8; ++j) {
                         g[j] = fmaf(on, tg[i][j], g[j]);
-                        u[j] = fmaf(on, tu[i][j], u[j]);
+                        if constexpr (GATED) u[j] = fmaf(on, tu[i][j], u[j]);
                     }
                 }
                 if (a.gu_splits > GU) {
                     add_splits8<GU>(a.gu + idx + GU * stride, a.gu_splits - GU, stride, g);
-                    add_splits8<GU>(a.gu + idx + GU * stride + k, a.gu_splits - GU, stride, u);
+                    if constexpr (GATED) add_splits8<GU>(a.gu + idx + GU * stride + k, a.gu_splits - GU, stride, u);
                 }
                 float ss = 0.f;
 #pragma unroll
@@ -287,7 +291,8 @@ __global__ __launch_bounds__(64 * NW) void gemm_skinny_kernel(SkinnyArgs a) {
 #pragma unroll
                 for (int j = 0; j < 8; ++j) {
                     const float gg = g[j] * inv;
-                    f[j] = (u[j] * inv) * gg * __builtin_amdgcn_rcpf(1.0f + __expf(-gate_exponent(gg, a.act)));
+                    if constexpr (GATED) f[j] = (u[j] * inv) * gg * __builtin_amdgcn_rcpf(1.0f + __expf(-gate_exponent(gg, a.act)));
+                    else f[j] = fmaxf(gg, 0.f) * fmaxf(gg, 0.f);
                 }
             } else {  // kAttn
                 const int head = kc / a.hd, d = kc % a.hd;
@@ -645,11 +650,11 @@ extern "C" int egpt_gemm_skinny(const void* x, const void* w, const void* bias, 
     return EGPT_OK;
 }
 
-// out[split][m][n] = partial sums of ((h_in + sum delta) * norm_w) w^T; h_out = h_in + sum delta;
+// out[split][m][n] = partial sums of ((h_in + sum delta) * (norm_offset + norm_w)) w^T; h_out = h_in + sum delta;
 // ss_out[split][m] = sums of squares of h_out over the split's k range.  m <= 16, k % 8 == 0.
 extern "C" int egpt_gemm_skinny_norm(const void* h_in, int h_fixed, float* h_out, const float* delta, int delta_splits,
-                                     const void* norm_w, const void* w, float* out, float* ss_out, int m, int n, int k,
-                                     int n_splits, int waves, void* stream) {
+                                     const void* norm_w, float norm_offset, const void* w, float* out, float* ss_out, int m,
+                                     int n, int k, int n_splits, int waves, void* stream) {
     if (!h_in || !norm_w || !w || !out || !ss_out || m <= 0 || n <= 0 || k <= 0 ||
         delta_splits < 0 || (delta && delta_splits == 0) || (waves != 4 && waves != 8 && waves != 16))
         return EGPT_BAD_ARGUMENT;
@@ -664,6 +669,7 @@ extern "C" int egpt_gemm_skinny_norm(const void* h_in, int h_fixed, float* h_out
     else a.h_in = static_cast<const float*>(h_in);
     a.h_out = h_out; a.delta = delta; a.delta_splits = delta ? delta_splits : 0;
     a.norm_w = static_cast<const bf16_t*>(norm_w);
+    a.norm_off = norm_offset;
     a.ss_out = ss_out;
     // Many partial sums to add and few workgroups (which then need not share a CU): more loads in flight.
     // As many loads in flight as there are partial sums to add, if registers allow: few workgroups need not
@@ -680,11 +686,12 @@ extern "C" int egpt_gemm_skinny_norm(const void* h_in, int h_fixed, float* h_out
 }
 
 // out[split][m][n] = partial sums of swiglu(inv_rms * sum gate_up) w^T, gate_up [gu_splits][m][2k];
-// inv_rms[m] = 1 / sqrt(sum_s ss_in[s][m] / hidden + eps), or 1 if ss_in is null.
+// inv_rms[m] = 1 / sqrt(sum_s ss_in[s][m] / hidden + eps), or 1 if ss_in is null.  act kUngatedRelu2: of relu(inv_rms * sum
+// up)^2 w^T with up [gu_splits][m][k].
 extern "C" int egpt_gemm_skinny_swiglu(const float* gate_up, int gu_splits, const float* ss_in, int ss_splits,
                                        int hidden, float eps, const void* w, float* out, void* acc_fixed, int m, int n,
                                        int k, int n_splits, int waves, int act, void* stream) {
-    if (!gate_up || gu_splits < 1 || (act != kGateSilu && act != kGateGeluTanh) || !w || (!out == !acc_fixed) || m <= 0 || n <= 0 || k <= 0 || (ss_in && (ss_splits < 1 || hidden < 1)) ||
+    if (!gate_up || gu_splits < 1 || (act != kGateSilu && act != kGateGeluTanh && act != kUngatedRelu2) || !w || (!out == !acc_fixed) || m <= 0 || n <= 0 || k <= 0 || (ss_in && (ss_splits < 1 || hidden < 1)) ||
         (waves != 4 && waves != 8 && waves != 16))
         return EGPT_BAD_ARGUMENT;
     if (m > 16 || (k % 8) != 0) return EGPT_UNSUPPORTED_SIZE;
@@ -698,7 +705,8 @@ extern "C" int egpt_gemm_skinny_swiglu(const float* gate_up, int gu_splits, cons
     a.inv_hidden = ss_in ? 1.0f / static_cast<float>(hidden) : 0.f;
     a.eps = eps;
     a.act = act;
-    EGPT_SKINNY(1, kSwiglu, 8);
+    if (act == kUngatedRelu2) EGPT_SKINNY(1, kRelu2, 8);
+    else EGPT_SKINNY(1, kSwiglu, 8);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }

@@ -11,20 +11,6 @@
 
 namespace egpt {
 
-// A product whose x operand was (h * norm weight) still lacks each row's factor 1 / sqrt(sum_s ss[s][row] / hidden + eps):
-// the sums of squares arrive beside it (null: the product is complete).
-struct RowFactor {
-    const float* ss;
-    int splits, n_rows, hidden;
-    float eps;
-    __device__ __forceinline__ float of(int row) const {
-        if (ss == nullptr) return 1.0f;
-        float total = 0.f;
-        for (int s = 0; s < splits; ++s) total += ss[static_cast<size_t>(s) * n_rows + row];
-        return inv_rms(total, 1.0f / static_cast<float>(hidden), eps);
-    }
-};
-
 constexpr int kMaxHeadWidth = 1024;                   // the widest head (or latent) these kernels take
 constexpr int kOwn = kMaxHeadWidth / kWave;           // values of it that a lane keeps
 
@@ -516,8 +502,8 @@ extern "C" int egpt_head_norm_store(const void* proj, int n_splits, const float*
                                     int dv, int page_size, float* values_out, const float* mix_with, float mix, int n_gates,
                                     int gate_off, float* gates_out, int dtype, void* stream) {
     if (n_gates < 0 || (n_gates > 0 && (!gates_out || gate_off < 0 || gate_off + n_gates > row_width))) return EGPT_BAD_ARGUMENT;
-    if (!proj || !q_out || n_splits < 0 || n_tokens < 0 || nq <= 0 || nkv <= 0 || dk <= 0 || dv <= 0 || page_size <= 0 ||
-        (dtype != 0 && dtype != 1) || flags < 0 || flags >= 32)
+    if (!proj || !q_out || n_splits < 0 || n_tokens < 0 || nq <= 0 || nkv < 0 || dk <= 0 || dv <= 0 || page_size <= 0 ||
+        (dtype != 0 && dtype != 1) || flags < 0 || flags >= 32 || (nkv == 0 && (slots || values_out)))
         return EGPT_BAD_ARGUMENT;
     if (slots && (!k_cache || !v_cache)) return EGPT_BAD_ARGUMENT;
     if (rot_dims < 0 || rot_dims % 2 || rot_dims > dk || (rot_dims > 0 && !cos_sin)) return EGPT_BAD_ARGUMENT;

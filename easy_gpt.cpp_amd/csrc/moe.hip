@@ -2,12 +2,15 @@
 // products as grouped products on the matrix cores, and the weighted sum of a token's choices in a fixed order.
 //
 //   egpt_moe_route     logits = x R^T + b (float32), the `top` largest, softmax over those; or the softmax over all
-//                      experts, the choice by score + a correction per expert, the chosen scores over their sum
+//                      outputs, the choice by score + a correction per output, within the best groups of neighbouring
+//                      outputs if there are groups, weighed by the chosen scores (over their sum or as they are)
 //   egpt_moe_up        act = relu(x Wu^T)^2 per grouped row: experts without a gate
-//   egpt_moe_group     (token, choice) rows grouped by expert; tiles of rows, each of one expert
+//   egpt_moe_group     (token, choice) rows grouped by expert; tiles of rows, each of one expert.  Router outputs from
+//                      `experts` on are identity experts: they hand on x itself and get no row
 //   egpt_moe_gate_up   act = silu(x Wg^T) * (x Wu^T) per grouped row, with that row's expert
 //   egpt_moe_down      y = act Wd^T per grouped row (float32)
-//   egpt_moe_combine   out[t] = sum_c weight[t][c] * y[place[t][c]]
+//   egpt_moe_combine   out[t] = sum_c weight[t][c] * y[place[t][c]] (x[t] where the choice has no row), written out or added
+//                      to the residual stream in fixed point
 //
 // Nothing is read back by the host: the grid of the grouped products is sized for the most tiles that the rows can
 // make (rows / tile + experts), and a workgroup whose tile does not exist leaves at once.  A row's result does not
@@ -60,7 +63,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
                                                         const T* __restrict__ bias, int32_t* __restrict__ chosen,
                                                         float* __restrict__ weight, int n_tokens, int hidden, int experts,
                                                         int top, int score_all, const float* __restrict__ correction,
-                                                        float weight_scale) {
+                                                        float weight_scale, int groups, int keep_groups, int normalized) {
     extern __shared__ float logits_s[];          // [experts]
     const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
     const int t = blockIdx.x;
@@ -85,8 +88,8 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
     __syncthreads();
     if (wave != 0) return;
     if (score_all) {
-        // scores s = softmax(z) over all experts; an expert is chosen by s + correction and weighs s over the sum of
-        // the chosen scores.  z[] keeps the choice scores, score_s[] (behind it) the scores themselves.
+        // scores s = softmax(z) over all experts; an expert is chosen by s + correction and weighs s, over the sum of
+        // the chosen scores if `normalized`.  z[] keeps the choice scores, score_s[] (behind it) the scores themselves.
         float* score_s = logits_s + experts;
         float mx = -INFINITY;
         for (int e = lane; e < experts; e += kWave) mx = fmaxf(mx, z[e]);
@@ -98,6 +101,48 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
             const float sc = expf(z[e] - mx) * inv_sum;
             score_s[e] = sc;
             z[e] = sc + (correction ? correction[e] : 0.f);
+        }
+        if (groups > 1) {
+            // A group's score is the largest choice score among its neighbours; outside the best keep_groups of them
+            // nothing can be chosen.  A lane owns the groups lane, lane + 64, ...; the best are picked one after the
+            // other (the lowest index among equals), and group_s[] says which group is still in the running.
+            __builtin_amdgcn_wave_barrier();
+            __threadfence_block();               // (a lane reads what other lanes wrote)
+            float* group_s = score_s + experts;
+            const int size = experts / groups;
+            for (int g = lane; g < groups; g += kWave) {
+                float best = -INFINITY;
+                for (int e = 0; e < size; ++e) best = fmaxf(best, z[g * size + e]);
+                group_s[g] = best;
+            }
+            unsigned int kept = 0;               // bit i: group lane + 64 i is kept (at most 1024 / 64 bits)
+            for (int c = 0; c < keep_groups; ++c) {
+                float best = -INFINITY;
+                int best_g = 0x7fffffff;
+                for (int g = lane; g < groups; g += kWave) {
+                    const bool taken = kept >> (g / kWave) & 1;
+                    const float v = group_s[g];
+                    if (!taken && (best_g == 0x7fffffff || v > best)) {
+                        best = v;
+                        best_g = g;
+                    }
+                }
+#pragma unroll
+                for (int off = kWave / 2; off > 0; off >>= 1) {
+                    const float ov = __shfl_xor(best, off, kWave);
+                    const int og = __shfl_xor(best_g, off, kWave);
+                    if (ov > best || (ov == best && og < best_g)) {
+                        best = ov;
+                        best_g = og;
+                    }
+                }
+                if (best_g % kWave == lane) kept |= 1u << (best_g / kWave);
+            }
+            for (int g = lane; g < groups; g += kWave)
+                if (!(kept >> (g / kWave) & 1))
+                    for (int e = 0; e < size; ++e) z[g * size + e] = -INFINITY;
+            __builtin_amdgcn_wave_barrier();
+            __threadfence_block();
         }
         float chosen_sum = 0.f;
         for (int c = 0; c < top; ++c) {
@@ -119,6 +164,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
                     best_e = oe;
                 }
             }
+            best_e = min(best_e, experts - 1);   // (logits that are no numbers leave none: any index in range)
             const float sc = score_s[best_e];
             chosen_sum += sc;
             if (lane == 0) {
@@ -128,7 +174,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
             if (lane == best_e % kWave) z[best_e] = -INFINITY;
         }
         if (lane == 0) {
-            const float f = weight_scale / (chosen_sum + 1e-20f);
+            const float f = normalized ? weight_scale / (chosen_sum + 1e-20f) : weight_scale;
             for (int c = 0; c < top; ++c) weight[static_cast<size_t>(t) * top + c] *= f;
         }
         return;
@@ -154,6 +200,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
                 best_e = oe;
             }
         }
+        best_e = min(best_e, experts - 1);       // (logits that are no numbers leave none: any index in range)
         if (c == 0) first = best;
         const float p = expf(best - first);      // the first choice is the largest
         total += p;
@@ -178,7 +225,8 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t* __restri
     __shared__ int first_s[kMaxExperts + 1];
     for (int e = threadIdx.x; e < experts; e += blockDim.x) count_s[e] = 0;
     __syncthreads();
-    for (int i = threadIdx.x; i < n_rows; i += blockDim.x) atomicAdd(&count_s[chosen[i]], 1);
+    for (int i = threadIdx.x; i < n_rows; i += blockDim.x)
+        if (chosen[i] < experts) atomicAdd(&count_s[chosen[i]], 1);
     __syncthreads();
     if (threadIdx.x == 0) {
         int at = 0, n_tiles = 0;
@@ -205,6 +253,10 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t* __restri
     // which row of its expert a (token, choice) gets does not matter to its result, only that it gets one
     for (int i = threadIdx.x; i < n_rows; i += blockDim.x) {
         const int e = chosen[i];
+        if (e >= experts) {                      // an identity expert
+            place[i] = -1;
+            continue;
+        }
         const int row = first_s[e] + atomicAdd(&count_s[e], 1);
         row_token[row] = i / top;
         place[i] = row;
@@ -368,15 +420,22 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ act
     }
 }
 
-__global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ y, const int32_t* __restrict__ place,
-                                                          const float* __restrict__ weight, float* __restrict__ out, int top,
-                                                          int hidden) {
+// out: the sum itself; stream: the residual stream in fixed point that it is added to (one of the two is null).
+template <typename T>
+__global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ y, const T* __restrict__ x,
+                                                          const int32_t* __restrict__ place, const float* __restrict__ weight,
+                                                          float* __restrict__ out, fixed_t* __restrict__ stream, int top, int hidden) {
     const int t = blockIdx.x;
     for (int j = threadIdx.x; j < hidden; j += blockDim.x) {
+        const size_t at = static_cast<size_t>(t) * hidden + j;
         float acc = 0.f;
-        for (int c = 0; c < top; ++c)
-            acc = fmaf(weight[static_cast<size_t>(t) * top + c], y[static_cast<size_t>(place[static_cast<size_t>(t) * top + c]) * hidden + j], acc);
-        out[static_cast<size_t>(t) * hidden + j] = acc;
+        for (int c = 0; c < top; ++c) {
+            const int row = place[static_cast<size_t>(t) * top + c];
+            const float v = row >= 0 ? y[static_cast<size_t>(row) * hidden + j] : to_float(x[at]);
+            acc = fmaf(weight[static_cast<size_t>(t) * top + c], v, acc);
+        }
+        if (stream != nullptr) stream[at] += to_fixed(acc);
+        else out[at] = acc;
     }
 }
 
@@ -386,23 +445,28 @@ using namespace egpt;
 
 extern "C" int egpt_moe_route(const void* x, const void* router, const void* bias, int32_t* chosen, float* weight, int n_tokens,
                               int hidden, int experts, int top, int score_all, const float* correction, float weight_scale,
-                              int dtype, void* stream) {
+                              int groups, int keep_groups, int normalized, int dtype, void* stream) {
     if (!x || !router || !chosen || !weight || n_tokens < 0 || hidden <= 0 || experts <= 0 || top <= 0 || top > experts ||
         (dtype != 0 && dtype != 1))
+        return EGPT_BAD_ARGUMENT;
+    if (groups < 1 || experts % groups || keep_groups < 1 || keep_groups > groups || experts / groups * keep_groups < top ||
+        (groups > 1 && !score_all))
         return EGPT_BAD_ARGUMENT;
     if (experts > kMaxExperts) return EGPT_UNSUPPORTED_SIZE;
     if (n_tokens == 0) return EGPT_OK;
     hipStream_t s = static_cast<hipStream_t>(stream);
-    const size_t lds = 2 * static_cast<size_t>(experts) * sizeof(float);
+    const size_t lds = 3 * static_cast<size_t>(experts) * sizeof(float);      // choice scores, scores, groups' scores
     const unsigned blocks = n_tokens;
     if (dtype == 0)
         moe_route_kernel<float><<<blocks, 256, lds, s>>>(static_cast<const float*>(x), static_cast<const float*>(router),
                                                          static_cast<const float*>(bias), chosen, weight, n_tokens, hidden,
-                                                         experts, top, score_all, correction, weight_scale);
+                                                         experts, top, score_all, correction, weight_scale, groups,
+                                                         keep_groups, normalized);
     else
         moe_route_kernel<bf16_t><<<blocks, 256, lds, s>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(router),
                                                           static_cast<const bf16_t*>(bias), chosen, weight, n_tokens, hidden,
-                                                          experts, top, score_all, correction, weight_scale);
+                                                          experts, top, score_all, correction, weight_scale, groups,
+                                                         keep_groups, normalized);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }
@@ -497,11 +561,17 @@ extern "C" int egpt_moe_down(const void* act, const void* w_down, const int32_t*
     return EGPT_OK;
 }
 
-extern "C" int egpt_moe_combine(const float* y, const int32_t* place, const float* weight, float* out, int n_tokens, int top,
-                                int hidden, void* stream) {
-    if (!y || !place || !weight || !out || n_tokens < 0 || top <= 0 || hidden <= 0) return EGPT_BAD_ARGUMENT;
+extern "C" int egpt_moe_combine(const float* y, const void* x, const int32_t* place, const float* weight, float* out,
+                                void* residual, int n_tokens, int top, int hidden, int dtype, void* stream) {
+    if (!y || !x || !place || !weight || (!out == !residual) || n_tokens < 0 || top <= 0 || hidden <= 0 || (dtype != 0 && dtype != 1))
+        return EGPT_BAD_ARGUMENT;
     if (n_tokens == 0) return EGPT_OK;
-    moe_combine_kernel<<<n_tokens, 256, 0, static_cast<hipStream_t>(stream)>>>(y, place, weight, out, top, hidden);
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    fixed_t* acc = static_cast<fixed_t*>(residual);
+    if (dtype == 0)
+        moe_combine_kernel<float><<<n_tokens, 256, 0, s>>>(y, static_cast<const float*>(x), place, weight, out, acc, top, hidden);
+    else
+        moe_combine_kernel<bf16_t><<<n_tokens, 256, 0, s>>>(y, static_cast<const bf16_t*>(x), place, weight, out, acc, top, hidden);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }

@@ -104,20 +104,20 @@ __global__ __launch_bounds__(256) void normed_pair_mean_kernel(ProductView<T> a,
                                              : factor_a * (a_s[j] * inv_a * to_float(wa[j])) + factor_b * (b_s[j] * inv_b * to_float(wb[j]));
 }
 
-// x[t, :] = E[id_t, :] + P[position_t, :]: a token's vector plus a learned vector of its position, added in float32
-// and written as the float32 residual stream.
-template <typename T>
+// x[t, :] = factor * E[id_t, :] + P[position_t, :]: a token's vector plus a learned vector of its position, added in float32
+// and written as the residual stream (float32 or fixed point).
+template <typename T, typename R>
 __global__ __launch_bounds__(256) void embed_positions_kernel(const int32_t* __restrict__ ids, const int32_t* __restrict__ positions,
                                                               const T* __restrict__ table, const T* __restrict__ pos_table,
-                                                              float* __restrict__ out, int hidden, int vocab, int max_pos) {
+                                                              float factor, R* __restrict__ out, int hidden, int vocab, int max_pos) {
     const int t = blockIdx.x;
     int id = ids[t], p = positions[t];
     id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);      // both are range-checked on the host; never read outside
     p = p < 0 ? 0 : (p >= max_pos ? max_pos - 1 : p);
     const T* row = table + static_cast<size_t>(id) * hidden;
     const T* prow = pos_table + static_cast<size_t>(p) * hidden;
-    float* o = out + static_cast<size_t>(t) * hidden;
-    for (int j = threadIdx.x; j < hidden; j += blockDim.x) o[j] = to_float(row[j]) + to_float(prow[j]);
+    R* o = out + static_cast<size_t>(t) * hidden;
+    for (int j = threadIdx.x; j < hidden; j += blockDim.x) residual_store(o + j, fmaf(to_float(row[j]), factor, to_float(prow[j])));
 }
 
 // A branch's output joins the stream behind a norm of its own:  x = h + mult * LN(y) * post_w  (LN without bias, the
@@ -397,18 +397,22 @@ extern "C" int egpt_normed_pair_mean(const void* a, int a_splits, const void* b,
 }
 
 extern "C" int egpt_embed_positions(const int32_t* ids, const int32_t* positions, const void* table, const void* pos_table,
-                                    float* out, int n_tokens, int hidden, int vocab, int max_pos, int dtype, void* stream) {
+                                    float factor, void* out, int fixed, int n_tokens, int hidden, int vocab, int max_pos, int dtype,
+                                    void* stream) {
     if (!ids || !positions || !table || !pos_table || !out || n_tokens < 0 || hidden <= 0 || vocab <= 0 || max_pos <= 0 ||
         (dtype != 0 && dtype != 1))
         return EGPT_BAD_ARGUMENT;
     if (n_tokens == 0) return EGPT_OK;
     hipStream_t s = static_cast<hipStream_t>(stream);
-    if (dtype == 0)
-        embed_positions_kernel<float><<<n_tokens, 256, 0, s>>>(ids, positions, static_cast<const float*>(table),
-                                                               static_cast<const float*>(pos_table), out, hidden, vocab, max_pos);
-    else
-        embed_positions_kernel<bf16_t><<<n_tokens, 256, 0, s>>>(ids, positions, static_cast<const bf16_t*>(table),
-                                                                static_cast<const bf16_t*>(pos_table), out, hidden, vocab, max_pos);
+#define EGPT_EMBED_POS(T_, R_)                                                                                   \
+    embed_positions_kernel<T_, R_><<<n_tokens, 256, 0, s>>>(ids, positions, static_cast<const T_*>(table),       \
+                                                            static_cast<const T_*>(pos_table), factor,           \
+                                                            static_cast<R_*>(out), hidden, vocab, max_pos)
+    if (dtype == 0 && !fixed) EGPT_EMBED_POS(float, float);
+    else if (dtype == 0) EGPT_EMBED_POS(float, fixed_t);
+    else if (!fixed) EGPT_EMBED_POS(bf16_t, float);
+    else EGPT_EMBED_POS(bf16_t, fixed_t);
+#undef EGPT_EMBED_POS
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }

@@ -11,7 +11,8 @@ Methods of a backend (T tokens, B requests, R rows, act = bfloat16 or float32):
 
   embed(token_ids i32[T], table act[V,H], out f32[T,H])
   add_rmsnorm(h f32[T,H], delta act[T,H]|None, weight act[H], eps, out act[T,H])
-        h += delta in float32 (in place), out = h * rsqrt(mean(h^2) + eps) * weight
+        h += delta in float32 (in place), out = h * rsqrt(mean(h^2) + eps) * weight; with weight_offset (0 unless given)
+        * (weight_offset + weight), which is added in float32
   rows_add_rmsnorm(h, delta|None, rows i32[R], weight, eps, out act[R,H])
         the same for rows `rows` only, h is not written
   linear(x act[T,K], w act[N,K], bias act[N]|None, out act|f32 [T,N])      out = x w^T + bias
@@ -72,6 +73,14 @@ Methods of a backend (T tokens, B requests, R rows, act = bfloat16 or float32):
         plain sum), the second the streams as they are now (in place where that is possible; with rows, or keep False, the
         ones given: nothing is kept)
 
+  window_attention(..., difference=(weight, eps, factor)): a head's query and key are two maps of dk / 2 side by side over the same
+        values, and its output is a / sqrt(mean(a^2) + eps) * factor with a = a1 - weight * a2 (the maps' outputs)
+  (head_norm_store with nkv 0: rows of queries alone, for a layer that reads another's keys and values)
+
+  embed_positions(token_ids, positions i32[T], table act[V,H], pos_table act[P,H], out, factor=1)
+        out = factor * table[id] + pos_table[position], a residual stream of either kind
+  ff_activation(z act[T,W]|f32[S,T,W], cols, mode, out act[T,cols], coef=None, eps=0, gate_col=-1; row_ss, hidden, norm_eps)
+        relu2: relu(z)^2; polynorm: a polynomial of normed powers; times the sigmoid of a further column
   embed_scaled(token_ids i32[T], table act[V,H], factor, out f32[T,H])          out = table[id] * factor
   add_layernorm(h f32[T,H], delta act[T,H]|f32[S,T,H]|None, rows i32[R]|None, weight act[H], bias act[H]|None, eps, out)
         h += delta; out = (h - mean) / sqrt(mean((h - mean)^2) + eps) * weight + bias; with rows only those, h untouched
@@ -113,6 +122,9 @@ Methods of a backend (T tokens, B requests, R rows, act = bfloat16 or float32):
   expert_mixture(x act[T,H], router act[E,H], router_bias act[E]|None, w_gate_up act[E,2F,H], w_down act[E,H,F], top) -> f32[T,H]
         float32 logits x router^T + bias, the `top` largest (lowest index among equals), softmax over those; the weighted
         sum of down_e(silu(gate_e x) * (up_e x)) over the chosen experts e, added in the order of the choices
+        (gated False: experts down_e(relu(up_e x)^2); score_all: softmax over all, choice by score + correction, within the best
+        keep_groups of `groups` groups of neighbours, weights the scores times weight_scale, over their sum if normalized;
+        identities: the router's last outputs hand on x itself; residual: the fixed-point stream that the sum is added to)
 
 Beside these, a backend has fused variants that fold neighbouring operations into one kernel.  They are part of
 the contract too (`KernelBackend` below): each returns None (False for the decode attention) where it does not
@@ -198,13 +210,13 @@ class KernelBackend:
         a residual stream in fixed point that the backend can add the product into, that stream."""
         raise NotImplementedError
 
-    def product_normed(self, h, delta, norm_weight, w):
-        """((h + delta) * norm_weight) w^T without the rows' 1/rms factor: (float32 partial sums [S, T, N], row sums
+    def product_normed(self, h, delta, norm_weight, w, weight_offset=0.0):
+        """((h + delta) * (weight_offset + norm_weight)) w^T without the rows' 1/rms factor: (float32 partial sums [S, T, N], row sums
         of squares [S2, T], h + delta as a new tensor), or None."""
         return None
 
     def product_swiglu(self, gate_up, row_ss, hidden, eps, w, residual=None, activation="silu"):
-        """swiglu(scale * sum of the partial sums gate_up) w^T as float32 partial sums (or added into `residual`,
+        """swiglu(scale * sum of the partial sums gate_up) w^T (activation 'relu2': there is no gate, relu(scale * up)^2 w^T) as float32 partial sums (or added into `residual`,
         which is then returned), or None."""
         return None
 

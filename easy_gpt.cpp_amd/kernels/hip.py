@@ -15,6 +15,7 @@ from . import KernelBackend, KernelsUnavailable, ProductSum, StreamUpdate
 _F32, _BF16, _I32, _I64 = torch.float32, torch.bfloat16, torch.int32, torch.int64
 _DT = {_F32: 0, _BF16: 1}
 _GATES = {"silu": 0, "gelu_tanh": 1}          # activations of a gated feed-forward's gate (gate_activation in common.h)
+_UNGATED_RELU2 = 2                            # no gate, where a product may begin with either
 
 
 def _load_library() -> ctypes.CDLL:
@@ -29,7 +30,7 @@ def _load_library() -> ctypes.CDLL:
         lib = ctypes.CDLL(path)
     except (build.BuildError, OSError) as e:
         raise KernelsUnavailable(f"the HIP kernel library could not be built or loaded: {e}") from e
-    if lib.egpt_abi_version() != 25:
+    if lib.egpt_abi_version() != 26:
         raise KernelsUnavailable(f"{path} has an unexpected ABI version")
     return lib
 
@@ -78,11 +79,11 @@ class HipKernels(KernelBackend):
         lib.egpt_error_string.argtypes = [i]
         sigs = {
             "egpt_embed": [vp, vp, vp, i, i, i, i, i, vp],
-            "egpt_add_rmsnorm": [vp, i, vp, i, i, vp, vp, f, vp, i, i, i, vp],
+            "egpt_add_rmsnorm": [vp, i, vp, i, i, vp, vp, f, f, vp, i, i, i, vp],
             "egpt_swiglu": [vp, i, vp, i, i, f, vp, i, i, i, i, vp],
             "egpt_qkv_rope_store": [vp, i, vp, i, i, f, vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, vp],
             "egpt_rope_table": [vp, vp, vp, i, i, vp],
-            "egpt_gemm_skinny_norm": [vp, i, vp, vp, i, vp, vp, vp, vp, i, i, i, i, i, vp],
+            "egpt_gemm_skinny_norm": [vp, i, vp, vp, i, vp, f, vp, vp, vp, i, i, i, i, i, vp],
             "egpt_gemm_skinny_swiglu": [vp, i, vp, i, i, f, vp, vp, vp, i, i, i, i, i, i, vp],
             "egpt_gemm_skinny_attn": [vp, vp, i, i, i, vp, vp, vp, i, i, i, i, vp],
             "egpt_attention_combine": [vp, vp, vp, i, i, i, vp],
@@ -107,13 +108,13 @@ class HipKernels(KernelBackend):
                                      vp],
             "egpt_latent_prep": [vp, i, vp, i, i, f, i, vp, i, i, vp, vp, vp, f, vp, f, i, vp, vp, vp, i, i, i, i, i, i, i, vp],
             "egpt_sigmoid_gate": [vp, i, vp, i, vp, i, i, f, i, i, vp, i, i, i, vp],
-            "egpt_window_attention": [vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, vp, vp, i, i, vp, f, vp, i, vp],
+            "egpt_window_attention": [vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, vp, vp, i, i, vp, f, vp, i, f, f, f, i, vp],
             "egpt_window_attention_tiled": [vp, vp, vp, vp, vp, vp, vp, i, vp, vp, vp, i, i, i, i, i, i, i, f, i, i, vp, vp, i,
-                                            i, vp, f, vp, i, i, i, vp],
-            "egpt_embed_positions": [vp, vp, vp, vp, vp, i, i, i, i, i, vp],
+                                            i, vp, f, vp, i, f, f, f, i, i, i, vp],
+            "egpt_embed_positions": [vp, vp, vp, vp, f, vp, i, i, i, i, i, i, vp],
             "egpt_post_norm_add": [vp, vp, i, vp, i, f, f, vp, f, f, vp, i, vp, vp, vp, vp, i, i, i, vp],
             "egpt_bounded_gate": [vp, i, i, i, vp, vp, vp, i, i, i, vp],
-            "egpt_ff_activation": [vp, i, i, i, i, vp, f, i, vp, i, i, vp],
+            "egpt_ff_activation": [vp, i, vp, i, i, f, i, i, i, vp, f, i, vp, i, i, vp],
             "egpt_moe_up": [vp, vp, vp, vp, vp, i, i, i, i, i, i, vp],
             "egpt_embed_scaled": [vp, vp, f, vp, i, i, i, i, vp],
             "egpt_add_layernorm": [vp, vp, i, i, vp, vp, vp, f, vp, i, i, i, vp],
@@ -127,11 +128,11 @@ class HipKernels(KernelBackend):
             "egpt_connect_streams": [vp, ctypes.c_longlong, i, vp, i, i, vp, vp, vp, vp, vp, ctypes.c_longlong, vp, vp, f, vp, i, i, i, vp],
             "egpt_short_conv": [vp, i, i, i, vp, i, i, i, i, i, f, f, i, i, vp, ctypes.c_longlong, vp, vp, vp, vp, i, i, i, vp, i, vp],
             "egpt_delta_rule_scan": [vp, i, i, i, i, i, vp, vp, ctypes.c_longlong, vp, vp, vp, vp, i, i, vp, i, i, i, i, vp],
-            "egpt_moe_route": [vp, vp, vp, vp, vp, i, i, i, i, i, vp, f, i, vp],
+            "egpt_moe_route": [vp, vp, vp, vp, vp, i, i, i, i, i, vp, f, i, i, i, i, vp],
             "egpt_moe_group": [vp, vp, vp, vp, vp, i, i, i, i, vp],
             "egpt_moe_gate_up": [vp, vp, vp, vp, vp, i, i, i, i, i, i, vp],
             "egpt_moe_down": [vp, vp, vp, vp, i, i, i, i, i, i, vp],
-            "egpt_moe_combine": [vp, vp, vp, vp, i, i, i, vp],
+            "egpt_moe_combine": [vp, vp, vp, vp, vp, vp, i, i, i, i, vp],
         }
         lib.egpt_scan_key_splits.restype = i
         lib.egpt_scan_key_splits.argtypes = [i]
@@ -236,7 +237,7 @@ class HipKernels(KernelBackend):
         self._need(residual, "residual", _I64, (t, n))
         return residual
 
-    def add_rmsnorm(self, h, delta, weight, eps, out):
+    def add_rmsnorm(self, h, delta, weight, eps, out, weight_offset=0.0):
         t, hid = h.shape
         dt = self._act(out, "out")
         self._need(h, "h")
@@ -244,9 +245,9 @@ class HipKernels(KernelBackend):
         self._need(out, "out", None, (t, hid))
         splits = self._product(delta, "delta", out.dtype, t, hid) if delta is not None else 0
         self._run("egpt_add_rmsnorm", h.data_ptr(), self._fixed(h, "h"), self._ptr(delta), splits, t, None,
-                  weight.data_ptr(), float(eps), out.data_ptr(), t, hid, dt, self._stream())
+                  weight.data_ptr(), float(weight_offset), float(eps), out.data_ptr(), t, hid, dt, self._stream())
 
-    def rows_add_rmsnorm(self, h, delta, rows, weight, eps, out):
+    def rows_add_rmsnorm(self, h, delta, rows, weight, eps, out, weight_offset=0.0):
         t, hid = h.shape
         r = rows.shape[0]
         dt = self._act(out, "out")
@@ -256,7 +257,7 @@ class HipKernels(KernelBackend):
         self._need(out, "out", None, (r, hid))
         splits = self._product(delta, "delta", out.dtype, t, hid) if delta is not None else 0
         self._run("egpt_add_rmsnorm", h.data_ptr(), self._fixed(h, "h"), self._ptr(delta), splits, t, rows.data_ptr(),
-                  weight.data_ptr(), float(eps), out.data_ptr(), r, hid, dt, self._stream())
+                  weight.data_ptr(), float(weight_offset), float(eps), out.data_ptr(), r, hid, dt, self._stream())
 
     @staticmethod
     def _library_rows(m: int, n: int, k: int) -> bool:
@@ -393,8 +394,8 @@ class HipKernels(KernelBackend):
         waves = min((4, 8, 16), key=lambda w: (rounds[w], w))
         return s, waves
 
-    def product_normed(self, h, delta, norm_weight, w, waves=None, splits=None):
-        """((h + delta) * norm_weight) w^T without the rows' 1/rms factor, for few rows in bfloat16.
+    def product_normed(self, h, delta, norm_weight, w, waves=None, splits=None, weight_offset=0.0):
+        """((h + delta) * (weight_offset + norm_weight)) w^T without the rows' 1/rms factor, for few rows in bfloat16.
         Returns (float32 partial sums [S, T, N], row sums of squares [S, T], h + delta as a new tensor),
         or None if this case is not covered or not worth it (the caller then runs the norm by itself)."""
         t, k = h.shape
@@ -428,19 +429,20 @@ class HipKernels(KernelBackend):
         ss = torch.empty((s, t), dtype=_F32, device=h.device)
         h_new = h if fixed else torch.empty_like(h)      # a stream in fixed point is complete: nothing is added here
         self._run("egpt_gemm_skinny_norm", h.data_ptr(), fixed, None if fixed else h_new.data_ptr(), self._ptr(delta),
-                  d_splits, norm_weight.data_ptr(), w.data_ptr(), out.data_ptr(), ss.data_ptr(), t, n, k, s, waves,
-                  self._stream())
+                  d_splits, norm_weight.data_ptr(), float(weight_offset), w.data_ptr(), out.data_ptr(), ss.data_ptr(), t, n, k,
+                  s, waves, self._stream())
         return out, ss, h_new
 
     def product_swiglu(self, gate_up, row_ss, hidden, eps, w, max_splits=20, waves=None, residual=None, activation="silu"):
         """swiglu(scale * sum gate_up) w^T for float32 partial sums gate_up [S, T, 2I]; scale is the rows' 1/rms
         from row_ss [S2, T] (or 1).  Returns float32 partial sums [S3, T, N] or None if not covered; with a residual
-        stream in fixed point [T, N] the product is added into it instead and the stream is returned."""
+        stream in fixed point [T, N] the product is added into it instead and the stream is returned.  activation 'relu2':
+        there is no gate, gate_up is an up product [S, T, I] and the operand relu(up)^2."""
         if gate_up.dim() != 3 or gate_up.dtype != _F32 or w.dtype != _BF16:
             return None
         g_splits, t, two_i = gate_up.shape
         n, k = w.shape
-        if two_i != 2 * k or not 0 < t <= self.fused_rows or k % 8:
+        if two_i != (k if activation == "relu2" else 2 * k) or not 0 < t <= self.fused_rows or k % 8:
             return None
         if waves is None and n >= 1536:
             # every workgroup computes its share of x from gate_up's partial sums, and with this many columns there
@@ -463,7 +465,8 @@ class HipKernels(KernelBackend):
         target = self._residual_target(residual, t, n, s)
         out = None if target is not None else torch.empty((s, t, n), dtype=_F32, device=w.device)
         self._run("egpt_gemm_skinny_swiglu", gate_up.data_ptr(), int(g_splits), self._ptr(row_ss), ss_splits, int(hidden),
-                  float(eps), w.data_ptr(), self._ptr(out), self._ptr(target), t, n, k, s, waves, _GATES[activation], self._stream())
+                  float(eps), w.data_ptr(), self._ptr(out), self._ptr(target), t, n, k, s, waves,
+                  _UNGATED_RELU2 if activation == "relu2" else _GATES[activation], self._stream())
         return out if target is None else target
 
     def product_attention(self, part_o, part_ml, w, max_splits=None, waves=None, residual=None):
@@ -931,6 +934,8 @@ class HipKernels(KernelBackend):
                              + ("" if values_are_keys else f" and {nkv} of {dv}"))
         if values_are_keys and (dv != dk or norm_values):
             raise ValueError("values that are the keys as projected have the keys' size and are not normed")
+        if nkv == 0 and (slots is not None or values_out is not None):
+            raise ValueError("rows of queries alone (nkv 0) have nothing to store")
         if pairing not in ("half", "interleaved"):
             raise ValueError(f"unknown pairing '{pairing}' of the rotation (half, interleaved)")
         splits = self._product(proj, "proj", q_out.dtype, t, width)
@@ -1010,8 +1015,19 @@ class HipKernels(KernelBackend):
 
     def window_attention(self, q, out, k_cache, v_cache, block_table, q_start, q_len, kv_len, nq, nkv, dk, dv, page_size,
                          scale, window, keep_first, sink, max_q_len, max_kv_len, dist_bias=None, block=0, slopes=None, softcap=None,
-                         head_gate=None):
+                         head_gate=None, difference=None):
+        """difference (weight, eps, factor): a head's query and key are two maps side by side, dk / 2 wide each, over the same
+        values; the head's output is the difference a1 - weight * a2 of the maps' outputs, divided by its root mean square
+        (eps inside) and multiplied by factor."""
         t = q.shape[0]
+        maps, map_weight, out_scale, out_eps = 1, 0.0, 1.0, 0.0
+        if difference is not None:
+            map_weight, out_eps, out_scale = (float(v) for v in difference)
+            maps = 2
+            if dk % 2:
+                raise ValueError(f"a key of two maps has an even size, not {dk}")
+            if sink is not None or dist_bias is not None or slopes is not None or head_gate is not None:
+                raise ValueError("heads of two maps take no sink, no bias by distance and no gate")
         block = int(block or 0)
         if block < 0:
             raise ValueError(f"block ({block}) must not be negative")
@@ -1050,24 +1066,25 @@ class HipKernels(KernelBackend):
         # (a block of positions bounds the keys that a row sees as a window of that many does)
         reach = min(window, block) if window and block else (window or block)
         shape = self._window_attention_shape(t, b, nq, nkv, dk, dv, page_size, reach, keep_first, max_q_len, max_kv_len,
-                                             q.element_size())
+                                             q.element_size(), maps)
         if shape is not None:
             row_tiles, n_splits = shape
             part_o = part_ml = None
             if n_splits > 1:
-                part_o = torch.empty((n_splits, t, nq, dv), dtype=_F32, device=q.device)
-                part_ml = torch.empty((n_splits, t, nq, 2), dtype=_F32, device=q.device)
+                part_o = torch.empty((n_splits, t, nq, maps, dv), dtype=_F32, device=q.device)
+                part_ml = torch.empty((n_splits, t, nq, maps, 2), dtype=_F32, device=q.device)
             self._run("egpt_window_attention_tiled", q.data_ptr(), out.data_ptr(), self._ptr(part_o), self._ptr(part_ml),
                       k_cache.data_ptr(), v_cache.data_ptr(), block_table.data_ptr(), width, q_start.data_ptr(),
                       q_len.data_ptr(), kv_len.data_ptr(), b, t, nq, nkv, dk, dv, page_size, float(scale), int(window),
                       int(keep_first), self._ptr(sink), self._ptr(dist_bias), dist_far, block, self._ptr(slopes), cap,
-                      self._ptr(head_gate), n_splits, row_tiles, dt, self._stream())
+                      self._ptr(head_gate), maps, map_weight, out_scale, out_eps, n_splits, row_tiles, dt, self._stream())
             return
         # sizes that the matrix-core kernel does not take: the general kernel
         self._run("egpt_window_attention", q.data_ptr(), out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                   block_table.data_ptr(), width, q_start.data_ptr(), q_len.data_ptr(), kv_len.data_ptr(), b, t, nq, nkv,
                   dk, dv, page_size, float(scale), int(window), int(keep_first), self._ptr(sink), self._ptr(dist_bias),
-                  dist_far, block, self._ptr(slopes), cap, self._ptr(head_gate), dt, self._stream())
+                  dist_far, block, self._ptr(slopes), cap, self._ptr(head_gate), maps, map_weight, out_scale, out_eps, dt,
+                  self._stream())
 
 
     # ------------------------------------------------------------------ stream operations beyond the RMS norm
@@ -1149,7 +1166,8 @@ class HipKernels(KernelBackend):
                   self._ptr(rows), weight.data_ptr(), float(eps), out.data_ptr(), n, hidden, dt, self._stream())
         return out, streams if kept is None else kept
 
-    def embed_positions(self, token_ids, positions, table, pos_table, out):
+    def embed_positions(self, token_ids, positions, table, pos_table, out, factor=1.0):
+        """out = factor * table[id] + pos_table[position], as a residual stream of either kind."""
         dt = self._act(table, "table")
         v, h = table.shape
         t = token_ids.shape[0]
@@ -1157,9 +1175,9 @@ class HipKernels(KernelBackend):
         self._need(positions, "positions", _I32, (t,))
         self._need(table, "table")
         self._need(pos_table, "pos_table", table.dtype, (pos_table.shape[0], h))
-        self._need(out, "out", _F32, (t, h))
+        self._need(out, "out", None, (t, h))
         self._run("egpt_embed_positions", token_ids.data_ptr(), positions.data_ptr(), table.data_ptr(), pos_table.data_ptr(),
-                  out.data_ptr(), t, h, v, int(pos_table.shape[0]), dt, self._stream())
+                  float(factor), out.data_ptr(), self._fixed(out, "out"), t, h, v, int(pos_table.shape[0]), dt, self._stream())
 
     def post_norm_add(self, h, y, post_weight, eps, mult, history=None, n_history=0, mix=None, next_weight=None, h_out=None):
         """x = h + mult * LN(y) * post_weight, LN without bias over y's rows (y a product: act [T, H] or float32 partial
@@ -1192,10 +1210,11 @@ class HipKernels(KernelBackend):
                   self._ptr(next_weight), self._ptr(out), t, hidden, dt, self._stream())
         return out
 
-    def ff_activation(self, z, cols, mode, out, coef=None, eps=0.0, gate_col=-1):
+    def ff_activation(self, z, cols, mode, out, coef=None, eps=0.0, gate_col=-1, row_ss=None, hidden=0, norm_eps=0.0):
         """out[t, j] = f(z[t, j]) for j < cols of a product z (act [T, W] or float32 partial sums [S, T, W]): mode
         'relu2' relu(z)^2; 'polynorm' coef[0] N(z) + coef[1] N(z^2) + coef[2] N(z^3) + coef[3], N(u) = u / sqrt(mean(u^2)
-        + eps) over the row's cols values (coef float32 [4]); gate_col >= 0: times sigmoid(z[t, gate_col])."""
+        + eps) over the row's cols values (coef float32 [4]); gate_col >= 0: times sigmoid(z[t, gate_col]).  row_ss: z's rows
+        still lack the factor of a norm that was folded into the product."""
         t, width = z.shape[-2], z.shape[-1]
         dt = self._act(out, "out")
         self._need(out, "out", None, (t, cols))
@@ -1207,7 +1226,7 @@ class HipKernels(KernelBackend):
             self._need(coef, "coef", _F32, (4,))
         if not 0 < cols <= width or not -1 <= gate_col < width:
             raise ValueError(f"{cols} columns and gate column {gate_col} do not fit rows of {width} values")
-        self._run("egpt_ff_activation", z.data_ptr(), splits, int(width), int(cols), modes[mode],
+        self._run("egpt_ff_activation", z.data_ptr(), splits, *self._row_factor(row_ss, splits, t, hidden, norm_eps), int(width), int(cols), modes[mode],
                   self._ptr(coef) if mode == "polynorm" else None, float(eps), int(gate_col), out.data_ptr(), t, dt, self._stream())
 
     def tanh_cap(self, x, cap, scale=1.0):
@@ -1477,28 +1496,39 @@ class HipKernels(KernelBackend):
         return 16 if per_expert <= 24 else (32 if per_expert <= 96 else 64)
 
     def expert_mixture(self, x, router, router_bias, w_gate_up, w_down, top, gated=True, score_all=False, correction=None,
-                       weight_scale=1.0):
+                       weight_scale=1.0, identities=0, groups=1, keep_groups=1, normalized=True, residual=None):
         """float32 [T, H]: for every token the `top` experts with the largest float32 router logits (x router^T + bias),
         weighted by the softmax over those logits; an expert is down(silu(gate x) * (up x)).  w_gate_up [E, 2 ff, H]
         (an expert's gate rows, then its up rows), w_down [E, H, ff].  gated False: an expert is down(relu(up x)^2) and
         w_gate_up is [E, ff, H].  score_all: the scores are the softmax over all experts, the choice goes by score +
-        correction (float32 [E] or None), the weights are the chosen scores over their sum, times weight_scale."""
+        correction (float32 [E] or None), the weights are the chosen scores over their sum (normalized False: as they are),
+        times weight_scale.  identities I: the router has E + I outputs (and the correction E + I numbers), the last I of
+        which hand on x itself.  groups > 1 (with score_all): the outputs are that many groups of neighbours, and only those
+        of the keep_groups groups with the largest score + correction in them can be chosen.  residual: a stream in fixed
+        point [T, H] that the sum is added into (and which is then returned)."""
         t, hidden = x.shape
         dt = self._act(x, "x")
         experts, ff2, _ = w_gate_up.shape
         ff = ff2 // 2 if gated else ff2
+        outputs = experts + int(identities)
+        if identities < 0 or outputs > 1024:
+            raise ValueError(f"{experts} experts and {identities} identity experts are not supported (at most 1024 together)")
         if correction is not None:
-            self._need(correction, "correction", _F32, (experts,))
+            self._need(correction, "correction", _F32, (outputs,))
         self._need(x, "x")
-        self._need(router, "router", x.dtype, (experts, hidden))
+        self._need(router, "router", x.dtype, (outputs, hidden))
         if router_bias is not None:
-            self._need(router_bias, "router_bias", x.dtype, (experts,))
+            self._need(router_bias, "router_bias", x.dtype, (outputs,))
         self._need(w_gate_up, "w_gate_up", x.dtype, (experts, 2 * ff if gated else ff, hidden))
         self._need(w_down, "w_down", x.dtype, (experts, hidden, ff))
-        if not 0 < top <= experts:
-            raise ValueError(f"top ({top}) must be between 1 and the number of experts ({experts})")
-        if experts > 1024:
-            raise ValueError(f"{experts} experts are not supported (at most 1024)")
+        if not 0 < top <= outputs:
+            raise ValueError(f"top ({top}) must be between 1 and the number of experts ({outputs})")
+        if groups < 1 or outputs % groups or not 0 < keep_groups <= groups or outputs // groups * keep_groups < top:
+            raise ValueError(f"{keep_groups} of {groups} groups of {outputs} experts cannot hold {top} choices")
+        if groups > 1 and not score_all:
+            raise ValueError("groups of experts are chosen by scores over all experts")
+        if residual is not None:
+            self._need(residual, "residual", _I64, (t, hidden))
         dev = x.device
         n_rows = t * top
         tile_rows = self._moe_tile_rows(n_rows, experts)
@@ -1510,38 +1540,40 @@ class HipKernels(KernelBackend):
         counts = torch.empty((experts,), dtype=_I32, device=dev)
         act = torch.empty((n_rows, ff), dtype=x.dtype, device=dev)
         y = torch.empty((n_rows, hidden), dtype=_F32, device=dev)
-        out = torch.empty((t, hidden), dtype=_F32, device=dev)
+        out = None if residual is not None else torch.empty((t, hidden), dtype=_F32, device=dev)
         st = self._stream()
         self._run("egpt_moe_route", x.data_ptr(), router.data_ptr(), self._ptr(router_bias), chosen.data_ptr(),
-                  weight.data_ptr(), t, hidden, experts, top, int(bool(score_all)), self._ptr(correction), float(weight_scale), dt, st)
+                  weight.data_ptr(), t, hidden, outputs, top, int(bool(score_all)), self._ptr(correction), float(weight_scale),
+                  int(groups), int(keep_groups), int(bool(normalized)), dt, st)
         self._run("egpt_moe_group", chosen.data_ptr(), row_token.data_ptr(), place.data_ptr(), tiles.data_ptr(),
                   counts.data_ptr(), t, top, experts, tile_rows, st)
         self._run("egpt_moe_gate_up" if gated else "egpt_moe_up", x.data_ptr(), w_gate_up.data_ptr(), row_token.data_ptr(),
                   tiles.data_ptr(), act.data_ptr(), n_rows, hidden, ff, experts, tile_rows, dt, st)
         self._run("egpt_moe_down", act.data_ptr(), w_down.data_ptr(), tiles.data_ptr(), y.data_ptr(), n_rows, hidden, ff,
                   experts, tile_rows, dt, st)
-        self._run("egpt_moe_combine", y.data_ptr(), place.data_ptr(), weight.data_ptr(), out.data_ptr(), t, top, hidden, st)
-        return out
+        self._run("egpt_moe_combine", y.data_ptr(), x.data_ptr(), place.data_ptr(), weight.data_ptr(), self._ptr(out),
+                  self._ptr(residual), t, top, hidden, dt, st)
+        return out if residual is None else residual
 
     wide_rows_from = 16384          # rows of a step from which the window attention gives a wavefront 32 of them,
     wide_rows_key_size = 192        # if its keys are wider than this
 
     @staticmethod
-    def _window_attention_shape(t, b, nq, nkv, dk, dv, page_size, window, keep_first, max_q_len, max_kv_len, elem):
+    def _window_attention_shape(t, b, nq, nkv, dk, dv, page_size, window, keep_first, max_q_len, max_kv_len, elem, maps=1):
         """(row tiles per workgroup, splits of the keys) of the matrix-core window attention, or None where its sizes
         are not covered.  Steps of many rows: 32 rows to a wavefront.  Steps of so few rows that their workgroups do
         not fill the GPU (single tokens, short portions): the chunks of keys that a workgroup's rows see are dealt
         over several workgroups, a chunk or more each, and a second kernel folds their results."""
         e = 16 // elem
-        if dk % e or dk > 256 or dv % 16 or dv > 256 or page_size % 16:
+        if dk % (e * maps) or dk > 256 or dv % 16 or dv > 256 or page_size % 16:
             return None
         chunk = 64 if elem == 2 else 32
         group = nq // nkv
         # (measured, us for a 2,048-token prompt behind nothing, 16 / 32 rows to a wavefront: 14 heads on 2 of 64 + 64, window
         # 1,024: 70 / 73; 14 on 1 of 160 + 128: 96 / 137; 16 on 4 of 128 + 128, window 2,048: 162 / 191; 16 on 1 of 256 + 192:
         # 310 / 274)
-        row_tiles = 8 if dk > HipKernels.wide_rows_key_size and t * group * nkv >= HipKernels.wide_rows_from else 4
-        krow = -(-dk // (4 * e)) * 4 * e + e
+        row_tiles = 8 if maps == 1 and dk > HipKernels.wide_rows_key_size and t * group * nkv >= HipKernels.wide_rows_from else 4
+        krow = maps * (-(-(dk // maps) // (4 * e)) * 4 * e) + e
         dv_tiles = next(n for n in (2, 4, 6, 8, 12, 16) if n * 16 >= dv)
         lds = lambda tiles: ((16 * tiles + chunk) * krow + dv_tiles * 16 * (chunk + e)) * elem
         if row_tiles == 8 and lds(8) > 160 * 1024:

@@ -108,7 +108,7 @@ class GQAttention(Mixer):
             fused = None
             rms = x.rms()
             if rms is not None and rot is not None:
-                fused = k.product_normed(x.h, x.delta, rms[0], self.w_qkv)
+                fused = k.product_normed(x.h, x.delta, rms[0], self.w_qkv, weight_offset=rms[2])
             if fused is not None:
                 prod, row_ss, h_new = fused
                 x.applied(h_new)

@@ -51,6 +51,15 @@ class CacheNeed:
     window: int | None = None
     keep_first: int = 0
 
+    def joined(self, other: "CacheNeed") -> "CacheNeed | None":
+        """What serves two mixers that share one cache: the same tensors, kept for as long as either reads them (None:
+        the tensors differ)."""
+        if self.tensors != other.tensors:
+            return None
+        if self.window is None or other.window is None:
+            return CacheNeed(self.tensors)
+        return CacheNeed(self.tensors, max(self.window, other.window), max(self.keep_first, other.keep_first))
+
     @classmethod
     def keys_and_values(cls, n_kv_heads: int, head_dim: int, window: int | None = None,
                         value_dim: int | None = None, keep_first: int = 0) -> "CacheNeed":
@@ -147,9 +156,9 @@ class Norm(Part):
     a norm hands it to the backend (`add_rmsnorm`; or `residual_add` and `residual_values` for a norm that the
     backend has no kernel for) and never reads it by itself."""
 
-    def rms_params(self) -> tuple[torch.Tensor, float] | None:
-        """(weight, eps) if this norm is y = x / sqrt(mean(x^2) + eps) * weight, so that a part may fold it into its
-        own first kernel; None for any other norm."""
+    def rms_params(self) -> tuple[torch.Tensor, float, float] | None:
+        """(weight, eps, offset) if this norm is y = x / sqrt(mean(x^2) + eps) * (offset + weight), so that a part may fold
+        it into its own first kernel; None for any other norm."""
         return None
 
     def forward(self, h: torch.Tensor, delta: torch.Tensor | None) -> torch.Tensor:
@@ -163,7 +172,7 @@ class PendingNorm:
     """x = norm(h + delta), not computed yet.
 
     A block hands this to a mixer or feed-forward that sets `takes_pending_norm`: such a part may fold the
-    addition and the norm into its own first kernel (`rms()` gives it the norm's weight and eps when the
+    addition and the norm into its own first kernel (`rms()` gives it the norm's weight, eps and offset when the
     norm is an RMSNorm) and must then call `applied(h_new)` with the updated residual stream; or it calls
     `materialize()` to get x as a tensor, as any other part would have been given.
     """
@@ -173,7 +182,7 @@ class PendingNorm:
         self.h_after: torch.Tensor | None = None
 
     def rms(self):
-        """(weight, eps) if the norm is y = x / rms(x) * weight, else None."""
+        """(weight, eps, offset) if the norm is y = x / rms(x) * (offset + weight), else None."""
         return self.norm.rms_params()
 
     def applied(self, h_new: torch.Tensor) -> None:

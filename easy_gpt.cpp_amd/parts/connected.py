@@ -52,7 +52,7 @@ class HyperConnection(StreamConnection):
             self.scale = take(self.scale_name)
 
     def read(self, h, delta, norm):
-        weight, eps = norm.rms_params()
+        weight, eps, _ = norm.rms_params()
         return kernels.backend().connect_streams(h, delta, self.read_weights, self.streams, None, weight, eps)
 
     def written(self, y) -> kernels.StreamUpdate:
@@ -69,8 +69,8 @@ class ConnectedBlock(Block):
         super().__init__(mixer, feed_forward, norms)
         self.connections = dict(connections)
         for slot in self.norm_slots:
-            if not isinstance(self.norms[slot], RMSNorm):
-                raise ValueError(f"the connected arrangement's norm '{slot}' must be an RMS norm")
+            if not isinstance(self.norms[slot], RMSNorm) or self.norms[slot].weight_offset:
+                raise ValueError(f"the connected arrangement's norm '{slot}' must be an RMS norm whose weight is stored as it is")
 
     def parts(self):
         return super().parts() + [self.connections[s] for s in self.connection_slots]

@@ -88,14 +88,16 @@ class ScaledTokenEmbedding(TokenEmbedding):
 
 
 class PositionedTokenEmbedding(TokenEmbedding):
-    """x[t, :] = E[id_t, :] + P[position_t, :] with a learned vector per position (the tensor `prefix + position_name`,
-    [max_positions, H]), added in float32 and written as a float32 residual stream.  A request cannot grow beyond the
-    table's rows (the model's `max_position`)."""
+    """x[t, :] = scale * E[id_t, :] + P[position_t, :] with a learned vector per position (the tensor `prefix +
+    position_name`, [max_positions, H]), added in float32 and written as a float32 residual stream, or with `any_stream`
+    as the kind that the backend names for the step's size (for layers that take either).  A request cannot grow beyond
+    the table's rows (the model's `max_position`)."""
 
     def __init__(self, prefix: str, hidden_size: int, vocab_size: int, max_positions: int, name: str = "weight",
-                 position_name: str = "pos"):
+                 position_name: str = "pos", scale: float = 1.0, any_stream: bool = False):
         super().__init__(prefix, hidden_size, vocab_size, name)
         self.max_positions = int(max_positions)
+        self.scale, self.any_stream = float(scale), bool(any_stream)
         self.position_name = position_name
         self.position_table: torch.Tensor | None = None
 
@@ -109,8 +111,10 @@ class PositionedTokenEmbedding(TokenEmbedding):
 
     def forward(self, ctx) -> torch.Tensor:
         token_ids = ctx.token_ids
-        out = torch.empty((token_ids.shape[0], self.hidden_size), device=token_ids.device, dtype=torch.float32)
-        kernels.backend().embed_positions(token_ids, ctx.positions, self.table, self.position_table, out)
+        k = kernels.backend()
+        dtype = k.residual_dtype(token_ids.shape[0], self.table.dtype) if self.any_stream else torch.float32
+        out = torch.empty((token_ids.shape[0], self.hidden_size), device=token_ids.device, dtype=dtype)
+        k.embed_positions(token_ids, ctx.positions, self.table, self.position_table, out, factor=self.scale)
         return out
 
 

@@ -62,7 +62,7 @@ class SwiGLU(FeedForward):
             rms = x.rms()
             fused = None
             if rms is not None and self.intermediate_size % 8 == 0:
-                fused = k.product_normed(x.h, x.delta, rms[0], self.w_gate_up)
+                fused = k.product_normed(x.h, x.delta, rms[0], self.w_gate_up, weight_offset=rms[2])
             if fused is not None:
                 gate_up, row_ss, h_new = fused
                 x.applied(h_new)
@@ -98,9 +98,11 @@ class ActivatedFeedForward(FeedForward):
     `coef`.  row_gate: the name of a [1, H] tensor g; the token's output is multiplied by sigmoid(g . x), one number
     per token (its weights ride as one more row of the up matrix, and since the down product is linear the factor is
     applied to the activated inner values).  The up product stays unrounded (float32) until the activation has used it;
-    the statistics and the activation are float32.  The output is float32 partial sums."""
+    the statistics and the activation are float32.  The output is float32 partial sums, or goes into the residual stream
+    of a pending norm."""
 
     graph_safe = True
+    takes_pending_norm = True
 
     def __init__(self, prefix: str, hidden_size: int, intermediate_size: int, activation: str = "relu2", eps: float = 0.0,
                  names: tuple[str, str] = ("up", "down"), coef: str = "act", row_gate: str | None = None):
@@ -135,10 +137,32 @@ class ActivatedFeedForward(FeedForward):
     def forward(self, x, ctx=None):
         k = kernels.backend()
         i = self.intermediate_size
-        z = k.product(x, self.w_up, unrounded=True)
-        act = torch.empty((x.shape[0], i), dtype=x.dtype, device=x.device)
-        k.ff_activation(z, i, self.activation, act, coef=self.coef, eps=self.eps, gate_col=i if self.row_gate is not None else -1)
-        out = k.product(act, self.w_down, unrounded=True)
+        residual, factor = None, {}
+        z = None
+        if isinstance(x, PendingNorm):
+            # with few tokens the norm folds into the up product's staging of x, and the rows' 1/rms factor that this
+            # leaves (and the squared relu, where the kernel has it) into what reads that product
+            pending, rms = x, x.rms()
+            fused = k.product_normed(x.h, x.delta, rms[0], self.w_up, weight_offset=rms[2]) if rms is not None else None
+            if fused is not None:
+                z, row_ss, h_new = fused
+                x.applied(h_new)
+                factor = dict(row_ss=row_ss, hidden=self.hidden_size, norm_eps=rms[1])
+                residual = pending.residual()
+                if self.activation == "relu2" and self.row_gate is None:
+                    out = k.product_swiglu(z, row_ss, self.hidden_size, rms[1], self.w_down, residual=residual, activation="relu2")
+                    if out is not None:
+                        return None if out is residual else out
+            else:
+                x = x.materialize()
+                residual = pending.residual()
+        if z is None:
+            z = k.product(x, self.w_up, unrounded=True)
+        act = torch.empty((z.shape[-2], i), dtype=self.w_up.dtype, device=z.device)
+        k.ff_activation(z, i, self.activation, act, coef=self.coef, eps=self.eps, gate_col=i if self.row_gate is not None else -1, **factor)
+        out = k.product(act, self.w_down, unrounded=True, residual=residual)
+        if out is residual and residual is not None:
+            return None
         return out if out.dim() == 3 else out.float()[None]
 
 

@@ -1,5 +1,6 @@
 """Attention mixers that treat single heads before the scores: norms per head, a window that keeps the first tokens,
-latent keys and values, a sink in the softmax, a tanh cap on the scores, values mixed with an earlier layer's, an output gate.
+latent keys and values, a sink in the softmax, a tanh cap on the scores, values mixed with an earlier layer's, an output gate,
+heads that take the difference of two softmax maps, another layer's keys and values.
 
 Both mixers here run the same three steps through the backend: one product for everything that reads the mixer's
 input, a preparation kernel that norms, rotates and stores into the cache pages, and `window_attention`, the
@@ -10,7 +11,12 @@ heads share, whose values are divided by their root mean square before they are 
 request's first tokens visible: position i sees j <= i if i - j < window or j < keep_first.  Each of these is an option;
 others are a rotation, a sink that is learned or constant, a cap on the scores, an output gate per value or per head, and a
 mixture of the layer's values with those that the first layer of the run order that mixes values made of the same tokens
-(`mixes_values`: they stay in the step's shared values, float32, and the mixed ones are cached).
+(`mixes_values`: they stay in the step's shared values, float32, and the mixed ones are cached).  With `difference` a head has two
+query/key maps of `key_dim` each over the same values, laid out [map 1 | map 2] in the projections and in the cached keys; with a1,
+a2 the maps' attention outputs the head gives o = a1 - lambda a2, divided by its root mean square and multiplied by
+1 - difference, where lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + difference is one number for the layer, made of four learned
+vectors when the weights are loaded.  A layer with `shares_cache` has no key and value tensors: it reads the pages that another
+entry of the run order wrote (`RunSpec(cache=j, writes_cache=False)`) with its own queries and its own mask.
 
 `LatentAttention`: every token leaves one latent vector c (RMS-normed, `latent_dim` wide) and one rotated key part
 that all heads share; a head's unrotated key is W_uk c and its value W_uv c.  Only c and the rotated part are cached.
@@ -51,7 +57,7 @@ def _input_product(x, w, hidden_size) -> _Projected:
     k = kernels.backend()
     if isinstance(x, PendingNorm):
         rms = x.rms()
-        fused = k.product_normed(x.h, x.delta, rms[0], w) if rms is not None else None
+        fused = k.product_normed(x.h, x.delta, rms[0], w, weight_offset=rms[2]) if rms is not None else None
         if fused is not None:
             proj, row_ss, h_new = fused
             x.applied(h_new)
@@ -84,7 +90,8 @@ class NormedAttention(_TwoPhases):
                  scale: float, eps: float, window: int | None = None, keep_first: int = 0, norm_queries_keys: bool = True,
                  norm_values: bool = False, norm_weighted: bool = True, norm_after_rotation: bool = False,
                  position: PartSpec | None = None, values_are_keys: bool = False, sink: bool | float = False,
-                 gated: bool | str = False, softcap: float | None = None, mixes_values: bool = False, names: dict | None = None):
+                 gated: bool | str = False, softcap: float | None = None, mixes_values: bool = False, names: dict | None = None,
+                 difference: float | None = None, shares_cache: bool = False):
         """norm_weighted False: queries and keys are divided by their root mean square and no more (no weight tensors);
         position: a rotary encoding of queries and keys (None: no rotation), applied behind the norm, or before it
         with norm_after_rotation; values_are_keys: there is no value projection, a value head is its key head as
@@ -92,8 +99,10 @@ class NormedAttention(_TwoPhases):
         same constant score for every head (a number); gated: the heads' outputs are multiplied by sigmoid(W_g x), one number
         per value, or with 'heads' one per head; softcap c: a score s becomes c tanh(s / c); mixes_values: the cached values are
         (1 - lambda) v + lambda v_first with lambda a tensor of one number, v_first the values of the run order's first layer
-        that mixes (whose own lambda is not used).  names: tensor names behind `prefix` of q, k, v, o, the weights q_norm,
-        k_norm, and sink, gate, value_mix."""
+        that mixes (whose own lambda is not used); difference: a head is the difference of two maps (key_dim is one map's
+        size), this number is lambda's constant part; shares_cache: queries only, the keys and values are another layer's.
+        names: tensor names behind `prefix` of q, k, v, o, the weights q_norm, k_norm, and sink, gate, value_mix, and lambda_q1,
+        lambda_k1, lambda_q2, lambda_k2."""
         if n_heads % n_kv_heads:
             raise ValueError(f"n_heads ({n_heads}) must be a multiple of n_kv_heads ({n_kv_heads})")
         widest = kernels.KernelBackend.max_window_attention_dim
@@ -103,6 +112,16 @@ class NormedAttention(_TwoPhases):
             raise ValueError(f"values that are the keys have the keys' size: value_dim ({value_dim}) must be {key_dim}")
         if values_are_keys and norm_values:
             raise ValueError("values that are the keys as projected are not normed")
+        self.difference, self.shares_cache = None if difference is None else float(difference), bool(shares_cache)
+        self.map_dim, self.map_weight = int(key_dim), 0.0
+        if self.difference is not None:
+            key_dim = 2 * int(key_dim)                # a head's key in the projections, the cache and the kernels
+            if key_dim > widest:
+                raise ValueError(f"two maps of {self.map_dim} to a key are not supported by the attention kernel (at most {widest} together)")
+            if sink is not False or gated or norm_queries_keys or position is not None or values_are_keys:
+                raise ValueError("heads that take the difference of two maps have no sink, gate, norms or rotation of queries and keys")
+        if self.shares_cache and (norm_values or values_are_keys or mixes_values):
+            raise ValueError("a layer that reads another's keys and values makes none of its own")
         self.prefix, self.hidden_size = prefix, int(hidden_size)
         self.n_heads, self.n_kv_heads = int(n_heads), int(n_kv_heads)
         self.key_dim, self.value_dim = int(key_dim), int(value_dim)
@@ -120,10 +139,13 @@ class NormedAttention(_TwoPhases):
         self.mixes_values, self.mix = bool(mixes_values), 0.0
         self.position = None if position is None else make_part("position_encoding", position, head_dim=self.key_dim)
         self.names = dict(q="q_proj.weight", k="k_proj.weight", v="v_proj.weight", o="o_proj.weight",
-                          q_norm="q_norm.weight", k_norm="k_norm.weight", sink="sink", gate="g_proj.weight", value_mix="value_mix")
+                          q_norm="q_norm.weight", k_norm="k_norm.weight", sink="sink", gate="g_proj.weight", value_mix="value_mix",
+                          lambda_q1="lambda_q1", lambda_k1="lambda_k1", lambda_q2="lambda_q2", lambda_k2="lambda_k2")
         self.names.update(names or {})
-        self.q_width, self.k_width = self.n_heads * self.key_dim, self.n_kv_heads * self.key_dim
-        self.v_width = 0 if self.values_are_keys else self.n_kv_heads * self.value_dim
+        self.q_width = self.n_heads * self.key_dim
+        self.stored_heads = 0 if self.shares_cache else self.n_kv_heads        # key/value heads that the layer makes
+        self.k_width = self.stored_heads * self.key_dim
+        self.v_width = 0 if self.values_are_keys else self.stored_heads * self.value_dim
         self.out_width = self.n_heads * self.value_dim
         self.w_qkv = self.w_o = self.q_weight = self.k_weight = self.sink = None
 
@@ -132,13 +154,18 @@ class NormedAttention(_TwoPhases):
 
     def param_specs(self):
         p, h, n = self.prefix, self.hidden_size, self.names
-        specs = [ParamSpec(p + n["q"], (self.q_width, h)), ParamSpec(p + n["k"], (self.k_width, h))]
-        if not self.values_are_keys:
-            specs.append(ParamSpec(p + n["v"], (self.v_width, h)))
+        specs = [ParamSpec(p + n["q"], (self.q_width, h))]
+        if not self.shares_cache:
+            specs.append(ParamSpec(p + n["k"], (self.k_width, h)))
+            if not self.values_are_keys:
+                specs.append(ParamSpec(p + n["v"], (self.v_width, h)))
         specs.append(ParamSpec(p + n["o"], (h, self.out_width)))
         if self.norm_queries_keys and self.norm_weighted:
-            specs += [ParamSpec(p + n["q_norm"], (self.key_dim,), role="norm_scale"),
-                      ParamSpec(p + n["k_norm"], (self.key_dim,), role="norm_scale")]
+            specs.append(ParamSpec(p + n["q_norm"], (self.key_dim,), role="norm_scale"))
+            if not self.shares_cache:
+                specs.append(ParamSpec(p + n["k_norm"], (self.key_dim,), role="norm_scale"))
+        if self.difference is not None:
+            specs += [ParamSpec(p + n[x], (self.map_dim,), role="bias", dtype="float32") for x in self._lambdas]
         if self.has_sink:
             specs.append(ParamSpec(p + n["sink"], (self.n_heads,), role="bias", dtype="float32"))
         if self.gated or self.gate_per_head:
@@ -149,15 +176,22 @@ class NormedAttention(_TwoPhases):
             specs += self.position.param_specs()
         return specs
 
+    _lambdas = ("lambda_q1", "lambda_k1", "lambda_q2", "lambda_k2")
+
     def load(self, get, dtype, device):
         p, n = self.prefix, self.names
-        which = ["q", "k"] + ([] if self.values_are_keys else ["v"]) + (["gate"] if self.gated or self.gate_per_head else [])
+        made = [] if self.shares_cache else (["k"] if self.values_are_keys else ["k", "v"])
+        which = ["q"] + made + (["gate"] if self.gated or self.gate_per_head else [])
         w = torch.cat([get(p + n[x]).to(dtype) for x in which], dim=0)      # one product serves all that reads x
         self.w_qkv = w.to(device).contiguous()
         self.w_o = self._to(get(p + n["o"]), "compute", dtype, device)
         if self.norm_queries_keys and self.norm_weighted:
             self.q_weight = self._to(get(p + n["q_norm"]), "compute", dtype, device)
-            self.k_weight = self._to(get(p + n["k_norm"]), "compute", dtype, device)
+            if not self.shares_cache:
+                self.k_weight = self._to(get(p + n["k_norm"]), "compute", dtype, device)
+        if self.difference is not None:
+            q1, k1, q2, k2 = (get(p + n[x]).to(torch.float64) for x in self._lambdas)
+            self.map_weight = float(torch.exp((q1 * k1).sum()) - torch.exp((q2 * k2).sum())) + self.difference
         if self.has_sink:
             self.sink = get(p + n["sink"]).to(torch.float32).to(device).contiguous()
         elif self.constant_sink is not None:
@@ -179,6 +213,8 @@ class NormedAttention(_TwoPhases):
         return kernels.backend().product(self._heads_out(p, ctx, cache), self.w_o, unrounded=True), None
 
     def _heads_out(self, p, ctx, cache):
+        if cache.writes and self.shares_cache:
+            raise RuntimeError("a layer that reads another's keys and values must not write its cache")
         k = kernels.backend()
         t = p.t
         q = torch.empty((t, self.q_width), dtype=p.dtype, device=p.device)
@@ -207,8 +243,10 @@ class NormedAttention(_TwoPhases):
         scores = {}
         if self.softcap is not None or head_gate is not None:
             scores = dict(softcap=self.softcap, head_gate=head_gate)
+        if self.difference is not None:
+            scores.update(difference=(self.map_weight, self.eps, 1.0 - self.difference))
         k.head_norm_store(p.proj, q, self.q_weight, self.k_weight, self.eps, self.norm_values,
-                          cache.slots if cache.writes else None, cache.k, cache.v, self.n_heads, self.n_kv_heads,
+                          cache.slots if cache.writes else None, cache.k, cache.v, self.n_heads, self.stored_heads,
                           self.key_dim, self.value_dim, cache.page_size, **p.factor, **rotation)
         attn = torch.empty((t, self.out_width), dtype=p.dtype, device=p.device)
         k.window_attention(q, attn, cache.k, cache.v, cache.block_table, ctx.q_start, ctx.q_len, ctx.kv_len,

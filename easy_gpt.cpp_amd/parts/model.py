@@ -75,8 +75,11 @@ class Model:
             else:
                 if run.cache is None:
                     raise ValueError(f"run order entry {i}: layer {run.layer}'s mixer needs a cache id")
-                if run.cache in needs and needs[run.cache] != need:
-                    raise ValueError(f"cache {run.cache} is shared by mixers with different needs")
+                if run.cache in needs:
+                    # (mixers that share a cache may look back differently far: it keeps what the farthest needs)
+                    need = needs[run.cache].joined(need)
+                    if need is None:
+                        raise ValueError(f"cache {run.cache} is shared by mixers with different needs")
                 if run.writes_cache:
                     if run.cache in writers:
                         raise ValueError(f"cache {run.cache} is written by two run-order entries")

@@ -2,7 +2,8 @@
 
 Formula as the reference computes it (/root/reference/src/models/norm.cpp:30-62,
 CUDA form /root/reference/src/cuda/ops/self_attn_detail.cuh:385-418):
-ss = sum_j x_j^2 in float32, inv = 1 / sqrt(ss / H + eps), y_j = x_j * inv * w_j.
+ss = sum_j x_j^2 in float32, inv = 1 / sqrt(ss / H + eps), y_j = x_j * inv * w_j.  A design may store the weight as its
+distance from one (`weight_offset`): y_j = x_j * inv * (weight_offset + w_j), the sum in float32.
 The reference fixes eps = 1e-6 in code (norm.cpp:41); here it is a parameter.
 """
 from __future__ import annotations
@@ -17,31 +18,36 @@ from .spec import ParamSpec
 class RMSNorm(Norm):
     graph_safe = True
 
-    def __init__(self, prefix: str, hidden_size: int, eps: float, name: str = "weight"):
+    def __init__(self, prefix: str, hidden_size: int, eps: float, name: str = "weight", weight_offset: float = 0.0):
         self.prefix = prefix
         self.hidden_size = int(hidden_size)
-        self.eps = float(eps)
+        self.eps, self.weight_offset = float(eps), float(weight_offset)
         self.name = name                   # the weight is the tensor `prefix + name`
         self.weight: torch.Tensor | None = None
 
     def param_specs(self):
         h = self.hidden_size
-        return [ParamSpec(self.prefix + self.name, (h,), role="norm_scale", alt_shapes=((h, 1),))]
+        # (random weights: what multiplies lies around one)
+        role = "bias" if self.weight_offset == 1.0 else "norm_scale"
+        return [ParamSpec(self.prefix + self.name, (h,), role=role, alt_shapes=((h, 1),))]
 
     def load(self, get, dtype, device):
         self.weight = self._to(get(self.prefix + self.name).reshape(self.hidden_size), "compute", dtype, device)
 
     def rms_params(self):
-        return self.weight, self.eps
+        return self.weight, self.eps, self.weight_offset
+
+    def _offset(self):
+        return dict(weight_offset=self.weight_offset) if self.weight_offset else {}
 
     def forward(self, h, delta):
         out = torch.empty(h.shape, dtype=self.weight.dtype, device=h.device)
-        kernels.backend().add_rmsnorm(h, delta, self.weight, self.eps, out)
+        kernels.backend().add_rmsnorm(h, delta, self.weight, self.eps, out, **self._offset())
         return out
 
     def forward_rows(self, h, delta, rows):
         out = torch.empty((rows.shape[0], h.shape[1]), dtype=self.weight.dtype, device=h.device)
-        kernels.backend().rows_add_rmsnorm(h, delta, rows, self.weight, self.eps, out)
+        kernels.backend().rows_add_rmsnorm(h, delta, rows, self.weight, self.eps, out, **self._offset())
         return out
 
 

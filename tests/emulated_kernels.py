@@ -31,21 +31,21 @@ class EmulatedKernels(KernelBackend):
     def embed(self, token_ids, table, out):
         out.copy_(table[token_ids.long()].to(out.dtype))
 
-    def add_rmsnorm(self, h, delta, weight, eps, out):
+    def add_rmsnorm(self, h, delta, weight, eps, out, weight_offset=0.0):
         delta = _whole(delta)
         if delta is not None:
             h.add_(delta.to(h.dtype))
         x = h.to(F64)
         inv = 1.0 / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
-        out.copy_((x * inv * weight.to(F64)).to(out.dtype))
+        out.copy_((x * inv * (weight.to(F64) + weight_offset)).to(out.dtype))
 
-    def rows_add_rmsnorm(self, h, delta, rows, weight, eps, out):
+    def rows_add_rmsnorm(self, h, delta, rows, weight, eps, out, weight_offset=0.0):
         delta = _whole(delta)
         x = h[rows.long()].to(F64)
         if delta is not None:
             x = (h[rows.long()] + delta[rows.long()].to(h.dtype)).to(F64)
         inv = 1.0 / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
-        out.copy_((x * inv * weight.to(F64)).to(out.dtype))
+        out.copy_((x * inv * (weight.to(F64) + weight_offset)).to(out.dtype))
 
     def linear(self, x, w, bias, out):
         y = x.to(F64) @ w.to(F64).T
@@ -213,7 +213,22 @@ class EmulatedKernels(KernelBackend):
 
     def window_attention(self, q, out, k_cache, v_cache, block_table, q_start, q_len, kv_len, nq, nkv, dk, dv, page_size,
                          scale, window, keep_first, sink, max_q_len, max_kv_len, dist_bias=None, block=0, slopes=None,
-                         softcap=None, head_gate=None):
+                         softcap=None, head_gate=None, difference=None):
+        if difference is not None:
+            # each map as heads of its own, then their difference
+            weight, eps, factor = difference
+            t, half = q.shape[0], dk // 2
+            q2 = q.view(t, nq, 2, half)
+            maps = []
+            for m in range(2):
+                a = torch.zeros((t, nq * dv), dtype=F64)
+                self.window_attention(q2[:, :, m].reshape(t, nq * half), a, k_cache[..., m * half : (m + 1) * half], v_cache, block_table,
+                                      q_start, q_len, kv_len, nq, nkv, half, dv, page_size, scale, window, keep_first, None, max_q_len,
+                                      max_kv_len, block=block, softcap=softcap)
+                maps.append(a.view(t, nq, dv))
+            a = maps[0] - weight * maps[1]
+            out.copy_((a / torch.sqrt((a * a).mean(-1, keepdim=True) + eps) * factor).reshape(t, nq * dv).to(out.dtype))
+            return
         group = nq // nkv
         q_all = q.view(q.shape[0], nq, dk).to(F64)
         for b in range(q_start.shape[0]):
@@ -403,7 +418,7 @@ class EmulatedKernels(KernelBackend):
         return out[None]
 
     def expert_mixture(self, x, router, router_bias, w_gate_up, w_down, top, gated=True, score_all=False, correction=None,
-                       weight_scale=1.0):
+                       weight_scale=1.0, identities=0, groups=1, keep_groups=1, normalized=True):
         xx = x.to(F64)
         z = xx @ router.to(F64).T
         if router_bias is not None:
@@ -411,9 +426,14 @@ class EmulatedKernels(KernelBackend):
         if score_all:
             sc = torch.softmax(z, dim=-1)
             pick = sc if correction is None else sc + correction.to(F64)
+            if groups > 1:
+                parts = pick.view(x.shape[0], groups, -1)
+                best = torch.argsort(-parts.max(-1).values, dim=-1, stable=True)[:, :keep_groups]
+                kept = torch.zeros((x.shape[0], groups), dtype=torch.bool).scatter_(1, best, True)
+                pick = parts.masked_fill(~kept[:, :, None], float("-inf")).reshape(pick.shape)
             idx = torch.argsort(-pick, dim=-1, stable=True)[:, :top]
             val = torch.gather(sc, -1, idx)
-            wt = val / (val.sum(-1, keepdim=True) + 1e-20) * weight_scale
+            wt = (val / (val.sum(-1, keepdim=True) + 1e-20) if normalized else val) * weight_scale
         else:
             val, idx = torch.topk(z, top, dim=-1)
             wt = torch.softmax(val, dim=-1)
@@ -422,6 +442,9 @@ class EmulatedKernels(KernelBackend):
         for t in range(x.shape[0]):
             for c in range(top):
                 e = int(idx[t, c])
+                if e >= w_gate_up.shape[0]:
+                    out[t] += wt[t, c] * xx[t]
+                    continue
                 gu = w_gate_up[e].to(F64) @ xx[t]
                 if gated:
                     act = (gu[:ff] * torch.sigmoid(gu[:ff]) * gu[ff:]).to(x.dtype).to(F64)
@@ -446,8 +469,8 @@ class EmulatedKernels(KernelBackend):
         out = u / torch.sqrt((u * u).mean(-1, keepdim=True) + eps) * weight.to(F64)
         return out.to(weight.dtype), kept
 
-    def embed_positions(self, token_ids, positions, table, pos_table, out):
-        out.copy_((table[token_ids.long()].to(F64) + pos_table[positions.long()].to(F64)).to(out.dtype))
+    def embed_positions(self, token_ids, positions, table, pos_table, out, factor=1.0):
+        out.copy_((table[token_ids.long()].to(F64) * factor + pos_table[positions.long()].to(F64)).to(out.dtype))
 
     def post_norm_add(self, h, y, post_weight, eps, mult, history=None, n_history=0, mix=None, next_weight=None, h_out=None):
         def normed(x, w):
