@@ -487,6 +487,31 @@ def tipezen_config(width, heads, kv_heads, hd, s_heads, s_dim, s_vdim, inner, wi
             "layers": [retention, attention] * (DESIGN_LAYERS // 2)}
 
 
+# `--design karesun`: the Karesun design (window attention whose heads are the difference of two maps with capped scores, every
+# second layer on the keys and values of the one before; dense layers with a squared relu and mixtures of gated experts in turn,
+# chosen within groups, with identity experts; a learned vector per position) beside the two models it shares most with at
+# equal sizes: Nebanex (experts of the same sizes) and Tipezen (window attention with capped scores, of the same window), and beside
+# the Qwen2 model of the same width, heads and inner width per token.  A head's two maps are half as wide as its values, so
+# that the projections and the cache are those of the other models.
+KARESUN_ROUTER = {"w896": (2, 3, 2), "w2048": (4, 6, 3)}         # identity experts, groups of outputs, groups kept
+
+
+def karesun_config(width, heads, kv_heads, hd, experts, top, ff, inner, window, identity, groups, keep) -> dict:
+    def mixer(own):
+        m = {"heads": heads, "kv_heads": kv_heads, "dim": hd // 2, "vdim": hd, "scale": (hd // 2) ** -0.5, "softcap": 50.0,
+             "mask": {"size": window}, "diff": 0.3}
+        return m if own is None else dict(m, kv_from=own)
+
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top, "scale": 2.5, "identity": identity,
+                                                            "groups": {"count": groups, "keep": keep}}}
+    layers = []
+    for i in range(0, DESIGN_LAYERS, 2):
+        layers += [{"type": "attention", "mixer": mixer(None), "mlp": {"kind": "dense", "ff": inner}},
+                   {"type": "attention", "mixer": mixer(i), "mlp": moe}]
+    return {"architecture": "Karesun", "vocab": DESIGN_VOCAB, "width": width, "max_positions": 8192, "norm": {"eps": 1e-6},
+            "embedding": {"scale": 3.0}, "layers": layers}
+
+
 def bubetar_sizes():
     """(label, sizes of the Bubetar model of the comparison)"""
     for s, d in zip(NEBANEX_SIZES, DESIGN_SIZES):
@@ -512,6 +537,13 @@ def design_models(design):
             sizes = (*of[:8], of[10], 4)
             width, heads, kv_heads, hd, inner = *sizes[:4], sizes[7]
             yield label, dict(zip(keys, sizes)), tipezen_config(*sizes), (width, inner, heads, kv_heads, hd)
+    elif design == "karesun":
+        keys = ("width", "heads", "kv_heads", "head", "experts", "chosen", "expert_inner", "inner", "window", "identities", "groups", "kept")
+        for s, d in zip(NEBANEX_SIZES, DESIGN_SIZES):
+            label, width, heads, kv_heads, hd = s[:5]
+            inner = s[9] * s[10] + s[11]
+            sizes = (width, heads, kv_heads, hd, s[8], s[9], s[10], inner, d[8], *KARESUN_ROUTER[label])
+            yield label, dict(zip(keys, sizes)), karesun_config(*sizes), (width, inner, heads, kv_heads, hd)
     else:
         keys = ("width", "heads", "kv_heads", "head", "state_heads", "state_key", "state_value", "experts", "chosen",
                 "expert_inner", "shared_inner")
@@ -535,8 +567,9 @@ def design_comparison(args) -> dict:
         sizes[label] = named
         models = {
             design: design_cfg,
-            **({"nebanex": nebanex_config(*next(s for s in NEBANEX_SIZES if s[0] == label)[1:])} if design in ("kezolix", "bubetar") else {}),
+            **({"nebanex": nebanex_config(*next(s for s in NEBANEX_SIZES if s[0] == label)[1:])} if design in ("kezolix", "bubetar", "karesun") else {}),
             **({"bubetar": bubetar_config(*dict(bubetar_sizes())[label])} if design == "tipezen" else {}),
+            **({"tipezen": next(c for name, _, c, _ in design_models("tipezen") if name == label)} if design == "karesun" else {}),
             "qwen2": dict(QWEN25_05B, hidden_size=width, intermediate_size=inner, num_attention_heads=heads,
                           num_key_value_heads=kv_heads, head_dim=hd, num_hidden_layers=DESIGN_LAYERS, vocab_size=DESIGN_VOCAB,
                           tie_word_embeddings=False),
@@ -602,9 +635,10 @@ def main() -> int:
     ap.add_argument("--no-lookahead", action="store_true",
                     help="wait for a step's tokens on the host before the next step is launched (the scheduler with --serve, "
                          "the decode loop otherwise)")
-    ap.add_argument("--design", default=None, choices=["pekasun", "nebanex", "kezolix", "bubetar", "tipezen"],
+    ap.add_argument("--design", default=None, choices=["pekasun", "nebanex", "kezolix", "bubetar", "tipezen", "karesun"],
                     help="instead of the record: prefill and decode of that design at a few layer sizes beside the Qwen2 "
-                         "model of equal sizes (kezolix, bubetar: also beside the Nebanex model of equal sizes, tipezen: beside the Bubetar model)")
+                         "model of equal sizes (kezolix, bubetar: also beside the Nebanex model of equal sizes, tipezen: beside the Bubetar model, "
+                         "karesun: beside the Nebanex and Tipezen models)")
     ap.add_argument("--direct-loop", action="store_true",
                     help="decode with the engine's step function in a loop of the benchmark's own instead of Scheduler.step")
     args = ap.parse_args()

@@ -71,7 +71,13 @@ CONFIG_D = config(199, 96, 700, 1e-5, 1.0, [
     (mixer(6, 2, 16, 32, 0.25, 0.5, 40, 8.0, kv_from=0), moe(32, 4, 3, 0.6)),
     (mixer(6, 2, 16, 32, 0.25, 0.5, 40, 8.0, kv_from=0), moe(32, 4, 1, 0.9)),
 ])
-CONFIGS = {"A": (CONFIG_A, 5), "B": (CONFIG_B, 6), "C": (CONFIG_C, 7), "D": (CONFIG_D, 8)}
+# dense layers alone: no router, so that bfloat16 has no close call
+CONFIG_F = config(211, 192, 900, 1e-5, 1.2, [
+    (mixer(6, 2, 32, 48, 0.12, 0.25, 70, 9.0), dense(264)),
+    (mixer(6, 2, 32, 48, 0.15, 0.5, 33, 14.0, kv_from=0), dense(304)),
+    (mixer(3, 1, 9, 21, 0.3, 0.6, 48, 6.0), dense(100)),
+])
+CONFIGS = {"A": (CONFIG_A, 5), "B": (CONFIG_B, 6), "C": (CONFIG_C, 7), "D": (CONFIG_D, 8), "F": (CONFIG_F, 10)}
 
 
 def draw_weights(cfg: dict, seed: int, sharp: float = 2.0) -> dict[str, torch.Tensor]:
