@@ -73,7 +73,7 @@ __global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, Ro
     if (gate_col >= 0) gate = 1.0f / (1.0f + expf(-z.at(row + gate_col) * rf));
     if constexpr (MODE == 0) {
         if constexpr (PIECES) {
-            for (int j = threadIdx.x * E; j < cols; j += 256 * E) {
+            for (int j = (blockIdx.y * 256 + threadIdx.x) * E; j < cols; j += gridDim.y * 256 * E) {
                 float v[E];
                 load_values<E>(src + row + j, v);
 #pragma unroll
@@ -84,7 +84,7 @@ __global__ __launch_bounds__(256) void ff_activation_kernel(ProductView<T> z, Ro
                 store_piece(o + j, v);
             }
         } else {
-            for (int j = threadIdx.x; j < cols; j += blockDim.x) {
+            for (int j = blockIdx.y * 256 + threadIdx.x; j < cols; j += gridDim.y * 256) {
                 const float v = fmaxf(z.at(row + j) * rf, 0.f);
                 o[j] = from_float<T>(v * v * gate);
             }
@@ -177,7 +177,10 @@ static void launch_activation(const void* z, int z_splits, const RowFactor& fact
                          reinterpret_cast<uintptr_t>(out) % 16 == 0;
     const int src = !aligned || z_splits > 1 ? 0 : (z_splits == 0 ? 1 : 2);      // as it comes; of T; of float
     T* o = static_cast<T*>(out);
-#define EGPT_ACTIVATION(MODE, S) ff_activation_kernel<T, MODE, S><<<n_tokens, 256, 0, s>>>(v, factor, z_width, cols, coef, eps, gate_col, o)
+    // (the squared relu needs nothing of the rest of its row: with few tokens its columns go over several workgroups)
+    const int per = src == 0 ? 256 : 256 * E;
+    const dim3 grid(n_tokens, mode == 0 && n_tokens <= 256 ? (cols + per - 1) / per : 1);
+#define EGPT_ACTIVATION(MODE, S) ff_activation_kernel<T, MODE, S><<<grid, 256, 0, s>>>(v, factor, z_width, cols, coef, eps, gate_col, o)
     if (mode == 0) {
         if (src == 0) EGPT_ACTIVATION(0, void);
         else if (src == 1) EGPT_ACTIVATION(0, T);

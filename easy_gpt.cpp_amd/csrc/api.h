@@ -187,7 +187,8 @@ int egpt_window_attention(const void* q, void* out, const void* k_cache, const v
 // or 4 (16).  With
 // n_splits > 1 the chunks of keys of a workgroup's rows are dealt over as many workgroups, whose results part_o
 // [n_splits][n_tokens][nq][dv] and part_ml [n_splits][n_tokens][nq][2] (float32; maps 2: [n_splits][n_tokens][nq][map]..) a
-// second kernel folds.  With maps 2 dk / 2 must be such a multiple, and row_tiles is 4.
+// second kernel folds.  With maps 2 dk / 2 must be such a multiple, and row_tiles is 2
+// (two pairs of wavefronts, one per map, with 16 rows each) or 4 (four pairs).
 int egpt_window_attention_tiled(const void* q, void* out, float* part_o, float* part_ml, const void* k_cache,
                                 const void* v_cache, const int32_t* block_table, int table_width, const int32_t* q_start,
                                 const int32_t* q_len, const int32_t* kv_len, int n_seqs, int n_tokens, int nq, int nkv,

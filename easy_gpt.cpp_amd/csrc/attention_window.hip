@@ -211,9 +211,10 @@ __global__ __launch_bounds__(64 * kSimpleWaves) void window_attention_simple_ker
 // chunks of a workgroup's rows are dealt over as many workgroups (grid z), which leave unnormalised results
 // part_o [split][token][head][dv] and (maximum, sum) part_ml [split][token][head][2] that window_attention_fold_kernel
 // combines; that kernel also adds the sink.  With one split the kernel finishes the rows itself.
-// With two maps to a head (MAPS) a wavefront's tiles come in pairs: tile 2 u is the first map of the 16 rows of pair u, tile
-// 2 u + 1 their second.  A map reads its own half of the query and key rows, which start on whole pieces in LDS; the values'
-// operands serve both.  The parts of a split are then [split][token][head][map].
+// With two maps to a head (MAPS) wavefronts come in pairs: wavefront 2 u takes the first map of its rows, wavefront 2 u + 1 the
+// second map of the same rows.  A map reads its own half of the query and key rows, which start on whole pieces in LDS; the
+// staged values serve both.  At the end the second map's sums go through LDS to the first's wavefront, which finishes the
+// rows.  The parts of a split are then [split][token][head][map].
 typedef __attribute__((ext_vector_type(8))) __bf16 w_bf16x8;
 typedef __attribute__((ext_vector_type(4))) float w_f32x4;
 typedef __attribute__((ext_vector_type(4))) unsigned int w_u32x4;
@@ -301,8 +302,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     constexpr int NKT = KT / 16;                  // tiles of 16 keys in a chunk
     constexpr int PF = 4 * E;                     // features (or keys) that one matrix_piece sums over
     constexpr int NP = KT / PF;                   // pieces of a chunk's keys
-    constexpr int TILES = RW / MAPS;              // tiles of 16 rows to a wavefront; RW tiles of scores, one per map
-    constexpr int ROWS = 16 * RT * TILES, THREADS = 64 * RT;
+    constexpr int ROWS = 16 * (RT / MAPS) * RW, THREADS = 64 * RT;     // a wavefront takes RW tiles of 16 rows (of one map)
     constexpr int VROW = KT + E;                  // padded LDS row of values (elements)
     constexpr int U = 8;                          // loads that a thread has in flight while the queries are staged
     constexpr int KU = 8;                         // 16-byte pieces of a chunk's keys per thread: 64 keys of 256 features
@@ -322,7 +322,8 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     T* k_s = q_s + ROWS * krow;
     T* v_s = k_s + KT * krow;
 
-    const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+    const int tid = threadIdx.x, lane = tid % kWave;
+    const int wave = tid / kWave / MAPS, map = tid / kWave % MAPS;      // which rows of the workgroup, which map
     const int lj = lane % 16, lg = lane / 16;
     const int kh = blockIdx.y;
     const int group_size = nq / nkv;
@@ -351,11 +352,11 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     const int c_begin = blockIdx.z * per_split, c_end = min(n_chunks, c_begin + per_split);
 
     // this wavefront's tiles of 16 rows, this lane's row in each
-    bool valid[TILES];
-    int tok[TILES], head[TILES], p_row[TILES], lo_row[TILES];
+    bool valid[RW];
+    int tok[RW], head[RW], p_row[RW], lo_row[RW];
 #pragma unroll
-    for (int w = 0; w < TILES; ++w) {
-        const int r = blk_first + (wave * TILES + w) * 16 + lj;
+    for (int w = 0; w < RW; ++w) {
+        const int r = blk_first + (wave * RW + w) * 16 + lj;
         valid[w] = r < rows;
         const int i_tok = valid[w] ? r / group_size : 0;
         tok[w] = qs + i_tok;
@@ -365,9 +366,9 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     }
 
     // the smallest position and the largest window start among a tile's rows (rows of no token aside)
-    int tile_p_min[TILES], tile_lo_max[TILES];
+    int tile_p_min[RW], tile_lo_max[RW];
 #pragma unroll
-    for (int w = 0; w < TILES; ++w) {
+    for (int w = 0; w < RW; ++w) {
         int pm = valid[w] ? p_row[w] : 0x7fffffff, lm = valid[w] ? lo_row[w] : 0;
 #pragma unroll
         for (int off = kWave / 2; off > 0; off >>= 1) {
@@ -436,7 +437,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     }
     const float scale = a.scale;
     constexpr float kLog2e = 1.4426950408889634f;
-    const bool wave_active = blk_first + wave * TILES * 16 < rows;      // a wavefront without rows only helps to stage
+    const bool wave_active = blk_first + wave * RW * 16 < rows;      // a wavefront without rows only helps to stage
 
     // A chunk's keys [KT][dk] and values, transposed [dv][KT], travel through registers: the loads of the chunk after
     // this one are issued before this one's products and stored to LDS behind them.  What no row of the workgroup sees
@@ -557,8 +558,8 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
         if (!wave_active) continue;
         // ---- scores of this wavefront's rows against the chunk's keys: a key operand serves all of its row tiles
         w_f32x4 acc[RW][NKT];
-        const T* ks = k_s + lj * krow + lg * E;
-        const T* qrow = q_s + (wave * TILES * 16 + lj) * krow + lg * E;
+        const T* ks = k_s + lj * krow + map * mrow + lg * E;
+        const T* qrow = q_s + (wave * RW * 16 + lj) * krow + map * mrow + lg * E;
 #pragma unroll
         for (int w = 0; w < RW; ++w)
 #pragma unroll
@@ -566,16 +567,12 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
         for (int j = 0; j < n_pieces; ++j) {
             w_u32x4 qv[RW];
 #pragma unroll
-            for (int w = 0; w < RW; ++w)
-                qv[w] = *reinterpret_cast<const w_u32x4*>(qrow + (w / MAPS) * 16 * krow + (w % MAPS) * mrow + j * PF);
+            for (int w = 0; w < RW; ++w) qv[w] = *reinterpret_cast<const w_u32x4*>(qrow + w * 16 * krow + j * PF);
 #pragma unroll
             for (int kt = 0; kt < NKT; ++kt) {
+                const w_u32x4 kvv = *reinterpret_cast<const w_u32x4*>(ks + kt * 16 * krow + j * PF);
 #pragma unroll
-                for (int m = 0; m < MAPS; ++m) {
-                    const w_u32x4 kvv = *reinterpret_cast<const w_u32x4*>(ks + kt * 16 * krow + m * mrow + j * PF);
-#pragma unroll
-                    for (int w = m; w < RW; w += MAPS) acc[w][kt] = matrix_piece<T>(kvv, qv[w], acc[w][kt]);
-                }
+                for (int w = 0; w < RW; ++w) acc[w][kt] = matrix_piece<T>(kvv, qv[w], acc[w][kt]);
             }
         }
         matrix_results_ready();
@@ -586,7 +583,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
             float mx = -INFINITY;
             // a chunk that every row of the tile sees whole (below the diagonal and inside the window, or all kept
             // tokens) needs no mask
-            const bool whole = key0 + KT - 1 <= tile_p_min[w / MAPS] && (key0 >= tile_lo_max[w / MAPS] || key0 + KT <= a.keep_first);
+            const bool whole = key0 + KT - 1 <= tile_p_min[w] && (key0 >= tile_lo_max[w] || key0 + KT <= a.keep_first);
             if constexpr (CAPPED) {
                 const float inner = scale / a.softcap;
 #pragma unroll
@@ -594,7 +591,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
 #pragma unroll
                     for (int v = 0; v < 4; ++v) {
                         const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = whole || (key <= p_row[w / MAPS] && (key >= lo_row[w / MAPS] || key < a.keep_first));
+                        const bool seen = whole || (key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first));
                         const float sc = seen ? a.softcap * bounded_tanh<T>(acc[w][kt][v] * inner) : -INFINITY;
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
@@ -602,31 +599,31 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
             } else if (a.dist_bias != nullptr) {
                 // the bias of the row's head by distance; a chunk that lies `far` or more behind every row of the tile
                 // gets the table's last entry throughout
-                const float* brow = a.dist_bias + static_cast<size_t>(head[w / MAPS]) * (a.dist_far + 1);
-                const bool all_far = whole && tile_p_min[w / MAPS] - (key0 + KT - 1) >= a.dist_far;
+                const float* brow = a.dist_bias + static_cast<size_t>(head[w]) * (a.dist_far + 1);
+                const bool all_far = whole && tile_p_min[w] - (key0 + KT - 1) >= a.dist_far;
                 const float b_far = brow[a.dist_far];
 #pragma unroll
                 for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
                     for (int v = 0; v < 4; ++v) {
                         const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = key <= p_row[w / MAPS] && (key >= lo_row[w / MAPS] || key < a.keep_first);
+                        const bool seen = key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first);
                         float sc = -INFINITY;
                         if (all_far) sc = fmaf(acc[w][kt][v], scale, b_far);
-                        else if (seen) sc = fmaf(acc[w][kt][v], scale, brow[min(p_row[w / MAPS] - key, a.dist_far)]);
+                        else if (seen) sc = fmaf(acc[w][kt][v], scale, brow[min(p_row[w] - key, a.dist_far)]);
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
                     }
             } else if (a.slopes != nullptr) {
                 // the penalty of the row's head times the distance
-                const float slope = a.slopes[head[w / MAPS]];
+                const float slope = a.slopes[head[w]];
 #pragma unroll
                 for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
                     for (int v = 0; v < 4; ++v) {
                         const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = whole || (key <= p_row[w / MAPS] && (key >= lo_row[w / MAPS] || key < a.keep_first));
-                        const float sc = seen ? fmaf(acc[w][kt][v], scale, -slope * static_cast<float>(p_row[w / MAPS] - key)) : -INFINITY;
+                        const bool seen = whole || (key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first));
+                        const float sc = seen ? fmaf(acc[w][kt][v], scale, -slope * static_cast<float>(p_row[w] - key)) : -INFINITY;
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
                     }
@@ -644,7 +641,7 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
 #pragma unroll
                     for (int v = 0; v < 4; ++v) {
                         const int key = key0 + kt * 16 + lg * 4 + v;
-                        const bool seen = key <= p_row[w / MAPS] && (key >= lo_row[w / MAPS] || key < a.keep_first);
+                        const bool seen = key <= p_row[w] && (key >= lo_row[w] || key < a.keep_first);
                         const float sc = seen ? acc[w][kt][v] * scale : -INFINITY;
                         acc[w][kt][v] = sc;
                         mx = fmaxf(mx, sc);
@@ -711,9 +708,8 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     if (a.n_splits > 1) {
 #pragma unroll
         for (int w = 0; w < RW; ++w) {
-            const int u = w / MAPS;
-            if (!valid[u]) continue;
-            const size_t row_at = ((static_cast<size_t>(blockIdx.z) * a.n_tokens + tok[u]) * nq + head[u]) * MAPS + w % MAPS;
+            if (!valid[w]) continue;
+            const size_t row_at = ((static_cast<size_t>(blockIdx.z) * a.n_tokens + tok[w]) * nq + head[w]) * MAPS + map;
             float* po = a.part_o + row_at * dv + lg * 4;
 #pragma unroll
             for (int d = 0; d < DT; ++d)
@@ -728,44 +724,58 @@ __global__ __launch_bounds__(64 * RT, (DT * RW <= 8 ? 2 : 1)) void window_attent
     if constexpr (MAPS == 2) {
         // the difference of the two maps, divided by its root mean square (a row's four lanes hold its features; those
         // beyond dv are zero)
+        w_f32x4* second = reinterpret_cast<w_f32x4*>(window_smem) + (wave * RW * DT) * kWave + lane;
+        __syncthreads();                  // the last chunk is read
+        if (map == 1) {
 #pragma unroll
-        for (int u = 0; u < TILES; ++u) {
-            const float f1 = valid[u] ? 1.0f / l_sum[2 * u] : 0.f, f2 = valid[u] ? a.map_weight / l_sum[2 * u + 1] : 0.f;
+            for (int w = 0; w < RW; ++w) {
+                const float f = valid[w] ? a.map_weight / l_sum[w] : 0.f;
+#pragma unroll
+                for (int d = 0; d < DT; ++d)
+                    second[(w * DT + d) * kWave] = w_f32x4{o[w][d][0] * f, o[w][d][1] * f, o[w][d][2] * f, o[w][d][3] * f};
+            }
+        }
+        __syncthreads();
+        if (map == 1) return;
+#pragma unroll
+        for (int w = 0; w < RW; ++w) {
+            const float f1 = valid[w] ? 1.0f / l_sum[w] : 0.f;
             float ss = 0.f;
 #pragma unroll
-            for (int d = 0; d < DT; ++d)
+            for (int d = 0; d < DT; ++d) {
+                const w_f32x4 o2 = second[(w * DT + d) * kWave];
 #pragma unroll
                 for (int v = 0; v < 4; ++v) {
-                    const float x = o[2 * u][d][v] * f1 - o[2 * u + 1][d][v] * f2;
-                    o[2 * u][d][v] = x;
+                    const float x = o[w][d][v] * f1 - o2[v];
+                    o[w][d][v] = x;
                     ss = fmaf(x, x, ss);
                 }
+            }
             ss += __shfl_xor(ss, 16, kWave);
             ss += __shfl_xor(ss, 32, kWave);
             const float f = a.out_scale * inv_rms(ss, 1.0f / static_cast<float>(dv), a.out_eps);
-            if (!valid[u]) continue;
-            T* op = static_cast<T*>(a.out) + (static_cast<size_t>(tok[u]) * nq + head[u]) * dv + lg * 4;
+            if (!valid[w]) continue;
+            T* op = static_cast<T*>(a.out) + (static_cast<size_t>(tok[w]) * nq + head[w]) * dv + lg * 4;
 #pragma unroll
             for (int d = 0; d < DT; ++d)
-                if (d * 16 < dv)
-                    store_four<T>(op + d * 16, o[2 * u][d][0] * f, o[2 * u][d][1] * f, o[2 * u][d][2] * f, o[2 * u][d][3] * f);
+                if (d * 16 < dv) store_four<T>(op + d * 16, o[w][d][0] * f, o[w][d][1] * f, o[w][d][2] * f, o[w][d][3] * f);
         }
         return;
     }
 #pragma unroll
     for (int w = 0; w < RW; ++w) {
-        if (!valid[w / MAPS]) continue;
+        if (!valid[w]) continue;
         float l = l_sum[w];
         float weight = 1.0f;
         if (a.sink != nullptr) {
-            const float sk = a.sink[head[w / MAPS]];
+            const float sk = a.sink[head[w]];
             const float m_all = fmaxf(m_run[w], sk);
             weight = __builtin_amdgcn_exp2f((m_run[w] - m_all) * kLog2e);
             l = l * weight + __builtin_amdgcn_exp2f((sk - m_all) * kLog2e);
         }
         float inv = weight / l;
-        if (a.head_gate != nullptr) inv *= a.head_gate[static_cast<size_t>(tok[w / MAPS]) * nq + head[w / MAPS]];
-        T* op = static_cast<T*>(a.out) + (static_cast<size_t>(tok[w / MAPS]) * nq + head[w / MAPS]) * dv + lg * 4;
+        if (a.head_gate != nullptr) inv *= a.head_gate[static_cast<size_t>(tok[w]) * nq + head[w]];
+        T* op = static_cast<T*>(a.out) + (static_cast<size_t>(tok[w]) * nq + head[w]) * dv + lg * 4;
 #pragma unroll
         for (int d = 0; d < DT; ++d)
             if (d * 16 < dv)
@@ -805,41 +815,61 @@ __global__ __launch_bounds__(kWave) void window_attention_fold_kernel(const floa
     }
 }
 
-// The same for heads of two maps: both maps' parts are folded, and their difference is divided by its root mean square.
+// The same for heads of two maps: both maps' parts are folded, and their difference is divided by its root mean square.  Four
+// wavefronts share a row's splits (split s to wavefront s modulo 4), their sums are added in that order.
+constexpr int kFoldWaves = 4;
 template <typename T>
-__global__ __launch_bounds__(kWave) void window_attention_fold_maps_kernel(const float* __restrict__ part_o,
+__global__ __launch_bounds__(kWave * kFoldWaves) void window_attention_fold_maps_kernel(const float* __restrict__ part_o,
                                                                          const float* __restrict__ part_ml, float map_weight,
                                                                          float out_scale, float out_eps, T* __restrict__ out,
                                                                          int n_rows, int dv, int n_splits) {
     constexpr int kOwn = 256 / kWave;          // features of a row that a lane holds (dv <= 256)
     __shared__ float weights[2][kWave];        // at most 64 splits
-    const int row = blockIdx.x, lane = threadIdx.x;
-#pragma unroll
-    for (int map = 0; map < 2; ++map) {
+    __shared__ float sums[kFoldWaves][256];
+    const int row = blockIdx.x, lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+    if (wave < 2) {                            // the splits' weights, a map to a wavefront
         float m = -INFINITY, l = 0.f;
         if (lane < n_splits) {
-            const float* ml = part_ml + ((static_cast<size_t>(lane) * n_rows + row) * 2 + map) * 2;
+            const float* ml = part_ml + ((static_cast<size_t>(lane) * n_rows + row) * 2 + wave) * 2;
             m = ml[0];
             l = ml[1];
         }
         const float m_all = wave_max(m);
         const float w = lane < n_splits ? expf(m - m_all) : 0.f;     // exp(-inf) = 0 for a split that saw nothing
-        weights[map][lane] = w / wave_sum(l * w) * (map == 0 ? 1.0f : -map_weight);
+        weights[wave][lane] = w / wave_sum(l * w) * (wave == 0 ? 1.0f : -map_weight);
     }
     __syncthreads();
     float acc[kOwn] = {};
-    for (int s = 0; s < n_splits; ++s) {
-        const float* po = part_o + (static_cast<size_t>(s) * n_rows + row) * 2 * dv;
-        const float w1 = weights[0][s], w2 = weights[1][s];
+    for (int s0 = wave; s0 < n_splits; s0 += kFoldWaves * 2) {       // two splits' loads in flight together
+        const int s1 = s0 + kFoldWaves;
+        const bool two = s1 < n_splits;
+        const float* p0 = part_o + (static_cast<size_t>(s0) * n_rows + row) * 2 * dv;
+        const float* p1 = part_o + (static_cast<size_t>(two ? s1 : s0) * n_rows + row) * 2 * dv;
+        float v[kOwn][4];
 #pragma unroll
         for (int r = 0; r < kOwn; ++r) {
             const int d = lane + r * kWave;
-            if (d < dv) acc[r] = fmaf(po[dv + d], w2, fmaf(po[d], w1, acc[r]));
+            const bool in = d < dv;
+            v[r][0] = in ? p0[d] : 0.f;
+            v[r][1] = in ? p0[dv + d] : 0.f;
+            v[r][2] = in && two ? p1[d] : 0.f;
+            v[r][3] = in && two ? p1[dv + d] : 0.f;
         }
+        const float w0 = weights[0][s0], w1 = weights[1][s0], w2 = two ? weights[0][s1] : 0.f, w3 = two ? weights[1][s1] : 0.f;
+#pragma unroll
+        for (int r = 0; r < kOwn; ++r) acc[r] = fmaf(v[r][3], w3, fmaf(v[r][2], w2, fmaf(v[r][1], w1, fmaf(v[r][0], w0, acc[r]))));
     }
+#pragma unroll
+    for (int r = 0; r < kOwn; ++r) sums[wave][lane + r * kWave] = acc[r];
+    __syncthreads();
+    if (wave != 0) return;
     float ss = 0.f;
 #pragma unroll
-    for (int r = 0; r < kOwn; ++r) ss = fmaf(acc[r], acc[r], ss);
+    for (int r = 0; r < kOwn; ++r) {
+#pragma unroll
+        for (int w = 1; w < kFoldWaves; ++w) acc[r] += sums[w][lane + r * kWave];
+        ss = fmaf(acc[r], acc[r], ss);
+    }
     const float f = out_scale * inv_rms(wave_sum(ss), 1.0f / static_cast<float>(dv), out_eps);
 #pragma unroll
     for (int r = 0; r < kOwn; ++r) {
@@ -850,9 +880,10 @@ __global__ __launch_bounds__(kWave) void window_attention_fold_maps_kernel(const
 
 template <typename T, int DT, int RT, int RW, int MAPS, bool CAPPED>
 static int launch_tiled(const WindowArgs& a, int max_rows, hipStream_t s) {
-    constexpr int E = 16 / sizeof(T), KT = sizeof(T) == 2 ? 64 : 32, PF = 4 * E, ROWS = 16 * RT * (RW / MAPS);
+    constexpr int E = 16 / sizeof(T), KT = sizeof(T) == 2 ? 64 : 32, PF = 4 * E, ROWS = 16 * (RT / MAPS) * RW;
     const int krow = MAPS * ((a.dk / MAPS + PF - 1) / PF * PF) + E;
-    const size_t lds = (static_cast<size_t>(ROWS + KT) * krow + static_cast<size_t>(DT) * 16 * (KT + E)) * sizeof(T);
+    size_t lds = (static_cast<size_t>(ROWS + KT) * krow + static_cast<size_t>(DT) * 16 * (KT + E)) * sizeof(T);
+    if (MAPS == 2 && lds < static_cast<size_t>(ROWS) * DT * 16 * sizeof(float)) lds = static_cast<size_t>(ROWS) * DT * 16 * sizeof(float);
     if (lds > 160 * 1024) return EGPT_UNSUPPORTED_SIZE;
     auto kernel = window_attention_tiled_kernel<T, DT, RT, RW, MAPS, CAPPED>;
     if (lds > 48 * 1024) {
@@ -871,13 +902,19 @@ static int launch_tiled(const WindowArgs& a, int max_rows, hipStream_t s) {
     return EGPT_OK;
 }
 
-// row_tiles: 4 (four wavefronts with 16 rows each) or 8 (with 32 rows each)
+// row_tiles: 4 (four wavefronts with 16 rows each) or 8 (with 32 rows each); with two maps to a head 2 (two pairs of wavefronts
+// with 16 rows each) or 4 (four pairs)
 template <typename T, int DT>
 static int launch_tiled_for_rows(const WindowArgs& a, int max_rows, int row_tiles, hipStream_t s) {
     if (a.maps == 2) {
-        if (row_tiles == 8) return EGPT_UNSUPPORTED_SIZE;
-        if (a.softcap > 0.f) return launch_tiled<T, DT, 4, 2, 2, true>(a, max_rows, s);
-        return launch_tiled<T, DT, 4, 2, 2, false>(a, max_rows, s);
+        if (row_tiles == 2 || DT > 8) {           // (eight wavefronts of wider values do not fit the registers)
+            if (a.softcap > 0.f) return launch_tiled<T, DT, 4, 1, 2, true>(a, max_rows, s);
+            return launch_tiled<T, DT, 4, 1, 2, false>(a, max_rows, s);
+        }
+        if constexpr (DT <= 8) {
+            if (a.softcap > 0.f) return launch_tiled<T, DT, 8, 1, 2, true>(a, max_rows, s);
+            return launch_tiled<T, DT, 8, 1, 2, false>(a, max_rows, s);
+        }
     }
     if (a.softcap > 0.f) {
         if (row_tiles == 8) return launch_tiled<T, DT, 4, 2, 1, true>(a, max_rows, s);
@@ -951,7 +988,7 @@ extern "C" int egpt_window_attention_tiled(const void* q, void* out, float* part
     if (!q || !out || !k_cache || !v_cache || !block_table || !q_start || !q_len || !kv_len) return EGPT_BAD_ARGUMENT;
     if (n_seqs <= 0 || n_tokens < 0 || nq <= 0 || nkv <= 0 || nq % nkv != 0 || dk <= 0 || dv <= 0 || page_size <= 0 ||
         table_width <= 0 || window < 0 || keep_first < 0 || n_splits < 1 || (dtype != 0 && dtype != 1) ||
-        (row_tiles != 4 && row_tiles != 8) || (dist_bias && dist_far < 0) || block < 0 || (dist_bias && slopes) ||
+        (row_tiles != 4 && row_tiles != (maps == 2 ? 2 : 8)) || (dist_bias && dist_far < 0) || block < 0 || (dist_bias && slopes) ||
         !(softcap >= 0.f) || (softcap > 0.f && (dist_bias || slopes)) || !maps_fit(maps, dk, sink, dist_bias, slopes, head_gate))
         return EGPT_BAD_ARGUMENT;
     if (n_splits > 1 && (!part_o || !part_ml)) return EGPT_BAD_ARGUMENT;
@@ -979,10 +1016,10 @@ extern "C" int egpt_window_attention_tiled(const void* q, void* out, float* part
     EGPT_CHECK_LAUNCH();
     if (n_splits > 1 && maps == 2) {
         if (dtype == 0)
-            window_attention_fold_maps_kernel<float><<<n_tokens * nq, kWave, 0, s>>>(
+            window_attention_fold_maps_kernel<float><<<n_tokens * nq, kWave * kFoldWaves, 0, s>>>(
                 part_o, part_ml, map_weight, out_scale, out_eps, static_cast<float*>(out), n_tokens * nq, dv, n_splits);
         else
-            window_attention_fold_maps_kernel<bf16_t><<<n_tokens * nq, kWave, 0, s>>>(
+            window_attention_fold_maps_kernel<bf16_t><<<n_tokens * nq, kWave * kFoldWaves, 0, s>>>(
                 part_o, part_ml, map_weight, out_scale, out_eps, static_cast<bf16_t*>(out), n_tokens * nq, dv, n_splits);
         EGPT_CHECK_LAUNCH();
     } else if (n_splits > 1) {

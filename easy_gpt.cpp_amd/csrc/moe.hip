@@ -56,10 +56,11 @@ __device__ __forceinline__ m_u32x4 row_piece(const T* row, int k, int n, bool al
 
 constexpr int kMaxExperts = 1024;
 
-// One workgroup of four wavefronts per token.  A wavefront takes the experts four at a time (all loads of the four rows
-// in flight together, then the four sums), wavefront w the groups w, w + 4, ...; the first wavefront then picks.
+// One workgroup of up to sixteen wavefronts per token.  A wavefront takes the experts four at a time (all loads of the four
+// rows in flight together, 16 bytes a lane where rows start on 16 bytes, then the four sums), wavefront w the groups w,
+// w + (wavefronts), ...; the first wavefront then picks.
 template <typename T>
-__global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x, const T* __restrict__ router,
+__global__ __launch_bounds__(1024) void moe_route_kernel(const T* __restrict__ x, const T* __restrict__ router,
                                                         const T* __restrict__ bias, int32_t* __restrict__ chosen,
                                                         float* __restrict__ weight, int n_tokens, int hidden, int experts,
                                                         int top, int score_all, const float* __restrict__ correction,
@@ -69,15 +70,29 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
     const int t = blockIdx.x;
     float* z = logits_s;
     const T* xr = x + static_cast<size_t>(t) * hidden;
-    for (int e0 = wave * 4; e0 < experts; e0 += 16) {
+    constexpr int E = 16 / sizeof(T);
+    const bool aligned = hidden % E == 0 && ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(router)) & 15) == 0;
+    for (int e0 = wave * 4; e0 < experts; e0 += static_cast<int>(blockDim.x) / kWave * 4) {
         float dot[4] = {0.f, 0.f, 0.f, 0.f};
         const T* wr[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) wr[i] = router + static_cast<size_t>(min(e0 + i, experts - 1)) * hidden;
-        for (int j = lane; j < hidden; j += kWave) {
-            const float xv = to_float(xr[j]);
+        if (aligned) {
+            for (int j = lane * E; j < hidden; j += kWave * E) {
+                struct { T v[E]; } xv = __builtin_bit_cast(decltype(xv), *reinterpret_cast<const m_u32x4*>(xr + j)), wv[4];
 #pragma unroll
-            for (int i = 0; i < 4; ++i) dot[i] = fmaf(xv, to_float(wr[i][j]), dot[i]);
+                for (int i = 0; i < 4; ++i) wv[i] = __builtin_bit_cast(decltype(xv), *reinterpret_cast<const m_u32x4*>(wr[i] + j));
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+#pragma unroll
+                    for (int e = 0; e < E; ++e) dot[i] = fmaf(to_float(xv.v[e]), to_float(wv[i].v[e]), dot[i]);
+            }
+        } else {
+            for (int j = lane; j < hidden; j += kWave) {
+                const float xv = to_float(xr[j]);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) dot[i] = fmaf(xv, to_float(wr[i][j]), dot[i]);
+            }
         }
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
@@ -426,9 +441,10 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
                                                           const int32_t* __restrict__ place, const float* __restrict__ weight,
                                                           float* __restrict__ out, fixed_t* __restrict__ stream, int top, int hidden) {
     const int t = blockIdx.x;
-    for (int j = threadIdx.x; j < hidden; j += blockDim.x) {
+    for (int j = blockIdx.y * blockDim.x + threadIdx.x; j < hidden; j += gridDim.y * blockDim.x) {
         const size_t at = static_cast<size_t>(t) * hidden + j;
         float acc = 0.f;
+#pragma unroll 4
         for (int c = 0; c < top; ++c) {
             const int row = place[static_cast<size_t>(t) * top + c];
             const float v = row >= 0 ? y[static_cast<size_t>(row) * hidden + j] : to_float(x[at]);
@@ -457,13 +473,16 @@ extern "C" int egpt_moe_route(const void* x, const void* router, const void* bia
     hipStream_t s = static_cast<hipStream_t>(stream);
     const size_t lds = 3 * static_cast<size_t>(experts) * sizeof(float);      // choice scores, scores, groups' scores
     const unsigned blocks = n_tokens;
+    // a group of four experts to a wavefront where the tokens are few, four wavefronts where they fill the GPU
+    const int most = n_tokens <= 512 ? 16 : 4, want = (experts + 3) / 4;
+    const unsigned threads = kWave * (want < most ? want : most);
     if (dtype == 0)
-        moe_route_kernel<float><<<blocks, 256, lds, s>>>(static_cast<const float*>(x), static_cast<const float*>(router),
+        moe_route_kernel<float><<<blocks, threads, lds, s>>>(static_cast<const float*>(x), static_cast<const float*>(router),
                                                          static_cast<const float*>(bias), chosen, weight, n_tokens, hidden,
                                                          experts, top, score_all, correction, weight_scale, groups,
                                                          keep_groups, normalized);
     else
-        moe_route_kernel<bf16_t><<<blocks, 256, lds, s>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(router),
+        moe_route_kernel<bf16_t><<<blocks, threads, lds, s>>>(static_cast<const bf16_t*>(x), static_cast<const bf16_t*>(router),
                                                           static_cast<const bf16_t*>(bias), chosen, weight, n_tokens, hidden,
                                                           experts, top, score_all, correction, weight_scale, groups,
                                                          keep_groups, normalized);
@@ -568,10 +587,12 @@ extern "C" int egpt_moe_combine(const float* y, const void* x, const int32_t* pl
     if (n_tokens == 0) return EGPT_OK;
     hipStream_t s = static_cast<hipStream_t>(stream);
     fixed_t* acc = static_cast<fixed_t*>(residual);
+    // few tokens: a column to a thread
+    const dim3 grid(n_tokens, n_tokens <= 64 ? (hidden + 255) / 256 : 1);
     if (dtype == 0)
-        moe_combine_kernel<float><<<n_tokens, 256, 0, s>>>(y, static_cast<const float*>(x), place, weight, out, acc, top, hidden);
+        moe_combine_kernel<float><<<grid, 256, 0, s>>>(y, static_cast<const float*>(x), place, weight, out, acc, top, hidden);
     else
-        moe_combine_kernel<bf16_t><<<n_tokens, 256, 0, s>>>(y, static_cast<const bf16_t*>(x), place, weight, out, acc, top, hidden);
+        moe_combine_kernel<bf16_t><<<grid, 256, 0, s>>>(y, static_cast<const bf16_t*>(x), place, weight, out, acc, top, hidden);
     EGPT_CHECK_LAUNCH();
     return EGPT_OK;
 }

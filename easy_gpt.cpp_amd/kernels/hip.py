@@ -1575,9 +1575,13 @@ class HipKernels(KernelBackend):
         row_tiles = 8 if maps == 1 and dk > HipKernels.wide_rows_key_size and t * group * nkv >= HipKernels.wide_rows_from else 4
         krow = maps * (-(-(dk // maps) // (4 * e)) * 4 * e) + e
         dv_tiles = next(n for n in (2, 4, 6, 8, 12, 16) if n * 16 >= dv)
-        lds = lambda tiles: ((16 * tiles + chunk) * krow + dv_tiles * 16 * (chunk + e)) * elem
+        lds = lambda tiles: max(((16 * tiles + chunk) * krow + dv_tiles * 16 * (chunk + e)) * elem, 16 * tiles * dv_tiles * 64 if maps == 2 else 0)
         if row_tiles == 8 and lds(8) > 160 * 1024:
             row_tiles = 4
+        if maps == 2 and (max_q_len * group <= 32 or dv <= 64 or dv > 128 or lds(4) > 160 * 1024):
+            # pairs of wavefronts, a map each, with 16 rows: two pairs to a workgroup, or four (measured, us for a 2,048-token
+            # prompt, two / four pairs: 14 heads on 2 of 2 x 32 + 64, window 1,024: 77 / 94; 16 on 4 of 2 x 64 + 128: 226 / 195)
+            row_tiles = 2
         if lds(row_tiles) > 160 * 1024:
             return None
         # workgroups that have rows (a request's rows start a workgroup of their own)
@@ -1588,7 +1592,9 @@ class HipKernels(KernelBackend):
         # (2,048-token prompts of 448 workgroups lose with splits: their parts are 44 MB; 64 single tokens on four
         # key/value heads, 256 workgroups that walk 33 chunks each, gain: 0.93 -> 0.86 ms a step at width 2,048)
         if workgroups <= 320 and chunks > 1:
-            n_splits = max(1, min(chunks, -(-1024 // workgroups), 64))
+            # (two maps leave twice the parts to fold: half as many splits; 8 single tokens on four key/value heads of 2 x 64 +
+            # 128 behind 2,048: 36 us with 32 splits, 28 with 16)
+            n_splits = max(1, min(chunks, -(-(1024 // maps) // workgroups), 64))
         return row_tiles, n_splits
 
     def swiglu(self, gate_up, out, row_ss=None, hidden=0, eps=0.0, activation="silu"):
